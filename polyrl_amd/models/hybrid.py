@@ -1,11 +1,11 @@
 """Configuration of hybrid decoders: a stack whose layers each pick one
 sequence mixer (recurrent, state-space, gated linear attention, a real-gated
-linear recurrence, latent attention or grouped-query attention) and one
-feed-forward (dense, table-routed experts, router-chosen experts, or none).
+linear recurrence, latent attention, grouped-query attention, or two of
+them side by side) and one feed-forward (dense, table-routed experts, router-chosen experts, or none).
 
 The Bizusun design is the first family described this way, Kuforax the
-second, Vurivik the third, Nasipel the fourth.  Everything that
-can differ between two models of a family is a field here and is read from
+second, Vurivik the third, Nasipel the fourth, Puvapel the fifth.
+Everything that can differ between two models of a family is a field here and is read from
 the checkpoint's ``config.json``; constants that the design fixes (the decay
 constant of the delta rule, its key epsilon) are defaults of the mixer
 parameters, so another design can set them differently.
@@ -28,6 +28,47 @@ class DeltaRuleSpec:
     decay_scale: float = math.exp(-0.5)   # w = exp(-decay_scale * sigmoid(.))
     key_eps: float = 1e-6                 # unit key: k / sqrt(sum k^2 + eps)
     kind: str = "general_delta"
+
+
+@dataclass
+class ChannelDeltaSpec:
+    """Gated delta rule with one decay per head and key channel,
+    ``exp(-exp(A_log) * softplus(low-rank projection + bias))``; q, k and v
+    pass a short convolution and SiLU, q and k heads are unit vectors (shared
+    by ``heads / kv_heads`` heads), the write strength is a sigmoid per head;
+    heads are normed over ``vdim`` and gated by a low-rank sigmoid gate."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    conv: int
+    decay_rank: Optional[int] = None      # rows of a1; None = from the tensor
+    gate_rank: Optional[int] = None       # rows of g1; None = from the tensor
+    key_eps: float = 1e-6                 # unit: x / sqrt(sum x^2 + eps)
+    kind: str = "channel_delta"
+
+
+@dataclass
+class SelectiveScanSpec:
+    """Mamba-1 style selective scan: one step size per channel (a low-rank
+    projection of the convolved branch), one decay per channel and state
+    entry, input and read-out vectors shared by the channels."""
+    inner: int
+    state: int
+    dt_rank: int
+    conv: int = 4
+    kind: str = "mamba"
+
+
+@dataclass
+class ParallelMixerSpec:
+    """Two mixers side by side on the same input:
+    ``left_scale * left(h) + right_scale * right(h)``."""
+    left: object
+    right: object
+    left_scale: float = 1.0
+    right_scale: float = 1.0
+    kind: str = "parallel"
 
 
 @dataclass
@@ -173,7 +214,14 @@ class WindowAttnSpec:
     (``weights="sigmoid"``), and values that are rotated by their position
     over all ``vdim`` entries before they are cached, the head's sum being
     turned back by the query's position (``value_rope_base`` > 0; pairs
-    (m, m + vdim/2), frequencies base^(-2m/vdim), never scaled)."""
+    (m, m + vdim/2), frequencies base^(-2m/vdim), never scaled).  A short
+    causal convolution of ``conv`` taps on every query, key and value
+    channel directly after the projection (``conv`` > 0), RMS norms per
+    head with one weight row shared by the heads, before the rotation
+    (``head_norm``), attention confined to chunks of ``chunk`` positions
+    counted from the sequence's start (``chunk`` > 0: key j is seen from p
+    when floor(j / chunk) = floor(p / chunk)), and a fixed sink of score 0,
+    i.e. one added to the softmax denominator (``unit_sink``)."""
     heads: int
     kv_heads: int
     dim: int
@@ -196,6 +244,10 @@ class WindowAttnSpec:
     head_bias: bool = False
     weights: str = "softmax"
     value_rope_base: float = 0.0
+    conv: int = 0
+    head_norm: bool = False
+    chunk: int = 0
+    unit_sink: bool = False
     kind: str = "attention"
 
     def bucket_of_distance(self) -> List[int]:
@@ -271,6 +323,7 @@ class HybridConfig:
     canon_taps: int = 4
     token_side_dim: int = 0
     logit_scale: float = 1.0
+    logit_softcap: float = 0.0            # c * tanh(logit / c); 0 = none
     max_position_embeddings: int = 1 << 20   # no learned positions: a fence
     # "canon": norm -> convolution -> mixer, norm -> ff, token-side input
     # (scalar norm weights).  "sandwich": x += norm(mixer(norm(x))),
@@ -278,7 +331,9 @@ class HybridConfig:
     # from ``norm_offset``.  "prenorm": x += m * mixer(norm(x)),
     # x += m * ff(norm(x)), x += m * token-side input, with per-channel
     # weights and m = ``residual_mult``.  "parallel": both sublayers read
-    # the same stream, x += mixer(norm1(x)) + ff(norm2(x)).
+    # the same stream, x += mixer(norm1(x)) + ff(norm2(x)).  "postnorm":
+    # sublayers read the stream itself, x += norm1(mixer(x)),
+    # x += norm2(ff(x)).
     layer_style: str = "canon"
     # "rms": x / sqrt(mean(x^2) + eps) * w.  "layer": (x - mean) /
     # sqrt(var + eps) * w (no bias); parallel layers only.
@@ -339,6 +394,34 @@ class HybridConfig:
             return None
         return li if m.kv_from is None else m.kv_from
 
+    @staticmethod
+    def _check_attention(li, m):
+        assert m.heads % m.kv_heads == 0 and m.window >= 1
+        if m.rope is not None:
+            assert m.rope.dims % 2 == 0 and m.rope.dims <= m.dim
+            if m.rope.interleaved:
+                raise ValueError(f"layer {li}: grouped-query "
+                                 "attention rotates halves")
+        assert m.weights in ("softmax", "sigmoid")
+        if m.weights == "sigmoid" and (m.sink or m.bias_far > 0):
+            raise ValueError(f"layer {li}: a sink or a distance "
+                             "bias needs softmax weights")
+        if m.value_rope_base > 0:
+            assert m.vdim % 2 == 0 and not m.values_from_keys
+        if m.bias_far > 0 and m.keep_first > 0:
+            raise ValueError(f"layer {li}: the distance bias covers "
+                             "the window only (no kept first tokens)")
+        if m.head_norm and (m.qk_norm or m.head_unit_norm or
+                            m.values_from_keys):
+            raise ValueError(f"layer {li}: per-head norm weights do not "
+                             "combine with another query/key norm")
+        assert m.chunk >= 0 and m.conv >= 0
+        if m.conv and (m.values_from_keys or m.head_gate or m.qkv_bias):
+            raise ValueError(f"layer {li}: the convolved projection has "
+                             "no gate, no bias and its own values")
+        if m.unit_sink and (m.sink or m.weights == "sigmoid"):
+            raise ValueError(f"layer {li}: one sink, softmax weights")
+
     def validate(self):
         for li, L in enumerate(self.layers):
             m = L.mixer
@@ -354,6 +437,20 @@ class HybridConfig:
                                      "equal latent and rotated sizes")
             if m.kind == "gla":
                 assert m.heads > 0 and m.dim > 0 and m.vdim > 0 and m.tau > 0
+            if m.kind == "channel_delta":
+                assert m.heads % m.kv_heads == 0 and m.conv >= 1
+            if m.kind == "parallel":
+                for part in (m.left, m.right):
+                    if part.kind not in ("attention", "mamba"):
+                        raise ValueError(f"layer {li}: {part.kind} cannot "
+                                         "be one of two mixers")
+                    if getattr(part, "bias_far", 0) > 0:
+                        raise ValueError(f"layer {li}: no distance bias in "
+                                         "side-by-side mixers")
+                    if part.kind == "attention":
+                        self._check_attention(li, part)
+                    else:
+                        assert part.inner > 0 and part.conv >= 1
             if m.kind == "rglru":
                 assert m.width % m.blocks == 0 and m.conv >= 1
             if m.kind == "latent_attention":
@@ -364,21 +461,7 @@ class HybridConfig:
                 assert m.heads % m.groups == 0
                 assert m.inner % m.norm_groups == 0
             if m.kind == "attention":
-                assert m.heads % m.kv_heads == 0 and m.window >= 1
-                if m.rope is not None:
-                    assert m.rope.dims % 2 == 0 and m.rope.dims <= m.dim
-                    if m.rope.interleaved:
-                        raise ValueError(f"layer {li}: grouped-query "
-                                         "attention rotates halves")
-                assert m.weights in ("softmax", "sigmoid")
-                if m.weights == "sigmoid" and (m.sink or m.bias_far > 0):
-                    raise ValueError(f"layer {li}: a sink or a distance "
-                                     "bias needs softmax weights")
-                if m.value_rope_base > 0:
-                    assert m.vdim % 2 == 0 and not m.values_from_keys
-                if m.bias_far > 0 and m.keep_first > 0:
-                    raise ValueError(f"layer {li}: the distance bias covers "
-                                     "the window only (no kept first tokens)")
+                self._check_attention(li, m)
             if L.ff is not None and L.ff.kind == "dense":
                 assert L.ff.act in ("silu", "clamped")
                 assert L.ff.act == "silu" or L.ff.limit > 0
@@ -933,6 +1016,109 @@ def nasipel_preset(width: int, layers: int, vocab: int = 32000,
                         norm_kind="layer", gated_residual=True).validate()
 
 
+def _puvapel_mixer_from_json(kind: str, m: dict):
+    """Puvapel mixers: 'channel_delta' and 'parallel' (left: convolved,
+    chunked grouped-query attention with per-head norms, capped scores and a
+    fixed sink; right: a selective scan)."""
+    if kind == "channel_delta":
+        return ChannelDeltaSpec(heads=int(m["heads"]),
+                                kv_heads=int(m["kv_heads"]),
+                                dim=int(m["dim"]), vdim=int(m["vdim"]),
+                                conv=int(m["conv"]))
+    if kind == "parallel":
+        a, r = m["left"], m["right"]
+        return ParallelMixerSpec(
+            left=WindowAttnSpec(
+                heads=int(a["heads"]), kv_heads=int(a["kv_heads"]),
+                dim=int(a["dim"]), vdim=int(a["vdim"]), window=UNBOUNDED,
+                scale=float(a["scale"]), rope=_rope_from_json(a.get("rot")),
+                softcap=float(a.get("softcap") or 0.0), conv=int(a["conv"]),
+                head_norm=True, chunk=int(a["mask"]["size"]),
+                unit_sink=True),
+            right=SelectiveScanSpec(
+                inner=int(r["inner"]), state=int(r["state"]),
+                dt_rank=int(r["dt_rank"]), conv=int(r["conv"])),
+            left_scale=float(m["left_scale"]),
+            right_scale=float(m["right_scale"]))
+    raise ValueError(f"unknown mixer type {kind!r}")
+
+
+def puvapel_config_from_json(d: dict) -> HybridConfig:
+    """Read a Puvapel ``config.json`` (already parsed)."""
+    layers = [HybridLayerSpec(_puvapel_mixer_from_json(L["type"], L["mixer"]),
+                              _ff_from_json(L.get("mlp")))
+              for L in d["layers"]]
+    return HybridConfig(
+        arch="puvapel", vocab_size=int(d["vocab"]),
+        hidden_size=int(d["width"]), layers=layers,
+        norm_eps=float(d["norm"]["eps"]), canon_taps=1, token_side_dim=0,
+        layer_style="postnorm", norm_offset=1.0,
+        logit_softcap=float(d.get("logit_softcap") or 0.0)).validate()
+
+
+def puvapel_config_to_json(cfg: HybridConfig) -> dict:
+    """Inverse of :func:`puvapel_config_from_json` (checkpoint export)."""
+    layers = []
+    for L in cfg.layers:
+        m = L.mixer
+        if m.kind == "channel_delta":
+            mj = {"heads": m.heads, "kv_heads": m.kv_heads, "dim": m.dim,
+                  "vdim": m.vdim, "conv": m.conv}
+        else:
+            a, r = m.left, m.right
+            mj = {"left": {"heads": a.heads, "kv_heads": a.kv_heads,
+                           "dim": a.dim, "vdim": a.vdim, "scale": a.scale,
+                           "softcap": a.softcap, "conv": a.conv,
+                           "mask": {"size": a.chunk}},
+                  "left_scale": m.left_scale,
+                  "right": {"inner": r.inner, "state": r.state,
+                            "dt_rank": r.dt_rank, "conv": r.conv},
+                  "right_scale": m.right_scale}
+            if a.rope is not None:
+                mj["left"]["rot"] = {"base": a.rope.base, "dims": a.rope.dims}
+        layers.append({"type": m.kind, "mixer": mj,
+                       "mlp": None if L.ff is None else
+                       {"kind": "dense", "ff": L.ff.ff}})
+    return {"architecture": "Puvapel", "vocab": cfg.vocab_size,
+            "width": cfg.hidden_size, "layers": layers,
+            "norm": {"eps": cfg.norm_eps},
+            "logit_softcap": cfg.logit_softcap}
+
+
+def puvapel_preset(width: int, layers: int, vocab: int = 32000,
+                   heads: int = 16, kv_heads: int = 4, ff: int = 0,
+                   chunk: int = 1024, inner: int = 0, state: int = 16,
+                   pattern=("channel_delta", "channel_delta",
+                            "channel_delta", "parallel")) -> HybridConfig:
+    """A Puvapel stack of realistic layer sizes (random weights): the mixer
+    kinds cycle through ``pattern``; every layer has the gated
+    feed-forward."""
+    hd = width // heads
+    rank = max(4, width // 16)
+    ff = ff or int(width * 2.75) // 64 * 64
+    out = []
+    for li in range(layers):
+        if pattern[li % len(pattern)] == "channel_delta":
+            mixer = ChannelDeltaSpec(heads=heads, kv_heads=heads, dim=hd,
+                                     vdim=hd, conv=4, decay_rank=rank,
+                                     gate_rank=rank)
+        else:
+            mixer = ParallelMixerSpec(
+                left=WindowAttnSpec(
+                    heads=heads, kv_heads=kv_heads, dim=hd, vdim=hd,
+                    window=UNBOUNDED, scale=1.0 / math.sqrt(hd),
+                    rope=RopeSpec(dims=hd // 2, base=500000.0), softcap=30.0,
+                    conv=3, head_norm=True, chunk=chunk, unit_sink=True),
+                right=SelectiveScanSpec(inner=inner or width, state=state,
+                                        dt_rank=max(2, width // 16), conv=4),
+                left_scale=0.7, right_scale=0.8)
+        out.append(HybridLayerSpec(mixer, FFSpec("dense", ff)))
+    return HybridConfig(arch="puvapel", vocab_size=vocab, hidden_size=width,
+                        layers=out, norm_eps=1e-5, canon_taps=1,
+                        token_side_dim=0, layer_style="postnorm",
+                        norm_offset=1.0, logit_softcap=30.0).validate()
+
+
 def read_config_dir(path: str):
     """Model config from a checkpoint folder's ``config.json``.  The
     ``architecture`` key names the family; HF-style folders
@@ -948,6 +1134,8 @@ def read_config_dir(path: str):
         return vurivik_config_from_json(d)
     if arch == "Nasipel":
         return nasipel_config_from_json(d)
+    if arch == "Puvapel":
+        return puvapel_config_from_json(d)
     mt = d.get("model_type")
     if mt in ("llama", "qwen2"):
         from .registry import DecoderConfig

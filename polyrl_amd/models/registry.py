@@ -108,8 +108,13 @@ MODEL_CONFIGS = {
 
 def _hybrid_presets():
     from .hybrid import (bizusun_preset, kuforax_preset, nasipel_preset,
-                         vurivik_preset)
+                         puvapel_preset, vurivik_preset)
     return {
+        # tiny stack for CPU unit tests / fast GPU smoke
+        "puvapel-debug": lambda: puvapel_preset(
+            width=64, layers=3, vocab=300, heads=4, kv_heads=2, ff=96,
+            chunk=24, inner=80, state=8,
+            pattern=("channel_delta", "parallel", "channel_delta")),
         # tiny stack for CPU unit tests / fast GPU smoke
         "nasipel-debug": lambda: nasipel_preset(
             width=64, layers=4, vocab=300, heads=4, kv_heads=2, experts=6,

@@ -19,7 +19,25 @@ void seq_gla_scan(torch::Tensor out, torch::Tensor q, torch::Tensor k,
 void seq_causal_conv(torch::Tensor out, torch::Tensor x, torch::Tensor w,
                      torch::Tensor bias, torch::Tensor state,
                      torch::Tensor cu_q, torch::Tensor state_slot,
-                     torch::Tensor seq_of_tok, bool add_input, bool act_silu);
+                     torch::Tensor seq_of_tok, bool add_input, bool act_silu,
+                     int64_t max_rows);
+void seq_postnorm_join(torch::Tensor out, torch::Tensor res, torch::Tensor y,
+                       torch::Tensor weight, double eps, double offset);
+void seq_softcap(torch::Tensor out, torch::Tensor x, double cap);
+void seq_channel_delta(torch::Tensor out, torch::Tensor q, torch::Tensor k,
+                       torch::Tensor v, torch::Tensor b_lin,
+                       torch::Tensor z_lin, torch::Tensor dt_bias,
+                       torch::Tensor a_log, torch::Tensor gate,
+                       torch::Tensor norm_w, torch::Tensor state,
+                       torch::Tensor cu_q, torch::Tensor state_slot,
+                       double key_eps, double eps);
+void seq_selective_scan(torch::Tensor out, torch::Tensor x,
+                        torch::Tensor dt_lin, torch::Tensor dt_bias,
+                        torch::Tensor Bm, torch::Tensor Cm,
+                        torch::Tensor a_log, torch::Tensor d_skip,
+                        torch::Tensor z, torch::Tensor state,
+                        torch::Tensor cu_q, torch::Tensor state_slot,
+                        double out_scale);
 void seq_group_rmsnorm(torch::Tensor out, torch::Tensor y,
                        torch::Tensor weight, int64_t groups, double eps,
                        torch::Tensor gate, int64_t gate_act);
@@ -94,7 +112,8 @@ void seq_gqa_window_attention(torch::Tensor out, torch::Tensor q,
                               double scale, torch::Tensor sink,
                               double q_temp_coef, int64_t q_temp_every,
                               double softcap, torch::Tensor head_bias,
-                              bool sigmoid_weights, torch::Tensor v_inv_freq);
+                              bool sigmoid_weights, torch::Tensor v_inv_freq,
+                              int64_t chunk, double out_scale);
 void seq_gqa_window_attention_mfma(
     torch::Tensor out, torch::Tensor q, torch::Tensor tile_n0,
     torch::Tensor tile_cnt, torch::Tensor cache, torch::Tensor page_table,
@@ -103,7 +122,8 @@ void seq_gqa_window_attention_mfma(
     torch::Tensor rel, torch::Tensor dist_bucket, torch::Tensor gate,
     double scale, torch::Tensor sink, double q_temp_coef,
     int64_t q_temp_every, double softcap, torch::Tensor head_bias,
-    bool sigmoid_weights, torch::Tensor v_inv_freq);
+    bool sigmoid_weights, torch::Tensor v_inv_freq, int64_t chunk,
+    double out_scale);
 void seq_moe_route(torch::Tensor idx, torch::Tensor w, torch::Tensor logits,
                    torch::Tensor correction, int64_t groups, int64_t keep,
                    int64_t act, int64_t group_top);
@@ -134,6 +154,13 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
         "real-gated linear recurrence (fp32 state, in place)");
   m.def("seq_moe_weighted_combine", &seq_moe_weighted_combine,
         "weighted sum of chosen experts, identity experts and shared");
+  m.def("seq_postnorm_join", &seq_postnorm_join,
+        "fp32 residual += normed branch, cast to the next input");
+  m.def("seq_softcap", &seq_softcap, "cap * tanh(x / cap) as fp32");
+  m.def("seq_channel_delta", &seq_channel_delta,
+        "gated delta rule with per-channel decays, head norm and gate");
+  m.def("seq_selective_scan", &seq_selective_scan,
+        "selective scan with per-channel steps and output gate");
   m.def("seq_embed_compose", &seq_embed_compose,
         "scaled embedding row + hashed pair row + sinusoid, fp32");
   m.def("seq_gla_scan", &seq_gla_scan,

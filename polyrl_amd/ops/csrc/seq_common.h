@@ -41,6 +41,75 @@ DEV_INLINE float lanegroup_sum(float x) {
   return x;
 }
 
+// sum over the four lanes 4j .. 4j+3 by two
+// quad permutes in the VALU data path: partner lane^2, then lane^1
+DEV_INLINE float quad_sum(float x) {
+  x += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(
+      0, __builtin_bit_cast(int, x), 0x4E, 0xF, 0xF, false));  // [2,3,0,1]
+  x += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(
+      0, __builtin_bit_cast(int, x), 0xB1, 0xF, 0xF, false));  // [1,0,3,2]
+  return x;
+}
+
+// sum over the eight lanes 8j .. 8j+7: the quads, then the mirrored half row
+DEV_INLINE float oct_sum(float x) {
+  x = quad_sum(x);
+  x += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(
+      0, __builtin_bit_cast(int, x), 0x141, 0xF, 0xF, false));
+  return x;
+}
+
+// four consecutive numbers as fp32: one 8- or 16-byte load when ``vec`` (the
+// caller has checked the alignment and that all four exist), else the first
+// ``valid`` of them and zeros
+template <typename T>
+DEV_INLINE f32x4v load4(const T* p, int valid, bool vec) {
+  f32x4v o;
+  if (vec) {
+    if constexpr (sizeof(T) == 2) {
+      const uint2 r = *reinterpret_cast<const uint2*>(p);
+      o.v[0] = __builtin_bit_cast(float, r.x << 16);
+      o.v[1] = __builtin_bit_cast(float, r.x & 0xffff0000u);
+      o.v[2] = __builtin_bit_cast(float, r.y << 16);
+      o.v[3] = __builtin_bit_cast(float, r.y & 0xffff0000u);
+    } else {
+      o = *reinterpret_cast<const f32x4v*>(p);
+    }
+    return o;
+  }
+#pragma unroll
+  for (int e = 0; e < 4; ++e) o.v[e] = e < valid ? ldf(p + e) : 0.f;
+  return o;
+}
+
+template <typename T>
+DEV_INLINE void store4(T* p, const f32x4v& x, int valid, bool vec) {
+  if (vec) {
+    if constexpr (sizeof(T) == 2) {
+      T q[4];
+#pragma unroll
+      for (int e = 0; e < 4; ++e) stf(q + e, x.v[e]);
+      uint2 r;
+      __builtin_memcpy(&r, q, 8);
+      *reinterpret_cast<uint2*>(p) = r;
+    } else {
+      *reinterpret_cast<f32x4v*>(p) = x;
+    }
+    return;
+  }
+#pragma unroll
+  for (int e = 0; e < 4; ++e)
+    if (e < valid) stf(p + e, x.v[e]);
+}
+
+// host check for load4 / store4's vector form: the view's base, row stride
+// and a column offset are multiples of four elements and aligned to them
+template <typename T>
+static bool rows_by4(const torch::Tensor& t, long cols) {
+  return (uintptr_t)t.data_ptr() % (4 * sizeof(T)) == 0 &&
+         t.stride(0) % 4 == 0 && cols % 4 == 0;
+}
+
 // activation-type dispatch on a torch dtype
 #define SEQ_DISPATCH_T(dtype, ...)                                   \
   do {                                                               \

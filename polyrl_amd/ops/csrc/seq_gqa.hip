@@ -32,7 +32,10 @@
 // weights sigmoid(score) per visible key with no normalisation over the
 // keys (the running maximum and sum are then unused).  The head sums can be
 // written as fp32 to a separate buffer for a pass that turns them back by
-// the row's position.
+// the row's position.  Keys can be confined to the row's own chunk of
+// positions (chunk > 0: floor(j / chunk) = floor(p / chunk)); the result can
+// go to a column slice of a wider row and be multiplied by a number before
+// it is rounded.
 #include <torch/extension.h>
 #include <ATen/hip/HIPContext.h>
 
@@ -164,6 +167,87 @@ __global__ __launch_bounds__(256) void gqa_prepare_heads_kernel(
   }
 }
 
+// One wave per ``hpw`` heads of a token (H query, G key, G value heads; four
+// waves a block, grid (tokens, waves / 4)).  Query and key heads: RMS norm
+// over the head with a weight row shared by the heads, then rotate the first
+// 2*half entries; the wave takes the token's cos and sin once for all its
+// heads, and a head's normed numbers meet their partners in a wave-private
+// LDS row.  Value heads are copied.
+template <typename T>
+__global__ __launch_bounds__(256) void gqa_prepare_headnorm_kernel(
+    T* __restrict__ q_out, const T* __restrict__ q, long ldq,
+    const T* __restrict__ k, long ldk, const T* __restrict__ v, long ldv,
+    const float* __restrict__ qn, const float* __restrict__ kn, float eps,
+    const float* __restrict__ inv_freq, int half, float amp,
+    const int* __restrict__ positions, T* __restrict__ cache,
+    const int* __restrict__ slot_mapping, int H, int G, int D, int Dv,
+    int hpw) {
+  extern __shared__ float lds[];
+  const long n = blockIdx.x;
+  const int wid = threadIdx.x >> 6, lane = threadIdx.x & 63;
+  const int h0 = (blockIdx.y * 4 + wid) * hpw;
+  const int h1 = min(h0 + hpw, H + 2 * G);
+  if (h0 >= h1) return;                 // whole wave; no barrier follows
+  float* xs = lds + wid * (D + 2 * half);
+  float* cs = xs + D;                   // [half cosines | half sines]
+  T* crow = cache + (long)slot_mapping[n] * (G * (D + Dv));
+  if (h0 < H + G) {
+    const float pos = (float)positions[n];
+    for (int i = lane; i < half; i += 64) {
+      const float ang = pos * inv_freq[i];
+      cs[i] = cosf(ang) * amp;
+      cs[half + i] = sinf(ang) * amp;
+    }
+  }
+  __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+  for (int hu = h0; hu < h1; ++hu) {
+    if (hu >= H + G) {
+      const T* src = v + n * ldv + (long)(hu - H - G) * Dv;
+      T* dst = crow + G * D + (hu - H - G) * Dv;
+      for (int i = lane; i < Dv; i += 64) dst[i] = src[i];
+      continue;
+    }
+    const bool isq = hu < H;
+    const T* src = isq ? q + n * ldq + (long)hu * D
+                       : k + n * ldk + (long)(hu - H) * D;
+    T* dst = isq ? q_out + (n * H + hu) * D : crow + (hu - H) * D;
+    const float* w = isq ? qn : kn;
+    float x[8];                         // D <= 512
+    float ss = 0.f;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      const int i = lane + 64 * e;
+      if (64 * e >= D) break;
+      x[e] = i < D ? ldf(src + i) : 0.f;
+      ss += x[e] * x[e];
+    }
+    const float inv = rsqrtf(wave_reduce_sum(ss) / D + eps);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      const int i = lane + 64 * e;
+      if (64 * e >= D) break;
+      if (i < D) {
+        x[e] *= inv * w[i];
+        xs[i] = x[e];
+      }
+    }
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      const int i = lane + 64 * e;
+      if (64 * e >= D) break;
+      if (i < D) {
+        float y = x[e];
+        if (i < half) y = x[e] * cs[i] - xs[i + half] * cs[half + i];
+        else if (i < 2 * half)
+          y = x[e] * cs[i - half] + xs[i - half] * cs[i];
+        stf(dst + i, y);
+      }
+    }
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+  }
+}
+
 void seq_gqa_prepare_store(torch::Tensor q_out, torch::Tensor q,
                            torch::Tensor k, torch::Tensor v,
                            torch::Tensor q_norm, torch::Tensor k_norm,
@@ -179,6 +263,7 @@ void seq_gqa_prepare_store(torch::Tensor q_out, torch::Tensor q,
   const long N = q.size(0);
   const bool has_v = v.defined() && v.numel() > 0;
   const bool has_norm = q_norm.defined() && q_norm.numel() > 0;
+  const bool head_norm = has_norm && q_norm.numel() == D;   // per head
   const int half = inv_freq.defined() ? (int)inv_freq.numel() : 0;
   TORCH_CHECK(H > 0 && G > 0 && H % G == 0 && D > 0 && Dv > 0);
   TORCH_CHECK(q.size(1) == H * D && k.size(0) == N && k.size(1) == G * D);
@@ -194,7 +279,8 @@ void seq_gqa_prepare_store(torch::Tensor q_out, torch::Tensor q,
   if (has_norm) {
     CHECK_F32(q_norm);
     CHECK_F32(k_norm);
-    TORCH_CHECK(q_norm.numel() == H * D && k_norm.numel() == G * D);
+    TORCH_CHECK(head_norm ? k_norm.numel() == D
+                          : q_norm.numel() == H * D && k_norm.numel() == G * D);
   }
   if (half) CHECK_F32(inv_freq);
   TORCH_CHECK(cache.is_cuda() && cache.is_contiguous() && cache.dim() == 3 &&
@@ -205,6 +291,25 @@ void seq_gqa_prepare_store(torch::Tensor q_out, torch::Tensor q,
   if (N == 0) return;
   auto stream = at::hip::getCurrentHIPStream();
   const bool v_rot = v_inv_freq.defined() && v_inv_freq.numel() > 0;
+  if (head_norm) {
+    TORCH_CHECK(has_v && !head_unit && !v_rot,
+                "per-head norm weights: values of their own, no other option");
+    TORCH_CHECK(D <= 512, "head sizes above 512 are not supported");
+    // heads per wave: enough waves to fill the chip first
+    const int heads = (int)(H + 2 * G);
+    const int hpw = N >= 4096 ? 8 : N >= 1024 ? 4 : 1;
+    const dim3 grid(N, (heads + 4 * hpw - 1) / (4 * hpw));
+    SEQ_DISPATCH_T(ty, { hipLaunchKernelGGL((gqa_prepare_headnorm_kernel<T>),
+        grid, dim3(256), 4 * (D + 2 * half) * sizeof(float), stream,
+        (T*)q_out.data_ptr(), (const T*)q.data_ptr(), q.stride(0),
+        (const T*)k.data_ptr(), k.stride(0), (const T*)v.data_ptr(),
+        v.stride(0), q_norm.data_ptr<float>(), k_norm.data_ptr<float>(),
+        (float)eps, half ? inv_freq.data_ptr<float>() : nullptr, half,
+        (float)amp, positions.data_ptr<int>(), (T*)cache.data_ptr(),
+        slot_mapping.data_ptr<int>(), (int)H, (int)G, (int)D, (int)Dv, hpw); });
+    HIP_CHECK_KERNEL();
+    return;
+  }
   if (head_unit || v_rot) {
     TORCH_CHECK(!has_norm, "whole-row and per-head norms do not combine");
     TORCH_CHECK(has_v, "the per-head writer needs a value projection");
@@ -309,7 +414,7 @@ struct Vec16<float> {
 // value row per key.  The waves never meet at a block barrier.
 template <typename T, int NCH>
 __global__ __launch_bounds__(256) void gqa_attn_kernel(
-    T* __restrict__ out,                // (N, H*Dv)
+    T* __restrict__ out,                // (N, H*Dv), row stride ldo
     const T* __restrict__ q,            // (N, H*D) contiguous
     const T* __restrict__ cache,        // (pages*page_size, G*(D+Dv))
     const int* __restrict__ page_table, int max_pages,
@@ -320,7 +425,8 @@ __global__ __launch_bounds__(256) void gqa_attn_kernel(
     int H, int G, int D, int Dv, int page_size, int window, int keep,
     float scale, bool vec, int lpr, const float* __restrict__ sink,
     float qt_coef, int qt_every, float cap, const float* __restrict__ hbias,
-    bool sigm, float* __restrict__ out32) {
+    bool sigm, float* __restrict__ out32, int chunk, long ldo,
+    float out_scale) {
   constexpr int EPL = Vec16<T>::N;
   __shared__ float q_sh[4][NCH * 64];
   __shared__ float p_sh[4][64];
@@ -337,7 +443,8 @@ __global__ __launch_bounds__(256) void gqa_attn_kernel(
   const int* ptab = page_table + (long)b * max_pages;
   if (qt_coef != 0.f)
     scale *= 1.f + qt_coef * logf((float)((pos + 1) / qt_every + 1));
-  const int lo = pos - window + 1 > 0 ? pos - window + 1 : 0;
+  int lo = pos - window + 1 > 0 ? pos - window + 1 : 0;
+  if (chunk > 0) lo = max(lo, pos / chunk * chunk);
   const int nkeep = keep < lo ? keep : lo;
   const int total = nkeep + (pos - lo + 1);
   float* qs = q_sh[wid];
@@ -410,7 +517,7 @@ __global__ __launch_bounds__(256) void gqa_attn_kernel(
       }
     }
   }
-  float inv = sigm ? 1.f : 1.f / l;
+  float inv = (sigm ? 1.f : 1.f / l) * out_scale;
   if (gate && !out32) inv *= sigmoidf_acc(ldf(gate + n * ldg + h));
   if (lpr) {
 #pragma unroll
@@ -421,7 +528,7 @@ __global__ __launch_bounds__(256) void gqa_attn_kernel(
 #pragma unroll
       for (int k = 0; k < EPL; ++k) {
         if (out32) out32[(n * H + h) * Dv + dcol + k] = ov[k] * inv;
-        else stf(out + (n * H + h) * Dv + dcol + k, ov[k] * inv);
+        else stf(out + n * ldo + h * Dv + dcol + k, ov[k] * inv);
       }
     }
     return;
@@ -431,7 +538,7 @@ __global__ __launch_bounds__(256) void gqa_attn_kernel(
     const int d = lane + 64 * c;
     if (d < Dv) {
       if (out32) out32[(n * H + h) * Dv + d] = o[c] * inv;
-      else stf(out + (n * H + h) * Dv + d, o[c] * inv);
+      else stf(out + n * ldo + h * Dv + d, o[c] * inv);
     }
   }
 }
@@ -455,7 +562,7 @@ void gqa_attention_check(torch::Tensor out, torch::Tensor q,
               keep_first >= 0);
   TORCH_CHECK(q.is_cuda() && q.is_contiguous() && q.dim() == 2 &&
               q.size(1) == H * D);
-  TORCH_CHECK(out.is_cuda() && out.is_contiguous() && out.dim() == 2 &&
+  TORCH_CHECK(out.is_cuda() && out.dim() == 2 && out.stride(1) == 1 &&
               out.size(0) == N && out.size(1) == H * Dv);
   TORCH_CHECK(cache.is_cuda() && cache.is_contiguous() && cache.dim() == 3 &&
               cache.size(2) == G * (D + Dv), "cache row must be G*(D+Dv)");
@@ -496,7 +603,7 @@ void gqa_attention_check(torch::Tensor out, torch::Tensor q,
       lpr, has_sink ? sink.data_ptr<float>() : nullptr, (float)q_temp_coef,   \
       (int)q_temp_every, (float)softcap,                                      \
       has_hb ? head_bias.data_ptr<float>() : nullptr, sigmoid_weights,        \
-      o32)
+      o32, (int)chunk, (long)out.stride(0), (float)out_scale)
 
 void seq_gqa_window_attention(torch::Tensor out, torch::Tensor q,
                               torch::Tensor cache, torch::Tensor page_table,
@@ -508,7 +615,8 @@ void seq_gqa_window_attention(torch::Tensor out, torch::Tensor q,
                               double scale, torch::Tensor sink,
                               double q_temp_coef, int64_t q_temp_every,
                               double softcap, torch::Tensor head_bias,
-                              bool sigmoid_weights, torch::Tensor v_inv_freq) {
+                              bool sigmoid_weights, torch::Tensor v_inv_freq,
+                              int64_t chunk, double out_scale) {
   gqa_attention_check(out, q, cache, page_table, seq_of_tok, positions, H, G,
                       D, Dv, window, keep_first, rel, dist_bucket, gate, sink,
                       q_temp_every);
@@ -526,6 +634,8 @@ void seq_gqa_window_attention(torch::Tensor out, torch::Tensor q,
   const bool v_rot = v_inv_freq.defined() && v_inv_freq.numel() > 0;
   torch::Tensor sums;
   float* o32 = nullptr;
+  TORCH_CHECK(chunk >= 0 && (!v_rot || (out.is_contiguous() && out_scale == 1.0)),
+              "rotated values are written unscaled to whole rows");
   if (v_rot) {
     sums = torch::empty({q.size(0), H * Dv}, q.options().dtype(torch::kFloat32));
     o32 = sums.data_ptr<float>();

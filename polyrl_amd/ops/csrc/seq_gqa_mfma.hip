@@ -7,7 +7,8 @@
 // of 32 -- first the kept first tokens that lie before the union's window
 // ([0, min(keep, kmin))), then [kmin, last position] -- and masks per
 // element: key j is live for the row at position p when j <= p and
-// (p - j < window or j < keep).  K and V tiles of the head's key/value group
+// (p - j < window or j < keep); with chunks a windowed key must also lie in
+// the row's own chunk of positions.  K and V tiles of the head's key/value group
 // come from the paged cache rows ([G*D keys | G*Dv values]) into LDS; QK^T
 // and P.V run on v_mfma_f32_16x16x32_bf16 with fp32 accumulators; scale, the
 // optional distance-bucket bias (this head's column of the table sits in
@@ -37,6 +38,13 @@
 
 #include "seq_common.h"
 
+// tanh through the hardware exponential and reciprocal: 1 - 2 / (1 + e^2x),
+// absolute error a few 1e-7, exact limits for large |x|
+DEV_INLINE float tanhf_fast(float x) {
+  return 1.f - 2.f * __builtin_amdgcn_rcpf(
+                         1.f + __builtin_amdgcn_exp2f(2.8853900817779268f * x));
+}
+
 typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8_t;
 typedef __attribute__((ext_vector_type(4))) float f32x4_t;
 typedef __attribute__((ext_vector_type(4))) int i32x4_t;
@@ -52,7 +60,7 @@ DEV_INLINE int gtile_off(int row, int byte_col) {
 
 template <int KS>
 __global__ __launch_bounds__(256) void gqa_attn_mfma_kernel(
-    bf16_t* __restrict__ out,            // (N, H*Dv)
+    bf16_t* __restrict__ out,            // (N, H*Dv), row stride ldo
     const bf16_t* __restrict__ q,        // (N, H*D)
     const bf16_t* __restrict__ cache,    // (slots, G*(D+Dv))
     const int* __restrict__ page_table, int max_pages,
@@ -63,7 +71,8 @@ __global__ __launch_bounds__(256) void gqa_attn_mfma_kernel(
     const bf16_t* __restrict__ gate, long ldg, int H, int G, int D, int Dv,
     int page_size, int window, int keep, float scale,
     const float* __restrict__ sink, float qt_coef, int qt_every, float cap,
-    const float* __restrict__ hbias, bool sigm, float* __restrict__ out32) {
+    const float* __restrict__ hbias, bool sigm, float* __restrict__ out32,
+    int chunk, long ldo, float out_scale) {
   constexpr int DKP = KS * 32;           // padded head size in LDS
   constexpr int NVT = KS * 2;            // 16-wide output tiles
   __shared__ __attribute__((aligned(16))) bf16_t Ks[GKV * DKP];
@@ -95,7 +104,13 @@ __global__ __launch_bounds__(256) void gqa_attn_mfma_kernel(
   const int* ptab = page_table + (long)b * max_pages;
   const int pos0 = positions[n0];
   const int pmax = pos0 + cnt - 1;
-  const int kmin = pos0 - window + 1 > 0 ? pos0 - window + 1 : 0;
+  // first windowed key of the row at position p
+  auto row_lo = [&](int p) {
+    int lo = p - window + 1 > 0 ? p - window + 1 : 0;
+    if (chunk > 0) lo = max(lo, p / chunk * chunk);
+    return lo;
+  };
+  const int kmin = row_lo(pos0);
   const int nk = keep < kmin ? keep : kmin;      // kept keys before kmin
   const int nkt = (nk + GKV - 1) / GKV;          // their tiles
   const int nwt = (pmax - kmin) / GKV + 1;       // window tiles
@@ -120,7 +135,7 @@ __global__ __launch_bounds__(256) void gqa_attn_mfma_kernel(
   const float hb = hbias ? hbias[h] : 0.f;
   const float inv_cap = cap > 0.f ? 1.f / cap : 0.f;
   float m_run[4], l_run[4], rscale[4];
-  int rpos[4];
+  int rpos[4], rlo[4];
   bool rok[4];
   f32x4_t o_acc[NVT];
 #pragma unroll
@@ -129,6 +144,7 @@ __global__ __launch_bounds__(256) void gqa_attn_mfma_kernel(
     m_run[r] = sink ? sink[h] : -1e30f;
     l_run[r] = sink ? 1.f : 0.f;
     rpos[r] = pos0 + i;
+    rlo[r] = row_lo(rpos[r]);
     rok[r] = i < cnt;
     rscale[r] = scale;
     if (qt_coef != 0.f)
@@ -208,10 +224,10 @@ __global__ __launch_bounds__(256) void gqa_attn_mfma_kernel(
         const int j = t0 + nt * 16 + l15;
         const int dist = rpos[r] - j;
         const bool live = rok[r] && j <= jmax && dist >= 0 &&
-                          (dist < window || j < keep);
+                          (j >= rlo[r] || j < keep);
         float sv = c[nt][r] * rscale[r];
         if (rel && live) sv += rel_s[dist_bucket[dist]];
-        if (cap > 0.f) sv = cap * tanhf(sv * inv_cap);
+        if (cap > 0.f) sv = cap * tanhf_fast(sv * inv_cap);
         sv += hb;
         s[nt] = live ? sv : -1e30f;
       }
@@ -279,9 +295,9 @@ __global__ __launch_bounds__(256) void gqa_attn_mfma_kernel(
     const int i = wid * 16 + lhi * 4 + r;
     if (!rok[r]) continue;
     const long tok = n0 + i;
-    float inv = sigm ? 1.f : 1.f / l_run[r];
+    float inv = (sigm ? 1.f : 1.f / l_run[r]) * out_scale;
     if (gate && !out32) inv *= sigmoidf_acc(bf2f(gate[tok * ldg + h]));
-    bf16_t* op = out + (tok * H + h) * Dv;
+    bf16_t* op = out + tok * ldo + h * Dv;
     float* op32 = out32 ? out32 + (tok * H + h) * Dv : nullptr;
 #pragma unroll
     for (int nt = 0; nt < NVT; ++nt) {
@@ -312,7 +328,8 @@ void seq_gqa_window_attention(torch::Tensor out, torch::Tensor q,
                               double scale, torch::Tensor sink,
                               double q_temp_coef, int64_t q_temp_every,
                               double softcap, torch::Tensor head_bias,
-                              bool sigmoid_weights, torch::Tensor v_inv_freq);
+                              bool sigmoid_weights, torch::Tensor v_inv_freq,
+                              int64_t chunk, double out_scale);
 void seq_rotate_back_heads(torch::Tensor out, torch::Tensor x,
                            torch::Tensor inv_freq, torch::Tensor positions,
                            torch::Tensor gate, int64_t H);
@@ -332,7 +349,8 @@ void seq_rotate_back_heads(torch::Tensor out, torch::Tensor x,
       (int)cache.size(1), (int)window, (int)keep_first, (float)scale,         \
       has_sink ? sink.data_ptr<float>() : nullptr, (float)q_temp_coef,        \
       (int)q_temp_every, (float)softcap,                                      \
-      has_hb ? head_bias.data_ptr<float>() : nullptr, sigmoid_weights, o32)
+      has_hb ? head_bias.data_ptr<float>() : nullptr, sigmoid_weights, o32,   \
+      (int)chunk, (long)out.stride(0), (float)out_scale)
 
 void seq_gqa_window_attention_mfma(
     torch::Tensor out, torch::Tensor q, torch::Tensor tile_n0,
@@ -342,7 +360,8 @@ void seq_gqa_window_attention_mfma(
     torch::Tensor rel, torch::Tensor dist_bucket, torch::Tensor gate,
     double scale, torch::Tensor sink, double q_temp_coef,
     int64_t q_temp_every, double softcap, torch::Tensor head_bias,
-    bool sigmoid_weights, torch::Tensor v_inv_freq) {
+    bool sigmoid_weights, torch::Tensor v_inv_freq, int64_t chunk,
+    double out_scale) {
   gqa_attention_check(out, q, cache, page_table, seq_of_tok, positions, H, G,
                       D, Dv, window, keep_first, rel, dist_bucket, gate, sink,
                       q_temp_every);
@@ -358,7 +377,7 @@ void seq_gqa_window_attention_mfma(
                              H, G, D, Dv, window, keep_first, rel,
                              dist_bucket, gate, scale, sink, q_temp_coef,
                              q_temp_every, softcap, head_bias,
-                             sigmoid_weights, v_inv_freq);
+                             sigmoid_weights, v_inv_freq, chunk, out_scale);
     return;
   }
   const int ntiles = tile_n0.numel();
@@ -370,6 +389,8 @@ void seq_gqa_window_attention_mfma(
   }
   TORCH_CHECK(!sigmoid_weights || !has_sink, "a sink needs softmax weights");
   const bool v_rot = v_inv_freq.defined() && v_inv_freq.numel() > 0;
+  TORCH_CHECK(chunk >= 0 && (!v_rot || (out.is_contiguous() && out_scale == 1.0)),
+              "rotated values are written unscaled to whole rows");
   torch::Tensor sums;
   float* o32 = nullptr;
   if (v_rot) {

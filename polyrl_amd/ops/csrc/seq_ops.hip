@@ -145,6 +145,125 @@ void seq_add_rmsnorm(torch::Tensor out, torch::Tensor res, torch::Tensor y,
   HIP_CHECK_KERNEL();
 }
 
+// ------------------------------------------- normed branch joins, then cast
+// res += y / rms(y) * (off + w); out = res as T (nothing for fp32: the next
+// sublayer reads the stream).  One block per row; four consecutive numbers
+// per thread and step, a row of up to 1024*EPT numbers staying in registers
+// between the reduction and the stores (EPT = 0: read again).
+template <typename T, int EPT>
+__global__ __launch_bounds__(256) void postnorm_join_kernel(
+    T* __restrict__ out, float* __restrict__ res, const T* __restrict__ y,
+    long ldy, const float* __restrict__ w, int D, float eps, float off,
+    bool vec) {
+  __shared__ float red[8];
+  const long row = blockIdx.x;
+  float* rr = res + row * D;
+  const T* yr = y + row * ldy;
+  constexpr int NE = EPT > 0 ? EPT : 1;
+  f32x4v yv[NE], rv[NE];
+  float ss = 0.f;
+  if (EPT > 0) {
+#pragma unroll
+    for (int e = 0; e < EPT; ++e) {
+      const int i = (threadIdx.x + e * 256) * 4;
+      if (i < D) {
+        yv[e] = load4(yr + i, D - i, vec);
+        rv[e] = load4((const float*)rr + i, D - i, vec);
+      } else {
+        yv[e] = {{0.f, 0.f, 0.f, 0.f}};
+      }
+    }
+#pragma unroll
+    for (int e = 0; e < EPT; ++e)
+#pragma unroll
+      for (int c = 0; c < 4; ++c) ss += yv[e].v[c] * yv[e].v[c];
+  } else {
+    for (int i = threadIdx.x * 4; i < D; i += 1024) {
+      const f32x4v a = load4(yr + i, D - i, vec);
+#pragma unroll
+      for (int c = 0; c < 4; ++c) ss += a.v[c] * a.v[c];
+    }
+  }
+  const float inv = rsqrtf(block_reduce_sum<4>(ss, red) / D + eps);
+  auto join = [&](int i, const f32x4v& a, f32x4v r) {
+    const f32x4v wv = load4(w + i, D - i, vec);
+#pragma unroll
+    for (int c = 0; c < 4; ++c) r.v[c] += a.v[c] * inv * (wv.v[c] + off);
+    store4(rr + i, r, D - i, vec);
+    if (out) store4(out + row * D + i, r, D - i, vec);
+  };
+  if (EPT > 0) {
+#pragma unroll
+    for (int e = 0; e < EPT; ++e) {
+      const int i = (threadIdx.x + e * 256) * 4;
+      if (i < D) join(i, yv[e], rv[e]);
+    }
+  } else {
+    for (int i = threadIdx.x * 4; i < D; i += 1024)
+      join(i, load4(yr + i, D - i, vec),
+           load4((const float*)rr + i, D - i, vec));
+  }
+}
+
+#define POSTNORM_LAUNCH(EPTV)                                                 \
+  hipLaunchKernelGGL((postnorm_join_kernel<T, EPTV>), dim3(rows), dim3(256),  \
+      0, stream, cast ? (T*)out.data_ptr() : nullptr, res.data_ptr<float>(),  \
+      (const T*)y.data_ptr(), y.stride(0), weight.data_ptr<float>(), D,       \
+      (float)eps, (float)offset, vec)
+
+void seq_postnorm_join(torch::Tensor out, torch::Tensor res, torch::Tensor y,
+                       torch::Tensor weight, double eps, double offset) {
+  CHECK_F32(res);
+  CHECK_F32(weight);
+  CHECK_ROWS(y);
+  TORCH_CHECK(res.dim() == 2 && y.sizes() == res.sizes(), "branch shape");
+  const long rows = res.size(0);
+  const int D = res.size(1);
+  TORCH_CHECK(weight.numel() == D, "one norm weight per channel");
+  const bool cast = out.data_ptr() != res.data_ptr();
+  TORCH_CHECK(out.is_cuda() && out.is_contiguous() &&
+              out.sizes() == res.sizes() &&
+              (!cast || out.scalar_type() == y.scalar_type()));
+  if (rows == 0) return;
+  auto stream = at::hip::getCurrentHIPStream();
+  SEQ_DISPATCH_T(y.scalar_type(), {
+    const bool vec = rows_by4<T>(y, D) && rows_by4<float>(res, D) &&
+                     (uintptr_t)weight.data_ptr() % 16 == 0 &&
+                     (!cast || rows_by4<T>(out, D));
+    if (D <= 1024) POSTNORM_LAUNCH(1);
+    else if (D <= 2048) POSTNORM_LAUNCH(2);
+    else if (D <= 4096) POSTNORM_LAUNCH(4);
+    else if (D <= 8192) POSTNORM_LAUNCH(8);
+    else POSTNORM_LAUNCH(0);
+  });
+  HIP_CHECK_KERNEL();
+}
+
+// --------------------------------------------------------- capped logits
+template <typename T>
+__global__ void softcap_kernel(float* __restrict__ out,
+                               const T* __restrict__ x, float cap, long n) {
+  const float inv = 1.f / cap;
+  const long stride = (long)gridDim.x * blockDim.x;
+  for (long i = (long)blockIdx.x * blockDim.x + threadIdx.x; i < n;
+       i += stride)
+    out[i] = cap * tanhf(ldf(x + i) * inv);
+}
+
+void seq_softcap(torch::Tensor out, torch::Tensor x, double cap) {
+  TORCH_CHECK(x.is_cuda() && x.is_contiguous() && cap > 0.0);
+  CHECK_F32(out);
+  TORCH_CHECK(out.sizes() == x.sizes());
+  const long n = x.numel();
+  if (n == 0) return;
+  const long nblk = std::min<long>((n + 255) / 256, MAX_RESIDENT_BLOCKS * 4);
+  auto stream = at::hip::getCurrentHIPStream();
+  SEQ_DISPATCH_T(x.scalar_type(), {
+    hipLaunchKernelGGL((softcap_kernel<T>), dim3(nblk), dim3(256), 0, stream,
+        out.data_ptr<float>(), (const T*)x.data_ptr(), (float)cap, n); });
+  HIP_CHECK_KERNEL();
+}
+
 // ------------------------------------------------------ composed embedding
 // out[n] = table[tok] * scale [+ pair[row]] [+ sinusoid(pos)], fp32.
 // row = (prev * mul_prev + tok * mul_cur) mod buckets, or ``buckets`` (the
@@ -251,6 +370,73 @@ __global__ __launch_bounds__(256) void causal_conv_kernel(
   stf(out + (long)n * C + c, acc);
 }
 
+// The same for channel counts and row strides in multiples of four: a thread
+// owns four neighbouring channels (one 8- or 16-byte load per row) and walks
+// ``run`` packed rows with the last TAPS-1 inputs in registers; where a new
+// sequence begins, the window is filled again from its rows or its history.
+// ``single``: every sequence brings one row, and the thread that read its
+// history shifts the row into it.
+template <typename T, int TAPS>
+__global__ __launch_bounds__(256) void causal_conv_run_kernel(
+    T* __restrict__ out, const T* __restrict__ x, long ldx,
+    const float* __restrict__ w, const float* __restrict__ bias,
+    float* __restrict__ state, const int* __restrict__ cu_q,
+    const int* __restrict__ state_slot, const int* __restrict__ seq_of_tok,
+    int N, int C, bool add_input, bool act_silu, int run, bool single) {
+  constexpr int HN = TAPS > 1 ? TAPS - 1 : 1;
+  const int c = (blockIdx.y * 256 + threadIdx.x) * 4;
+  if (c >= C) return;
+  const int n0 = blockIdx.x * run;
+  const int n1 = n0 + run < N ? n0 + run : N;
+  float wv[4][TAPS], bv[4];
+#pragma unroll
+  for (int e = 0; e < 4; ++e) {
+    bv[e] = bias ? bias[c + e] : 0.f;
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) wv[e][j] = w[(long)(c + e) * TAPS + j];
+  }
+  f32x4v hist[HN];
+  int b = -1;
+  for (int n = n0; n < n1; ++n) {
+    const int bn = seq_of_tok[n];
+    if (bn != b) {
+      b = bn;
+      const int q0 = cu_q[b], t = n - q0;
+      const float* st = state + (long)state_slot[b] * (TAPS - 1) * C + c;
+#pragma unroll
+      for (int j = 0; j < TAPS - 1; ++j) {
+        const int src = t - (TAPS - 1) + j;
+        hist[j] = src >= 0 ? load4(x + (long)(q0 + src) * ldx + c, 4, true)
+                           : load4(st + (long)(TAPS - 1 + src) * C, 4, true);
+      }
+    }
+    const f32x4v cur = load4(x + (long)n * ldx + c, 4, true);
+    f32x4v y;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      float acc = bv[e];
+#pragma unroll
+      for (int j = 0; j < TAPS - 1; ++j) acc += wv[e][j] * hist[j].v[e];
+      acc += wv[e][TAPS - 1] * cur.v[e];
+      if (add_input) acc += cur.v[e];
+      if (act_silu) acc = siluf_acc(acc);
+      y.v[e] = acc;
+    }
+    store4(out + (long)n * C + c, y, 4, true);
+    if (TAPS > 1) {
+#pragma unroll
+      for (int j = 0; j < TAPS - 2; ++j) hist[j] = hist[j + 1];
+      hist[HN - 1] = cur;
+      if (single) {
+        float* st = state + (long)state_slot[b] * (TAPS - 1) * C + c;
+#pragma unroll
+        for (int j = 0; j < TAPS - 1; ++j)
+          store4(st + (long)j * C, hist[j], 4, true);
+      }
+    }
+  }
+}
+
 // new history = last taps-1 rows of [old history ; portion].  Ascending
 // order is safe in place: row i reads old row i+L (L >= 1), never a row
 // already overwritten; each thread owns one channel column.
@@ -274,10 +460,18 @@ __global__ __launch_bounds__(256) void conv_state_kernel(
   }
 }
 
+#define CONV_RUN(TAPSV)                                                       \
+hipLaunchKernelGGL((causal_conv_run_kernel<T, TAPSV>), grid, dim3(256),       \
+    0, stream, (T*)out.data_ptr(), (const T*)x.data_ptr(), x.stride(0),       \
+    w.data_ptr<float>(), bp, state.data_ptr<float>(),                         \
+    cu_q.data_ptr<int>(), state_slot.data_ptr<int>(),                         \
+    seq_of_tok.data_ptr<int>(), N, C, add_input, act_silu, run, single)
+
 void seq_causal_conv(torch::Tensor out, torch::Tensor x, torch::Tensor w,
                      torch::Tensor bias, torch::Tensor state,
                      torch::Tensor cu_q, torch::Tensor state_slot,
-                     torch::Tensor seq_of_tok, bool add_input, bool act_silu) {
+                     torch::Tensor seq_of_tok, bool add_input, bool act_silu,
+                     int64_t max_rows) {
   CHECK_ROWS(x);
   CHECK_F32(w);
   CHECK_F32(state);
@@ -300,6 +494,25 @@ void seq_causal_conv(torch::Tensor out, torch::Tensor x, torch::Tensor w,
   auto stream = at::hip::getCurrentHIPStream();
   const int cb = (C + 255) / 256;
   SEQ_DISPATCH_T(x.scalar_type(), {
+    const bool by4 = rows_by4<T>(x, C) && rows_by4<T>(out, C) &&
+                     (uintptr_t)state.data_ptr() % 16 == 0 && taps <= 4;
+    if (by4) {
+      // rows per thread: long runs once they leave enough waves to fill the
+      // chip; single-token steps finish with their history updated
+      const bool single = max_rows == 1;
+      const int run = single || N < 1024 ? 1 : N < 8192 ? 4 : 16;
+      const dim3 grid((N + run - 1) / run, (C / 4 + 255) / 256);
+      if (taps == 1) CONV_RUN(1);
+      else if (taps == 2) CONV_RUN(2);
+      else if (taps == 3) CONV_RUN(3);
+      else CONV_RUN(4);
+      if (taps > 1 && !single)
+        hipLaunchKernelGGL((conv_state_kernel<T>), dim3(B, cb), dim3(256), 0, stream,
+            state.data_ptr<float>(), (const T*)x.data_ptr(), x.stride(0),
+            cu_q.data_ptr<int>(), state_slot.data_ptr<int>(), C, taps);
+      HIP_CHECK_KERNEL();
+      return;
+    }
     hipLaunchKernelGGL((causal_conv_kernel<T>), dim3(N, cb), dim3(256), 0, stream, 
         (T*)out.data_ptr(), (const T*)x.data_ptr(), x.stride(0),
         w.data_ptr<float>(), bp, state.data_ptr<float>(),

@@ -248,16 +248,6 @@ void seq_delta_rule(torch::Tensor out, torch::Tensor r, torch::Tensor k,
 // the 16 column lanes of a row group read the same words (broadcast).  A
 // thread's words of the next tile are requested into registers before the
 // current tile is walked.
-// sum over the four lanes 4j .. 4j+3 (the row groups of one column) by two
-// quad permutes in the VALU data path: partner lane^2, then lane^1
-DEV_INLINE float quad_sum(float x) {
-  x += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(
-      0, __builtin_bit_cast(int, x), 0x4E, 0xF, 0xF, false));  // [2,3,0,1]
-  x += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(
-      0, __builtin_bit_cast(int, x), 0xB1, 0xF, 0xF, false));  // [1,0,3,2]
-  return x;
-}
-
 // tokens per LDS tile: at most 32, and the tile within 48 KB
 constexpr int gla_tile_tokens(int dkp) {
   const int fit = 48 * 1024 / (4 * (3 * dkp + 64));

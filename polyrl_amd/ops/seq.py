@@ -127,6 +127,33 @@ def embed_compose(table, tokens, scale: float, pair_table, prev_tokens,
                            mul_prev, mul_cur, buckets, positions, inv_freq)
 
 
+def add_unit_rms_then_cast(res: torch.Tensor, y: torch.Tensor,
+                           weight: torch.Tensor, eps: float,
+                           out_dtype: torch.dtype,
+                           offset: float = 0.0) -> torch.Tensor:
+    """The joint behind a sublayer whose output is normed and whose
+    successor reads the stream itself, in one pass over the row:
+    res += y / rms(y) * (offset + weight) in place; returns res as
+    out_dtype (res itself for fp32)."""
+    if res.is_cuda:
+        out = res if out_dtype == torch.float32 else \
+            torch.empty(res.shape, dtype=out_dtype, device=res.device)
+        if res.shape[0]:
+            _ext().seq_postnorm_join(out, res, y, weight, eps, offset)
+        return out
+    return R.add_unit_rms_then_cast(res, y, weight, eps, out_dtype, offset)
+
+
+def softcap_f32(x: torch.Tensor, cap: float) -> torch.Tensor:
+    """cap * tanh(x / cap) as fp32."""
+    if x.is_cuda:
+        out = torch.empty(x.shape, dtype=torch.float32, device=x.device)
+        if x.numel():
+            _ext().seq_softcap(out, x, cap)
+        return out
+    return R.softcap_f32(x, cap)
+
+
 def add_unit_rms_then_norm(res: torch.Tensor, y: torch.Tensor,
                            w_post: torch.Tensor, w_next: torch.Tensor,
                            eps: float, out_dtype: torch.dtype,
@@ -151,11 +178,13 @@ def add_unit_rms_then_norm(res: torch.Tensor, y: torch.Tensor,
 
 def causal_conv_state(x, w, bias, state, cu_q, state_slot, seq_of_tok,
                       add_input: bool, act_silu: bool,
-                      out_dtype) -> torch.Tensor:
+                      out_dtype, max_rows: int = 0) -> torch.Tensor:
     """Depthwise causal convolution over each sequence's rows with the last
     taps-1 inputs carried in ``state`` (slots, taps-1, C) fp32.
     y_t = sum_j w[:, j] x_(t-taps+1+j) [+ bias] [+ x_t], optional SiLU.
-    ``x`` may be a column slice (row-strided view)."""
+    ``x`` may be a column slice (row-strided view).  ``max_rows`` bounds the
+    rows of one sequence (0 = unknown): a step of single tokens updates the
+    history in the same launch."""
     if x.is_cuda:
         out = torch.empty(x.shape[0], w.shape[0], dtype=out_dtype,
                           device=x.device)
@@ -163,7 +192,7 @@ def causal_conv_state(x, w, bias, state, cu_q, state_slot, seq_of_tok,
             _ext().seq_causal_conv(out, x, w,
                                    bias if bias is not None else torch.Tensor(),
                                    state, cu_q, state_slot, seq_of_tok,
-                                   add_input, act_silu)
+                                   add_input, act_silu, max_rows)
         return out
     return R.causal_conv_state(x, w, bias, state, cu_q, state_slot,
                                seq_of_tok, add_input, act_silu, out_dtype)
@@ -242,6 +271,51 @@ def gla_scan(q, k, v, z_lin, z_bias, state, cu_q, state_slot,
         return out
     return R.gla_scan(q, k, v, z_lin, z_bias, state, cu_q, state_slot,
                       q_scale, inv_tau)
+
+
+def channel_delta_scan(q, k, v, b_lin, z_lin, dt_bias, a_log, gate, norm_w,
+                       state, cu_q, state_slot, key_eps: float, eps: float,
+                       out_dtype) -> torch.Tensor:
+    """Gated delta rule with per-channel decays over packed rows; ``state``
+    (slots, H, Dk, Dv) fp32 in place.  q, k (N, G*Dk): head h uses q/k head
+    h // (H/G); both are made unit vectors x / sqrt(sum x^2 + key_eps), q is
+    also multiplied by Dk^(-1/2).  Per head: beta = sigmoid(b_lin),
+    g = exp(-exp(a_log) * softplus(z_lin + dt_bias)) per key channel,
+    S <- g S, u = beta (v - S^T k), S <- S + k u^T, o = S^T q; returns
+    o / rms_head(o) * norm_w * sigmoid(gate) (N, H*Dv), norm_w (Dv,) shared
+    by the heads.  Inputs may be column slices."""
+    if q.is_cuda:
+        slots, H, Dk, Dv = state.shape
+        out = torch.empty(q.shape[0], H * Dv, dtype=out_dtype,
+                          device=q.device)
+        if q.shape[0]:
+            _ext().seq_channel_delta(out, q, k, v, b_lin, z_lin, dt_bias,
+                                     a_log, gate, norm_w, state, cu_q,
+                                     state_slot, key_eps, eps)
+        return out
+    return R.channel_delta_scan(q, k, v, b_lin, z_lin, dt_bias, a_log, gate,
+                                norm_w, state, cu_q, state_slot, key_eps,
+                                eps, out_dtype)
+
+
+def selective_scan(x, dt_lin, dt_bias, Bm, Cm, a_log, d_skip, z, state, cu_q,
+                   state_slot, out=None,
+                   out_scale: float = 1.0) -> torch.Tensor:
+    """Selective scan over packed rows; ``state`` (slots, C, Ns) fp32 in
+    place.  dt = softplus(dt_lin + dt_bias) per channel;
+    S <- exp(-exp(a_log) dt) S + dt x B^T, y = S C + d_skip x; returns
+    y * silu(z) * out_scale (N, C) in ``out`` (a column slice is allowed)
+    or a new tensor.  Inputs may be column slices."""
+    if x.is_cuda:
+        if out is None:
+            out = torch.empty(x.shape, dtype=x.dtype, device=x.device)
+        if x.shape[0]:
+            _ext().seq_selective_scan(out, x, dt_lin, dt_bias, Bm, Cm, a_log,
+                                      d_skip, z, state, cu_q, state_slot,
+                                      out_scale)
+        return out
+    return R.selective_scan(x, dt_lin, dt_bias, Bm, Cm, a_log, d_skip, z,
+                            state, cu_q, state_slot, out, out_scale)
 
 
 def rope_inv_freq(dims: int, base: float, device) -> torch.Tensor:
@@ -333,7 +407,8 @@ def gqa_prepare_store(q, k, v, q_norm, k_norm, eps: float, inv_freq,
                       v_inv_freq=None) -> torch.Tensor:
     """Queries and cache rows of grouped-query attention from a step's
     projections (column slices allowed).  Optional RMS norm over the WHOLE
-    query row and the whole key row (weights q_norm / k_norm), then
+    query row and the whole key row (weights q_norm / k_norm; weights of D
+    numbers norm every head on its own and are shared by the heads), then
     rotate-half RoPE on the first 2*len(inv_freq) entries of every head with
     angle fp32(position)*inv_freq and cos/sin scaled by ``amp``.  The cache
     row of a token, (pages, page_size, G*D + G*Dv) at slot_mapping[n], is
@@ -367,10 +442,13 @@ def gqa_window_attention(q, cache, page_table, seq_of_tok, positions, H: int,
                          q_temp_coef: float = 0.0,
                          q_temp_every: int = 1, softcap: float = 0.0,
                          head_bias=None, sigmoid_weights: bool = False,
-                         v_inv_freq=None) -> torch.Tensor:
+                         v_inv_freq=None, chunk: int = 0, out=None,
+                         out_scale: float = 1.0) -> torch.Tensor:
     """Attention of every row against its sequence's paged K/V rows
     (layout of :func:`gqa_prepare_store`).  Row at position p sees key j if
-    j <= p and (p - j < window or j < keep_first).  score = q.k * scale
+    j <= p and (p - j < window or j < keep_first); with ``chunk`` > 0 also
+    only keys of its own chunk, floor(j / chunk) = floor(p / chunk) (kept
+    first tokens apart).  score = q.k * scale
     * (1 + q_temp_coef * ln(floor((p + 1) / q_temp_every) + 1))
     [+ rel[dist_bucket[p - j], head]]; with ``sink`` (H,) fp32 the
     denominator also holds exp(sink[h]) once; ``gate`` (N, H) multiplies
@@ -381,10 +459,13 @@ def gqa_window_attention(q, cache, page_table, seq_of_tok, positions, H: int,
     sigmoid(score) instead of its softmax share (no normalisation over
     keys); ``v_inv_freq`` (Dv/2,) turns every head's sum back by the row's
     position (the inverse of the value rotation of
-    :func:`gqa_prepare_store`) before the gate.  Returns (N, H*Dv)."""
+    :func:`gqa_prepare_store`) before the gate.  Returns (N, H*Dv) in
+    ``out`` (a column slice is allowed) or a new tensor, times
+    ``out_scale``."""
     if q.is_cuda:
-        out = torch.empty(q.shape[0], H * Dv, dtype=out_dtype,
-                          device=q.device)
+        if out is None:
+            out = torch.empty(q.shape[0], H * Dv, dtype=out_dtype,
+                              device=q.device)
         if q.shape[0]:
             e = torch.Tensor()
             args = (cache, page_table, seq_of_tok, positions, H, G, D, Dv,
@@ -395,7 +476,8 @@ def gqa_window_attention(q, cache, page_table, seq_of_tok, positions, H: int,
                     q_temp_every, softcap,
                     head_bias if head_bias is not None else e,
                     sigmoid_weights,
-                    v_inv_freq if v_inv_freq is not None else e)
+                    v_inv_freq if v_inv_freq is not None else e, chunk,
+                    out_scale)
             if tiles is not None and tiles[2] == 0 and \
                     gqa_mfma_supported(q, D, Dv):
                 _ext().seq_gqa_window_attention_mfma(out, q, tiles[0],
@@ -407,7 +489,8 @@ def gqa_window_attention(q, cache, page_table, seq_of_tok, positions, H: int,
                                   H, G, D, Dv, window, keep_first, rel,
                                   dist_bucket, gate, scale, out_dtype, sink,
                                   q_temp_coef, q_temp_every, softcap,
-                                  head_bias, sigmoid_weights, v_inv_freq)
+                                  head_bias, sigmoid_weights, v_inv_freq,
+                                  chunk, out, out_scale)
 
 
 def gqa_mfma_supported(q, D: int, Dv: int) -> bool:

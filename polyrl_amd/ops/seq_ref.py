@@ -306,7 +306,13 @@ def gqa_prepare_store(q, k, v, q_norm, k_norm, eps, inv_freq, amp, positions,
     N = q.shape[0]
     qf, kf = q.float(), k.float()
     vf = kf if v is None else v.float()
-    if q_norm is not None:
+    if q_norm is not None and q_norm.numel() == D:      # per head
+        def unit(x, n, w):
+            x = x.reshape(N, n, D)
+            return (x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps)
+                    * w.float()).reshape(N, n * D)
+        qf, kf = unit(qf, H, q_norm), unit(kf, G, k_norm)
+    elif q_norm is not None:
         qf = qf * torch.rsqrt(qf.pow(2).mean(-1, keepdim=True) + eps) \
             * q_norm.float()
         kf = kf * torch.rsqrt(kf.pow(2).mean(-1, keepdim=True) + eps) \
@@ -336,7 +342,8 @@ def gqa_window_attention(q, cache, page_table, seq_of_tok, positions, H, G,
                          D, Dv, window, keep_first, rel, dist_bucket, gate,
                          scale, out_dtype, sink=None, q_temp_coef=0.0,
                          q_temp_every=1, softcap=0.0, head_bias=None,
-                         sigmoid_weights=False, v_inv_freq=None):
+                         sigmoid_weights=False, v_inv_freq=None, chunk=0,
+                         res=None, out_scale=1.0):
     N = q.shape[0]
     ps = cache.shape[1]
     flat = cache.view(-1, cache.shape[-1]).float()
@@ -346,6 +353,8 @@ def gqa_window_attention(q, cache, page_table, seq_of_tok, positions, H, G,
     per = H // G
     for n, (b, p) in enumerate(zip(seq_of_tok.tolist(), positions.tolist())):
         lo = max(0, p - window + 1)
+        if chunk > 0:
+            lo = max(lo, p // chunk * chunk)
         js = list(range(0, min(keep_first, lo))) + list(range(lo, p + 1))
         rows = torch.tensor([ptab[b][j // ps] * ps + j % ps for j in js],
                             dtype=torch.long)
@@ -378,7 +387,8 @@ def gqa_window_attention(q, cache, page_table, seq_of_tok, positions, H, G,
         if gate is not None:
             o = o * torch.sigmoid(gate[n].float()).unsqueeze(-1)
         out[n] = o
-    return out.view(N, H * Dv).to(out_dtype)
+    out = (out.view(N, H * Dv) * out_scale).to(out_dtype)
+    return out if res is None else res.copy_(out)
 
 
 def moe_route(logits, correction, top, groups, keep, act="softmax",
@@ -480,3 +490,68 @@ def rglru_scan(u, gates, gate_bias, lam, y_lin, state, cu_q, state_slot,
             out[n] = S * y[n]
         state[slot] = S
     return out.to(out_dtype)
+
+
+def add_unit_rms_then_cast(res, y, weight, eps, out_dtype, offset=0.0):
+    add_scaled_unit_rms(res, y, weight, eps, offset)
+    return res if out_dtype == torch.float32 else res.to(out_dtype)
+
+
+def softcap_f32(x, cap):
+    return cap * torch.tanh(x.float() / cap)
+
+
+def channel_delta_scan(q, k, v, b_lin, z_lin, dt_bias, a_log, gate, norm_w,
+                       state, cu_q, state_slot, key_eps, eps, out_dtype):
+    slots, H, Dk, Dv = state.shape
+    N = q.shape[0]
+    G = q.shape[1] // Dk
+    per = H // G
+
+    def unit(x):
+        x = x.float().reshape(N, G, Dk)
+        x = x * torch.rsqrt(x.pow(2).sum(-1, keepdim=True) + key_eps)
+        return x.repeat_interleave(per, dim=1)           # (N, H, Dk)
+    qf, kf = unit(q) * Dk ** -0.5, unit(k)
+    vf = v.float().reshape(N, H, Dv)
+    beta = torch.sigmoid(b_lin.float())
+    dec = torch.exp(-torch.exp(a_log.float()).view(1, H, 1)
+                    * torch.nn.functional.softplus(
+                        z_lin.float() + dt_bias.float(),
+                        threshold=1e9).view(N, H, Dk))
+    out = torch.empty(N, H, Dv, dtype=torch.float32, device=q.device)
+    cu = cu_q.tolist()
+    for b, slot in enumerate(state_slot.tolist()):
+        S = state[slot]                                  # (H, Dk, Dv)
+        for n in range(cu[b], cu[b + 1]):
+            S = dec[n].unsqueeze(-1) * S
+            u = beta[n].unsqueeze(-1) * (
+                vf[n] - torch.einsum("hk,hkv->hv", kf[n], S))
+            S = S + kf[n].unsqueeze(-1) * u.unsqueeze(1)
+            out[n] = torch.einsum("hk,hkv->hv", qf[n], S)
+        state[slot] = S
+    out = out * torch.rsqrt(out.pow(2).mean(-1, keepdim=True) + eps) \
+        * norm_w.float()
+    return (out.reshape(N, H * Dv) * torch.sigmoid(gate.float())) \
+        .to(out_dtype)
+
+
+def selective_scan(x, dt_lin, dt_bias, Bm, Cm, a_log, d_skip, z, state, cu_q,
+                   state_slot, res=None, out_scale=1.0):
+    xf = x.float()
+    dt = torch.nn.functional.softplus(dt_lin.float() + dt_bias.float(),
+                                      threshold=1e9)
+    A = -torch.exp(a_log.float())
+    Bf, Cf = Bm.float(), Cm.float()
+    y = torch.empty_like(xf)
+    cu = cu_q.tolist()
+    for b, slot in enumerate(state_slot.tolist()):
+        S = state[slot]                                  # (C, Ns)
+        for n in range(cu[b], cu[b + 1]):
+            S = torch.exp(dt[n].unsqueeze(-1) * A) * S \
+                + (dt[n] * xf[n]).unsqueeze(-1) * Bf[n]
+            y[n] = S @ Cf[n] + d_skip.float() * xf[n]
+        state[slot] = S
+    zf = z.float()
+    out = (y * zf * torch.sigmoid(zf) * out_scale).to(x.dtype)
+    return out if res is None else res.copy_(out)

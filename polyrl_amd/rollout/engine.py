@@ -475,9 +475,10 @@ class Engine:
         # pure decode steps of a model whose forward takes no decision on
         # the host replay one captured hipGraph per batch size instead of
         # issuing every launch from Python
+        cfg_style = self.model.cfg.layer_style
         self.enable_hybrid_graphs = (
-            str(dev) != "cpu" and (getattr(self.model, "prenorm", False)
-                                   or getattr(self.model, "parallel", False))
+            str(dev) != "cpu"
+            and cfg_style in ("prenorm", "parallel", "postnorm")
             and bool(int(__import__("os").environ.get(
                 "POLYRL_HIP_GRAPHS", "1"))))
         self._graph_seen: Dict[int, int] = {}

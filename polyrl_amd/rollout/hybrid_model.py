@@ -78,6 +78,11 @@ class _Part:
     ``tail_b`` and every forward leaves their result in ``tail_out``."""
     TAIL = False
     tail_w = tail_b = tail_out = None
+    key = ""              # prefix of its state names inside another mixer
+
+    def cache_row(self) -> Optional[int]:
+        """Numbers per paged cache row, None for a mixer without rows."""
+        return None
 
     def _with_tail(self, rows: int, tail: int, width, device, dtype,
                    bias: bool):
@@ -138,6 +143,175 @@ class DeltaRuleMixer(_Part):
                            states.tensors[(li, "S")], bt.cu_q, bt.state_slot,
                            s.decay_scale, s.key_eps, model.cfg.norm_eps,
                            h.dtype)
+        return _mm(y, self.wo)
+
+
+class ChannelDeltaMixer(_Part):
+    """Gated delta rule with per-channel decays (models.hybrid.
+    ChannelDeltaSpec): one fused projection for q, k, v, both low-rank
+    inputs and the write strength; one stateful convolution over the q, k
+    and v channels; one product for both low-rank outputs (block-diagonal:
+    decay rows read the decay input, gate rows the gate input); one kernel
+    for unit vectors, decays, the recurrence, the per-head norm and the
+    output gate.  State per sequence: one fp32 (dim, vdim) matrix per head
+    and the convolution's last taps-1 inputs."""
+
+    def __init__(self, spec, width, device, dtype):
+        self.spec = s = spec
+        self.nk, self.nv = s.kv_heads * s.dim, s.heads * s.vdim
+        self.nz = s.heads * s.dim
+        self.nc = 2 * self.nk + self.nv          # convolved channels
+        self.ra, self.rg = int(s.decay_rank), int(s.gate_rank)
+        z = lambda *a, dt=dtype: torch.empty(*a, device=device, dtype=dt)
+        f32 = torch.float32
+        self.w_in = z(self.nc + self.ra + self.rg + s.heads, width)
+        self.conv = z(self.nc, s.conv, dt=f32)
+        self.w_low = torch.zeros(self.nz + self.nv, self.ra + self.rg,
+                                 device=device, dtype=dtype)
+        self.dt_bias = z(self.nz, dt=f32)
+        self.a_log = z(s.heads, dt=f32)
+        self.norm = z(s.vdim, dt=f32)
+        self.wo = z(width, self.nv)
+
+    def named(self, p):
+        nk, nc, ra, nz = self.nk, self.nc, self.ra, self.nz
+        a = nc + ra + self.rg
+        out = {p + "a1": self.w_in[nc:nc + ra], p + "g1": self.w_in[nc + ra:a],
+               p + "b": self.w_in[a:], p + "a2": self.w_low[:nz, :ra],
+               p + "g2": self.w_low[nz:, ra:], p + "dt_bias": self.dt_bias,
+               p + "A_log": self.a_log, p + "norm": self.norm,
+               p + "o": self.wo}
+        for n, lo, hi in (("q", 0, nk), ("k", nk, 2 * nk), ("v", 2 * nk, nc)):
+            out[p + n] = self.w_in[lo:hi]
+            out[p + n + ".conv"] = self.conv[lo:hi]
+        return out
+
+    def state_shapes(self):
+        s = self.spec
+        out = {"S": (s.heads, s.dim, s.vdim)}
+        if s.conv > 1:
+            out["conv"] = (s.conv - 1, self.nc)
+        return out
+
+    def forward(self, h, bt, li, model, cache, states):
+        s, nk, nc = self.spec, self.nk, self.nc
+        proj = _mm(h, self.w_in)
+        qkv = seq.causal_conv_state(
+            proj.narrow(1, 0, nc), self.conv, None,
+            model._state(states, (li, "conv"), nc), bt.cu_q, bt.state_slot,
+            bt.seq_of_tok, False, True, h.dtype, max_rows=bt.max_q)
+        low = _mm(proj.narrow(1, nc, self.ra + self.rg), self.w_low)
+        y = seq.channel_delta_scan(
+            qkv.narrow(1, 0, nk), qkv.narrow(1, nk, nk),
+            qkv.narrow(1, 2 * nk, self.nv),
+            proj.narrow(1, nc + self.ra + self.rg, s.heads),
+            low.narrow(1, 0, self.nz), self.dt_bias, self.a_log,
+            low.narrow(1, self.nz, self.nv), self.norm,
+            states.tensors[(li, "S")], bt.cu_q, bt.state_slot, s.key_eps,
+            model.cfg.norm_eps, h.dtype)
+        return _mm(y, self.wo)
+
+
+class SelectiveScanMixer(_Part):
+    """Selective scan (models.hybrid.SelectiveScanSpec).  ``w_in`` / ``wo``
+    may be slices of another mixer's fused projections; ``mix`` takes the
+    input projection's rows and writes the scaled result before the output
+    projection."""
+
+    @staticmethod
+    def sizes(s):
+        """(rows of the input projection, columns of the output one)."""
+        return 2 * s.inner, s.inner
+
+    def __init__(self, spec, width, device, dtype, w_in=None, wo=None):
+        self.spec = s = spec
+        C, N, R = s.inner, s.state, s.dt_rank
+        z = lambda *a, dt=dtype: torch.empty(*a, device=device, dtype=dt)
+        f32 = torch.float32
+        self.w_in = w_in if w_in is not None else z(2 * C, width)
+        self.conv, self.conv_b = z(C, s.conv, dt=f32), z(C, dt=f32)
+        self.w_x, self.w_dt = z(R + 2 * N, C), z(C, R)
+        self.dt_b, self.d = z(C, dt=f32), z(C, dt=f32)
+        self.a_log = z(C, N, dt=f32)
+        self.wo = wo if wo is not None else z(width, C)
+
+    def named(self, p):
+        return {p + "in": self.w_in, p + "conv": self.conv,
+                p + "conv.b": self.conv_b, p + "x": self.w_x,
+                p + "dt": self.w_dt, p + "dt.b": self.dt_b,
+                p + "A_log": self.a_log, p + "D": self.d, p + "o": self.wo}
+
+    def state_shapes(self):
+        s = self.spec
+        out = {"S": (s.inner, s.state)}
+        if s.conv > 1:
+            out["conv"] = (s.conv - 1, s.inner)
+        return out
+
+    def mix(self, proj, bt, li, model, cache, states, out=None, scale=1.0):
+        s = self.spec
+        C, N, R = s.inner, s.state, s.dt_rank
+        x = seq.causal_conv_state(
+            proj.narrow(1, 0, C), self.conv, self.conv_b,
+            model._state(states, (li, self.key + "conv"), C), bt.cu_q,
+            bt.state_slot, bt.seq_of_tok, False, True, proj.dtype,
+            max_rows=bt.max_q)
+        dbc = _mm(x, self.w_x)
+        dt = _mm(dbc.narrow(1, 0, R), self.w_dt)
+        return seq.selective_scan(
+            x, dt, self.dt_b, dbc.narrow(1, R, N), dbc.narrow(1, R + N, N),
+            self.a_log, self.d, proj.narrow(1, C, C),
+            states.tensors[(li, self.key + "S")], bt.cu_q, bt.state_slot,
+            out=out, out_scale=scale)
+
+    def forward(self, h, bt, li, model, cache, states):
+        return _mm(self.mix(_mm(h, self.w_in), bt, li, model, cache, states),
+                   self.wo)
+
+
+class ParallelMixer(_Part):
+    """Two mixers side by side (models.hybrid.ParallelMixerSpec): one fused
+    input projection, and one output product over both results, which the
+    mixers' last kernels write next to each other already multiplied by
+    their scales."""
+
+    def __init__(self, spec, width, device, dtype):
+        self.spec = s = spec
+        cl, cr = _MIXERS[s.left.kind], _MIXERS[s.right.kind]
+        (self.rl, self.cl), (self.rr, self.cr) = cl.sizes(s.left), \
+            cr.sizes(s.right)
+        self.w_in = torch.empty(self.rl + self.rr, width, device=device,
+                                dtype=dtype)
+        self.wo = torch.empty(width, self.cl + self.cr, device=device,
+                              dtype=dtype)
+        self.left = cl(s.left, width, device, dtype, w_in=self.w_in[:self.rl],
+                       wo=self.wo[:, :self.cl])
+        self.right = cr(s.right, width, device, dtype,
+                        w_in=self.w_in[self.rl:], wo=self.wo[:, self.cl:])
+        self.left.key, self.right.key = "left.", "right."
+
+    def named(self, p):
+        return {**self.left.named(p + "left."),
+                **self.right.named(p + "right.")}
+
+    def cache_row(self):
+        rows = [m.cache_row() for m in (self.left, self.right)]
+        assert None in rows, "one paged mixer per layer"
+        return rows[0] if rows[1] is None else rows[1]
+
+    def state_shapes(self):
+        return {m.key + k: v for m in (self.left, self.right)
+                for k, v in m.state_shapes().items()}
+
+    def forward(self, h, bt, li, model, cache, states):
+        proj = _mm(h, self.w_in)
+        y = torch.empty(h.shape[0], self.cl + self.cr, device=h.device,
+                        dtype=h.dtype)
+        self.left.mix(proj.narrow(1, 0, self.rl), bt, li, model, cache,
+                      states, y.narrow(1, 0, self.cl), self.spec.left_scale)
+        self.right.mix(proj.narrow(1, self.rl, self.rr), bt, li, model, cache,
+                       states, y.narrow(1, self.cl, self.cr),
+                       self.spec.right_scale)
         return _mm(y, self.wo)
 
 
@@ -330,6 +504,9 @@ class LatentAttnMixer(_Part):
             self.inv_freq = seq.rope_inv_freq(s.rope_dims, s.rope_base,
                                               device)
 
+    def cache_row(self):
+        return self.row if self.owner else None
+
     def named(self, p):
         a, b = self.n0, self.n0 + self.ng
         out = {p + "g": self.w_in[a:b],
@@ -444,11 +621,21 @@ class LatentAttnMixer(_Part):
 class WindowAttnMixer(_Part):
     """Grouped-query attention over a sliding window of paged K/V rows
     (models.hybrid.WindowAttnSpec): one fused projection for queries, keys,
-    values (unless the keys serve as values) and the per-head gate; one
-    kernel norms, rotates and writes the cache rows; one attends."""
+    values (unless the keys serve as values) and the per-head gate; an
+    optional stateful convolution over the query, key and value channels;
+    one kernel norms, rotates and writes the cache rows; one attends.
+    ``w_in`` / ``wo`` may be slices of another mixer's fused projections."""
     TAIL = True
 
-    def __init__(self, spec, width, device, dtype, tail=0):
+    @staticmethod
+    def sizes(s):
+        """(rows of the input projection, columns of the output one)."""
+        return ((s.heads + s.kv_heads) * s.dim
+                + (0 if s.values_from_keys else s.kv_heads * s.vdim)
+                + (s.heads if s.head_gate else 0)), s.heads * s.vdim
+
+    def __init__(self, spec, width, device, dtype, tail=0, w_in=None,
+                 wo=None):
         self.spec = s = spec
         z = lambda *a, dt=dtype: torch.empty(*a, device=device, dtype=dt)
         f32 = torch.float32
@@ -457,17 +644,23 @@ class WindowAttnMixer(_Part):
         self.ng = s.heads if s.head_gate else 0
         self.row = s.kv_heads * (s.dim + s.vdim)
         # (the head gate has no bias: its entries stay zero)
-        self.w_in, self.b_in = self._with_tail(
-            self.nq + self.nk + self.nv + self.ng, tail, width, device, dtype,
-            s.qkv_bias)
+        self.w_in, self.b_in = (w_in, None) if w_in is not None else \
+            self._with_tail(self.nq + self.nk + self.nv + self.ng, tail,
+                            width, device, dtype, s.qkv_bias)
         self.sink = z(s.heads, dt=f32) if s.sink else None
+        self.unit_sink = torch.zeros(s.heads, device=device, dtype=f32) \
+            if s.unit_sink else None
+        self.nc = self.nq + self.nk + self.nv
+        self.conv = z(self.nc, s.conv, dt=f32) if s.conv else None
         self.head_bias = z(s.heads, dt=f32) if s.head_bias else None
         self.v_inv_freq = seq.rope_inv_freq(s.vdim, s.value_rope_base,
                                             device) \
             if s.value_rope_base > 0 else None
-        self.q_norm = z(self.nq, dt=f32) if s.qk_norm else None
-        self.k_norm = z(self.nk, dt=f32) if s.qk_norm else None
-        self.wo = z(width, s.heads * s.vdim)
+        nqn, nkn = (s.dim, s.dim) if s.head_norm else (self.nq, self.nk)
+        normed = s.qk_norm or s.head_norm
+        self.q_norm = z(nqn, dt=f32) if normed else None
+        self.k_norm = z(nkn, dt=f32) if normed else None
+        self.wo = wo if wo is not None else z(width, s.heads * s.vdim)
         self.inv_freq, self.amp = None, 1.0
         if s.rope is not None:
             f, self.amp = s.rope.inv_freq_and_amp()
@@ -502,13 +695,34 @@ class WindowAttnMixer(_Part):
             out[p + "sink"] = self.sink
         if self.head_bias is not None:
             out[p + "pb"] = self.head_bias
+        if self.conv is not None:
+            out[p + "q.conv"], out[p + "k.conv"] = self.conv[:a], \
+                self.conv[a:b]
+            if self.nv:
+                out[p + "v.conv"] = self.conv[b:]
         return out
 
-    def forward(self, h, bt, li, model, cache, states):
+    def cache_row(self):
+        return self.row
+
+    def state_shapes(self):
         s = self.spec
-        a, b = self.nq, self.nq + self.nk
+        return {"conv": (s.conv - 1, self.nc)} if s.conv > 1 else {}
+
+    def forward(self, h, bt, li, model, cache, states):
         proj = _mm(h, self.w_in, self.b_in)
         self._split_tail(proj)
+        return _mm(self.mix(proj, bt, li, model, cache, states), self.wo)
+
+    def mix(self, proj, bt, li, model, cache, states, out=None, scale=1.0):
+        s = self.spec
+        a, b = self.nq, self.nq + self.nk
+        if self.conv is not None:
+            proj = seq.causal_conv_state(
+                proj.narrow(1, 0, self.nc), self.conv, None,
+                model._state(states, (li, self.key + "conv"), self.nc),
+                bt.cu_q, bt.state_slot, bt.seq_of_tok, False, False,
+                proj.dtype, max_rows=bt.max_q)
         rows = cache.rows[li]
         q = seq.gqa_prepare_store(
             proj.narrow(1, 0, a), proj.narrow(1, a, self.nk),
@@ -517,17 +731,18 @@ class WindowAttnMixer(_Part):
             self.amp, bt.positions, rows, bt.slot_mapping, s.heads,
             s.kv_heads, s.dim, s.vdim, head_unit=s.head_unit_norm,
             v_inv_freq=self.v_inv_freq)
-        o = seq.gqa_window_attention(
+        return seq.gqa_window_attention(
             q, rows, bt.page_table, bt.seq_of_tok, bt.positions, s.heads,
             s.kv_heads, s.dim, s.vdim, s.window, s.keep_first, self.rel,
             self.dist_bucket,
             proj.narrow(1, b + self.nv, self.ng) if self.ng else None,
-            s.scale, h.dtype, tiles=bt.attn_tiles, sink=self.sink,
+            s.scale, proj.dtype, tiles=bt.attn_tiles,
+            sink=self.sink if self.sink is not None else self.unit_sink,
             q_temp_coef=s.q_temp_coef, q_temp_every=s.q_temp_every,
             softcap=s.softcap, head_bias=self.head_bias,
             sigmoid_weights=s.weights == "sigmoid",
-            v_inv_freq=self.v_inv_freq)
-        return _mm(o, self.wo)
+            v_inv_freq=self.v_inv_freq, chunk=s.chunk, out=out,
+            out_scale=scale)
 
 
 class DenseFF(_Part):
@@ -728,6 +943,8 @@ class RoutedMoE(_Part):
 
 _MIXERS = {"general_delta": DeltaRuleMixer, "mamba2": SSMMixer,
            "gla": GLAMixer, "rglru": RGLRUMixer,
+           "channel_delta": ChannelDeltaMixer, "mamba": SelectiveScanMixer,
+           "parallel": ParallelMixer,
            "latent_attention": LatentAttnMixer, "attention": WindowAttnMixer}
 _FFS = {"dense": DenseFF, "moe": TableMoE, "routed_moe": RoutedMoE}
 
@@ -782,6 +999,30 @@ class SandwichLayer:
         if self.ff is not None:
             out[p + "norm2"] = self.norm2
             out[p + "norm2b"] = self.norm2b
+            out.update(self.ff.named(p + "mlp."))
+        return out
+
+
+class PostNormLayer:
+    """x += norm1(mixer(x)), x += norm2(ff(x)): one per-channel norm weight
+    per sublayer, on its output, stored as an offset from
+    ``cfg.norm_offset``."""
+
+    def __init__(self, cfg: HybridConfig, li: int, device, dtype):
+        L = cfg.layers[li]
+        W = cfg.hidden_size
+        z = lambda: torch.empty(W, device=device, dtype=torch.float32)
+        self.norm1 = z()
+        self.mixer = _MIXERS[L.mixer.kind](L.mixer, W, device, dtype)
+        self.ff = None if L.ff is None else \
+            _FFS[L.ff.kind](L.ff, W, cfg.vocab_size, device, dtype)
+        self.norm2 = z() if self.ff is not None else None
+
+    def named(self, p: str) -> Dict[str, torch.Tensor]:
+        out = {p + "norm1": self.norm1}
+        out.update(self.mixer.named(p + "mix."))
+        if self.ff is not None:
+            out[p + "norm2"] = self.norm2
             out.update(self.ff.named(p + "mlp."))
         return out
 
@@ -879,14 +1120,20 @@ class HybridInferenceModel:
                     and L.mixer.bias_rows is None:
                 raise ValueError("the distance-bias table's rows come from "
                                  "the checkpoint: call resolve_shapes first")
+            if L.mixer.kind == "channel_delta" and \
+                    None in (L.mixer.decay_rank, L.mixer.gate_rank):
+                raise ValueError("the low-rank projections' ranks come from "
+                                 "the checkpoint: call resolve_shapes first")
             if L.mixer.kind == "gla" and L.mixer.decay_rank is None:
                 raise ValueError("the decay projection's rank comes from "
                                  "the checkpoint: call resolve_shapes first")
         self.sandwich = cfg.layer_style == "sandwich"
         self.prenorm = cfg.layer_style == "prenorm"
         self.parallel = cfg.layer_style == "parallel"
+        self.postnorm = cfg.layer_style == "postnorm"
         layer_cls = SandwichLayer if self.sandwich else \
             PreNormLayer if self.prenorm else \
+            PostNormLayer if self.postnorm else \
             ParallelLayer if self.parallel else HybridLayer
         self.layers = [layer_cls(cfg, li, device, dtype)
                        for li in range(cfg.num_hidden_layers)]
@@ -897,7 +1144,7 @@ class HybridInferenceModel:
             cfg.vocab_size, cfg.num_hidden_layers * cfg.token_side_dim,
             device=device, dtype=dtype)
         self.final_norm = torch.empty(
-            W if self.sandwich or self.prenorm or self.parallel else 1,
+            1 if cfg.layer_style == "canon" else W,
             device=device, dtype=torch.float32)
         self.lm_head = torch.empty(cfg.vocab_size, W, device=device,
                                    dtype=dtype)
@@ -932,10 +1179,14 @@ class HybridInferenceModel:
                 shp = shapes.get(f"l{li}.mix.w1")
                 if shp is not None:
                     L.mixer.decay_rank = int(shp[0])
-            if L.mixer.kind == "gla":
+            if L.mixer.kind in ("gla", "channel_delta"):
                 shp = shapes.get(f"l{li}.mix.a1")
                 if shp is not None:
                     L.mixer.decay_rank = int(shp[0])
+            if L.mixer.kind == "channel_delta":
+                shp = shapes.get(f"l{li}.mix.g1")
+                if shp is not None:
+                    L.mixer.gate_rank = int(shp[0])
             if L.mixer.kind == "attention" and L.mixer.bias_far > 0:
                 shp = shapes.get(f"l{li}.mix.rel")
                 if shp is not None:
@@ -945,16 +1196,16 @@ class HybridInferenceModel:
     def graph_safe_decode(self, B: int) -> bool:
         """Whether a decode step of B single tokens runs without a decision
         on the host (so it can be captured in a graph): pre-norm stacks
-        always; parallel stacks when every routed feed-forward takes the
+        always; post-norm and parallel stacks when every routed feed-forward takes the
         fused expert kernels (bf16, sizes in multiples of 32, a batch the
         kernels' slot list holds)."""
         if self.prenorm:
             return True
-        if not self.parallel:
+        if not self.parallel and not self.postnorm:
             return False
         for L in self.layers:
             f = L.ff
-            if f is None:
+            if f is None or isinstance(f, DenseFF):
                 continue
             if not isinstance(f, RoutedMoE) or f.E == 0 or \
                     self.dtype != torch.bfloat16 or B > 256 or \
@@ -968,10 +1219,9 @@ class HybridInferenceModel:
         layer owns one set of rows per pass)."""
         out = {}
         for ri, li in enumerate(self.runs):
-            m = self.layers[li].mixer
-            if isinstance(m, WindowAttnMixer) or \
-                    (isinstance(m, LatentAttnMixer) and m.owner):
-                out[ri] = m.row
+            row = self.layers[li].mixer.cache_row()
+            if row is not None:
+                out[ri] = row
         return out
 
     def state_shapes(self) -> Dict[tuple, tuple]:
@@ -1056,19 +1306,21 @@ class HybridInferenceModel:
                 buf.copy_(torch.randn(buf.shape, generator=g) * 0.2)
             elif name.endswith("mix.pb"):
                 buf.copy_(torch.randn(buf.shape, generator=g) * 0.5 - 4.0)
-            elif self.sandwich and name.endswith(
+            elif (self.sandwich or self.postnorm) and name.endswith(
                     ("norm1", "norm2", "norm1b", "norm2b", "final.norm")):
                 buf.copy_(torch.randn(buf.shape, generator=g) * 0.1)
             elif name.endswith(("mix.rel", "mlp.correction")):
                 buf.copy_(torch.randn(buf.shape, generator=g) *
                           (0.5 if name.endswith("rel") else 0.02))
+            elif self.postnorm and name.endswith(("dt_bias", "dt.b")):
+                buf.copy_(torch.randn(buf.shape, generator=g) - 2.0)
             elif name.endswith(("norm1", "norm2", "final.norm", ".norm",
-                                "mix.D")):
+                                "mix.D", "right.D")):
                 buf.fill_(1.0)
             elif name.endswith(("A_log", "dt_bias", "w0", "a.b", "sink",
                                 "conv.b")):
                 buf.copy_(torch.randn(buf.shape, generator=g) * 0.5)
-            elif name.endswith(("canon1", "mix.conv")):
+            elif name.endswith(("canon1", ".conv")):
                 buf.copy_(torch.randn(buf.shape, generator=g) * 0.3)
             elif name == "embed" and self.cfg.embed_scale != 1.0:
                 buf.copy_(torch.randn(buf.shape, generator=g)
@@ -1105,6 +1357,8 @@ class HybridInferenceModel:
             return self._forward_prenorm(bt, cache, states)
         if self.parallel:
             return self._forward_parallel(bt, cache, states)
+        if self.postnorm:
+            return self._forward_postnorm(bt, cache, states)
         cfg, dt = self.cfg, self.dtype
         eps = cfg.norm_eps
         res = self.embed[bt.tokens].float()
@@ -1159,6 +1413,25 @@ class HybridInferenceModel:
                                                off)
             else:
                 seq.add_scaled_unit_rms(res, y, post, eps, off)
+            if self.capture_layers is not None:
+                self.capture_layers.append(res.clone())
+        return res
+
+    def _forward_postnorm(self, bt: HybridBatch, cache, states):
+        """Layer runs of the post-norm style: a sublayer reads the stream
+        itself (in the engine dtype); one fused pass adds its normed output
+        to the fp32 stream and writes the next sublayer's input."""
+        cfg, dt = self.cfg, self.dtype
+        eps, off = cfg.norm_eps, cfg.norm_offset
+        h = self.embed[bt.tokens]
+        res = h.float()
+        for ri, li in enumerate(self.runs):
+            L = self.layers[li]
+            y = L.mixer.forward(h, bt, ri, self, cache, states)
+            h = seq.add_unit_rms_then_cast(res, y, L.norm1, eps, dt, off)
+            if L.ff is not None:
+                y = L.ff.forward(h, res, bt)
+                h = seq.add_unit_rms_then_cast(res, y, L.norm2, eps, dt, off)
             if self.capture_layers is not None:
                 self.capture_layers.append(res.clone())
         return res
@@ -1282,7 +1555,11 @@ class HybridInferenceModel:
             h = seq.add_rmsnorm_f32res(res_rows.contiguous(), None,
                                        self.final_norm, self.cfg.norm_eps,
                                        self.dtype, self.cfg.norm_offset)
-        out = _mm(h, self.lm_head).float()
+        out = _mm(h, self.lm_head)
+        if self.cfg.logit_softcap > 0:
+            assert self.cfg.logit_scale == 1.0
+            return seq.softcap_f32(out, self.cfg.logit_softcap)
+        out = out.float()
         if self.cfg.logit_scale != 1.0:
             out = out * self.cfg.logit_scale
         return out
