@@ -115,6 +115,18 @@ def _hybrid_presets():
             width=64, layers=3, vocab=300, heads=4, kv_heads=2, ff=96,
             chunk=24, inner=80, state=8,
             pattern=("channel_delta", "parallel", "channel_delta")),
+        # bench pairs: beside vurivik-400m / -1b / -8b-l8 (equal width, depth,
+        # heads and vocabulary; the feed-forward is set so that the parameter
+        # totals agree within 1 %)
+        "puvapel-400m": lambda: puvapel_preset(
+            width=1024, layers=12, vocab=32000, heads=16, kv_heads=4,
+            ff=4672, chunk=512),
+        "puvapel-1b": lambda: puvapel_preset(
+            width=2048, layers=16, vocab=128256, heads=32, kv_heads=8,
+            ff=9088, chunk=1024),
+        "puvapel-8b-l8": lambda: puvapel_preset(
+            width=4096, layers=8, vocab=128256, heads=32, kv_heads=8,
+            ff=13952, chunk=2048),
         # tiny stack for CPU unit tests / fast GPU smoke
         "nasipel-debug": lambda: nasipel_preset(
             width=64, layers=4, vocab=300, heads=4, kv_heads=2, experts=6,

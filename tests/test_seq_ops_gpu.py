@@ -744,3 +744,174 @@ def test_gated_routed_experts_bf16(N, top, E):
     got = seq.moe_weighted_combine(ys1, idx.to(DEV), w.to(DEV), h.to(DEV),
                                    None, E, 1e-20, dt, 1.75)
     torch.testing.assert_close(got.cpu().float(), want.float(), **tol(dt))
+
+
+@pytest.mark.parametrize("dt", DTYPES)
+@pytest.mark.parametrize("taps", [1, 2, 3, 4])
+@pytest.mark.parametrize("lens", [[5, 1, 2, 9], [1, 1, 1, 1], [900, 3, 200],
+                                  [5000, 1, 2, 3300]])
+def test_causal_conv_in_runs_of_rows(dt, taps, lens):
+    """Channel counts in multiples of four: a thread walks several packed
+    rows across sequence borders; single-token steps update the history in
+    the same launch."""
+    C, slots = 52, [3, 0, 5, 1][:len(lens)]
+    bt = batch(lens, slots)
+    big = rnd(sum(lens), C + 12, dt=dt)
+    w, bias = rnd(C, taps, scale=0.5), rnd(C)
+    st0 = rnd(6, taps - 1, C)
+    for silu, b, add in ((True, bias, False), (False, None, True)):
+        sc, sg = st0.clone(), st0.clone().to(DEV)
+        want = R.causal_conv_state(big[:, 8:8 + C], w, b, sc, *bt["cpu"],
+                                   add, silu, dt)
+        got = seq.causal_conv_state(
+            big.to(DEV)[:, 8:8 + C], w.to(DEV),
+            None if b is None else b.to(DEV), sg, *bt[DEV], add, silu, dt,
+            max_rows=max(lens))
+        torch.testing.assert_close(got.cpu().float(), want.float(), **tol(dt))
+        torch.testing.assert_close(sg.cpu(), sc, rtol=0, atol=0)
+
+
+@pytest.mark.parametrize("dt", DTYPES)
+@pytest.mark.parametrize("D", [36, 130, 1030, 1500, 4096, 6000, 9000, 9002])
+def test_postnorm_join(dt, D):
+    res, y, w = rnd(5, D), rnd(5, D, dt=dt, scale=3.0), rnd(D, scale=0.3)
+    r0, r1 = res.clone(), res.clone().to(DEV)
+    want = R.add_unit_rms_then_cast(r0, y, w, 1e-5, dt, 1.0)
+    got = seq.add_unit_rms_then_cast(r1, y.to(DEV), w.to(DEV), 1e-5, dt, 1.0)
+    torch.testing.assert_close(r1.cpu(), r0, rtol=1e-5, atol=1e-5)
+    torch.testing.assert_close(got.cpu().float(), want.float(), **tol(dt))
+    assert (got.data_ptr() == r1.data_ptr()) == (dt == torch.float32)
+
+
+@pytest.mark.parametrize("dt", DTYPES)
+def test_softcap_logits(dt):
+    x = rnd(3, 301, dt=dt, scale=40.0)
+    got = seq.softcap_f32(x.to(DEV), 15.0)
+    assert got.dtype == torch.float32
+    torch.testing.assert_close(got.cpu(), R.softcap_f32(x, 15.0), rtol=1e-5,
+                               atol=1e-5)
+
+
+@pytest.mark.parametrize("dt", DTYPES)
+@pytest.mark.parametrize("H,G,Dk,Dv,lens", [
+    (4, 2, 12, 8, [5, 1, 40]), (1, 1, 3, 5, [2, 33]), (3, 1, 33, 64, [65, 1]),
+    (2, 2, 64, 64, [1, 1, 1]), (2, 2, 64, 64, [31, 32, 33, 100]),
+    (2, 1, 64, 128, [70, 3]), (1, 1, 128, 128, [50, 1]),
+    (2, 1, 20, 150, [9, 40]), (1, 1, 200, 24, [30]), (1, 1, 256, 70, [20]),
+    (1, 1, 300, 40, [21, 1]), (2, 2, 512, 64, [11])])
+def test_channel_delta_scan(dt, H, G, Dk, Dv, lens):
+    """Unit vectors, decays, recurrence, per-head norm and gate, with
+    inputs as column slices and states in shuffled slots."""
+    slots = [3, 0, 5, 1][:len(lens)]
+    bt = batch(lens, slots)
+    N = sum(lens)
+    nk, nv, nz = G * Dk, H * Dv, H * Dk
+    p = rnd(N, 2 * nk + nv + H + 5, dt=dt)
+    low = rnd(N, nz + nv, dt=dt)
+    dtb, alog, nw = rnd(nz) - 3.0, rnd(H) * 0.5, rnd(Dv).abs() + 0.5
+    st = rnd(6, H, Dk, Dv, scale=0.3)
+
+    def go(mod, d, s):
+        x, lo = p.to(d), low.to(d)
+        c, sl, _ = bt[d]
+        return mod.channel_delta_scan(
+            x[:, :nk], x[:, nk:2 * nk], x[:, 2 * nk:2 * nk + nv],
+            x[:, 2 * nk + nv:2 * nk + nv + H], lo[:, :nz], dtb.to(d),
+            alog.to(d), lo[:, nz:], nw.to(d), s, c, sl, 1e-6, 1e-5, dt)
+    s0, s1 = st.clone(), st.clone().to(DEV)
+    want, got = go(R, "cpu", s0), go(seq, DEV, s1)
+    torch.testing.assert_close(s1.cpu(), s0, rtol=1e-4, atol=1e-5)
+    torch.testing.assert_close(
+        got.cpu().float(), want.float(),
+        **(tol(dt) if dt == torch.bfloat16 else dict(rtol=2e-4, atol=2e-5)))
+
+
+@pytest.mark.parametrize("dt", DTYPES)
+@pytest.mark.parametrize("C,Ns,R_,lens", [
+    (20, 6, 3, [5, 1, 40]), (64, 16, 4, [33, 1, 70]), (13, 5, 1, [9, 3]),
+    (130, 20, 7, [1, 1, 1]), (256, 32, 16, [64, 31]), (72, 70, 4, [20]),
+    (1, 150, 1, [7, 2]), (68, 256, 4, [40, 1])])
+def test_selective_scan(dt, C, Ns, R_, lens):
+    slots = [3, 0, 5, 1][:len(lens)]
+    bt = batch(lens, slots)
+    N = sum(lens)
+    x, dtl = rnd(N, C, dt=dt), rnd(N, C, dt=dt)
+    dbc, zz = rnd(N, R_ + 2 * Ns, dt=dt), rnd(N, 2 * C, dt=dt)
+    dtb, alog, ds = rnd(C) - 2.0, rnd(C, Ns) * 0.7, rnd(C)
+    st = rnd(6, C, Ns)
+    out = torch.zeros(N, C + 24, dtype=dt, device=DEV)
+
+    def go(mod, d, s, **kw):
+        c, sl, _ = bt[d]
+        b = dbc.to(d)
+        return mod.selective_scan(x.to(d), dtl.to(d), dtb.to(d),
+                                  b[:, R_:R_ + Ns], b[:, R_ + Ns:],
+                                  alog.to(d), ds.to(d), zz.to(d)[:, C:], s,
+                                  c, sl, out_scale=0.7, **kw)
+    s0, s1 = st.clone(), st.clone().to(DEV)
+    want = go(R, "cpu", s0)
+    got = go(seq, DEV, s1, out=out[:, 12:12 + C])
+    torch.testing.assert_close(s1.cpu(), s0, rtol=1e-4, atol=1e-5)
+    torch.testing.assert_close(
+        got.cpu().float(), want.float(),
+        **(tol(dt) if dt == torch.bfloat16 else dict(rtol=2e-4, atol=2e-4)))
+    assert not out[:, :12].any() and not out[:, 12 + C:].any()
+
+
+@pytest.mark.parametrize("dt", DTYPES)
+@pytest.mark.parametrize("H,G,D,Dv,half,chunk,lens,starts", [
+    (4, 2, 16, 24, 4, 8, [5, 1, 30], [0, 37, 6]),
+    (4, 4, 64, 64, 16, 50, [70, 1, 130], [3, 300, 40]),
+    (6, 2, 24, 16, 0, 1, [20, 3], [5, 0]),
+    (3, 3, 10, 6, 5, 7, [6, 2, 90], [0, 9, 33]),
+    (2, 1, 136, 72, 68, 33, [40, 1], [10, 65]),
+    (8, 1, 64, 128, 32, 96, [200, 64, 1], [0, 96, 191]),
+    (8, 2, 32, 80, 16, 20, [1, 1, 1], [0, 19, 200]),
+])
+def test_chunked_attention_with_head_norms(dt, H, G, D, Dv, half, chunk, lens,
+                                           starts):
+    """Writer: per-head RMS norms with shared weights before the rotation.
+    Attention: keys of the row's own chunk only, a sink of score zero,
+    capped scores, scaled result in a column slice; one wave per row and
+    the matrix-core kernel."""
+    page = 4
+    cache, ptab, pos, sot, slot = _paged(lens, starts, page, G * (D + Dv), dt)
+    all_lens = [s + n for s, n in zip(starts, lens)]
+    pos2 = torch.tensor([p for n in all_lens for p in range(n)],
+                        dtype=torch.int32)
+    slot2 = torch.tensor([int(ptab[b, p // page]) * page + p % page
+                          for b, n in enumerate(all_lens) for p in range(n)],
+                         dtype=torch.int32)
+    N2 = sum(all_lens)
+    inv = torch.rand(half) if half else None
+    kv = rnd(N2, G * D + G * Dv + H * D, dt=dt)
+    qn, kn = rnd(D).abs() + 0.5, rnd(D).abs() + 0.5
+    c0, c1 = cache.clone(), cache.clone().to(DEV)
+    g = lambda t: None if t is None else t.to(DEV)
+    a, b = G * D, G * D + G * Dv
+    q0 = R.gqa_prepare_store(kv[:, b:], kv[:, :a], kv[:, a:b], qn, kn, 1e-5,
+                             inv, 1.0, pos2, c0, slot2, H, G, D, Dv)
+    kd = kv.to(DEV)
+    q1 = seq.gqa_prepare_store(kd[:, b:], kd[:, :a], kd[:, a:b], g(qn), g(kn),
+                               1e-5, g(inv), 1.0, g(pos2), c1, g(slot2), H, G,
+                               D, Dv)
+    torch.testing.assert_close(q1.cpu().float(), q0.float(), **tol(dt))
+    torch.testing.assert_close(c1.cpu().float(), c0.float(), **tol(dt))
+    rows = torch.cat([torch.arange(s, s + n) + sum(all_lens[:i])
+                      for i, (s, n) in enumerate(zip(starts, lens))])
+    q = q0[rows].contiguous()
+    scale, cap, sink = 2.0 / math.sqrt(D), 6.0, torch.zeros(H)
+    want = R.gqa_window_attention(
+        q, c0, ptab, sot, pos, H, G, D, Dv, 1 << 30, 0, None, None, None,
+        scale, dt, sink=sink, softcap=cap, chunk=chunk, out_scale=0.6)
+    for tl in (None, seq.attention_tiles(lens, DEV)):
+        out = torch.zeros(len(rows), H * Dv + 16, dtype=dt, device=DEV)
+        got = seq.gqa_window_attention(
+            g(q), g(c0), g(ptab), g(sot), g(pos), H, G, D, Dv, 1 << 30, 0,
+            None, None, None, scale, dt, tiles=tl, sink=g(sink), softcap=cap,
+            chunk=chunk, out=out[:, 8:8 + H * Dv], out_scale=0.6)
+        ref = want.float()
+        lim = dict(rtol=2e-2, atol=2e-2 * float(ref.abs().max())) \
+            if dt == torch.bfloat16 else dict(rtol=1e-4, atol=1e-4)
+        torch.testing.assert_close(got.cpu().float(), ref, **lim)
+        assert not out[:, :8].any() and not out[:, 8 + H * Dv:].any()
