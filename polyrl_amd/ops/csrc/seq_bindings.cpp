@@ -30,14 +30,14 @@ void seq_channel_delta(torch::Tensor out, torch::Tensor q, torch::Tensor k,
                        torch::Tensor a_log, torch::Tensor gate,
                        torch::Tensor norm_w, torch::Tensor state,
                        torch::Tensor cu_q, torch::Tensor state_slot,
-                       double key_eps, double eps);
+                       double key_eps, double eps, int64_t max_rows);
 void seq_selective_scan(torch::Tensor out, torch::Tensor x,
                         torch::Tensor dt_lin, torch::Tensor dt_bias,
                         torch::Tensor Bm, torch::Tensor Cm,
                         torch::Tensor a_log, torch::Tensor d_skip,
                         torch::Tensor z, torch::Tensor state,
                         torch::Tensor cu_q, torch::Tensor state_slot,
-                        double out_scale);
+                        double out_scale, int64_t max_rows);
 void seq_group_rmsnorm(torch::Tensor out, torch::Tensor y,
                        torch::Tensor weight, int64_t groups, double eps,
                        torch::Tensor gate, int64_t gate_act);

@@ -24,6 +24,28 @@ DEV_INLINE float siluf_acc(float x) { return x / (1.f + expf(-x)); }
 DEV_INLINE float softplusf_acc(float x) {
   return fmaxf(x, 0.f) + log1pf(expf(-fabsf(x)));
 }
+// The same through the hardware exponential and reciprocal (each good to an
+// ulp), for kernels whose lanes spend most of their time in them.
+DEV_INLINE float sigmoidf_fast(float x) {
+  return __builtin_amdgcn_rcpf(
+      1.f + __builtin_amdgcn_exp2f(-1.4426950408889634f * x));
+}
+// log(1 + e) for e = exp(-|x|) in [0, 1] as 2 atanh(s), s = e / (2 + e) <=
+// 1/3, by the odd power series of atanh: relative error below 3e-7 for every
+// e, also where 1 + e rounds to one
+DEV_INLINE float softplusf_fast(float x) {
+  const float e = __builtin_amdgcn_exp2f(-1.4426950408889634f * fabsf(x));
+  const float s = e * __builtin_amdgcn_rcpf(2.f + e);
+  const float w = s * s;
+  float p = 1.f / 13.f;
+  p = p * w + 1.f / 11.f;
+  p = p * w + 1.f / 9.f;
+  p = p * w + 1.f / 7.f;
+  p = p * w + 1.f / 5.f;
+  p = p * w + 1.f / 3.f;
+  p = p * w + 1.f;
+  return fmaxf(x, 0.f) + 2.f * s * p;
+}
 DEV_INLINE float gelu_tanhf_acc(float z) {
   const float c = 0.7978845608028654f;  // sqrt(2/pi)
   return 0.5f * z * (1.f + tanhf(c * (z + 0.044715f * z * z * z)));
@@ -58,6 +80,51 @@ DEV_INLINE float oct_sum(float x) {
       0, __builtin_bit_cast(int, x), 0x141, 0xF, 0xF, false));
   return x;
 }
+
+// Four consecutive activations as they lie in memory: fetched ahead of their
+// use, turned into fp32 where they are used (a conversion next to the load
+// would wait for it there).
+template <typename T>
+struct Raw4;
+template <>
+struct Raw4<bf16_t> {
+  uint2 r;
+  template <bool VEC>
+  DEV_INLINE void load(const bf16_t* p, int valid) {
+    if (VEC) {
+      r = *reinterpret_cast<const uint2*>(p);
+    } else {
+      unsigned short h[4];
+#pragma unroll
+      for (int e = 0; e < 4; ++e)
+        h[e] = e < valid ? reinterpret_cast<const unsigned short*>(p)[e] : 0;
+      r.x = h[0] | (unsigned)h[1] << 16;
+      r.y = h[2] | (unsigned)h[3] << 16;
+    }
+  }
+  DEV_INLINE f32x4v get() const {
+    f32x4v o;
+    o.v[0] = __builtin_bit_cast(float, r.x << 16);
+    o.v[1] = __builtin_bit_cast(float, r.x & 0xffff0000u);
+    o.v[2] = __builtin_bit_cast(float, r.y << 16);
+    o.v[3] = __builtin_bit_cast(float, r.y & 0xffff0000u);
+    return o;
+  }
+};
+template <>
+struct Raw4<float> {
+  f32x4v r;
+  template <bool VEC>
+  DEV_INLINE void load(const float* p, int valid) {
+    if (VEC) {
+      r = *reinterpret_cast<const f32x4v*>(p);
+    } else {
+#pragma unroll
+      for (int e = 0; e < 4; ++e) r.v[e] = e < valid ? p[e] : 0.f;
+    }
+  }
+  DEV_INLINE f32x4v get() const { return r; }
+};
 
 // four consecutive numbers as fp32: one 8- or 16-byte load when ``vec`` (the
 // caller has checked the alignment and that all four exist), else the first

@@ -31,14 +31,31 @@
 
 #include "seq_common.h"
 
-// tokens per tile: at most 32, the tile within 60 KB of LDS
+// tokens per tile: at most 32, the tile within 58 KB of LDS
 constexpr int cdelta_tile(int dkp, int cols) {
-  const int fit = 60 * 1024 / (4 * (3 * dkp + 2 * cols + 4));
+  const int fit = 58 * 1024 / (4 * (3 * dkp + 2 * cols + 4));
   return fit < 32 ? fit : 32;
 }
 
-template <typename T, int RPL, int CPL, int NW>
-__global__ __launch_bounds__(64 * NW) void channel_delta_kernel(
+// waves per SIMD that single-token steps are compiled for
+#ifndef CDELTA_WAVES
+#define CDELTA_WAVES 4
+#endif
+
+// a token's words of one lane
+template <int RPL, int CPL>
+struct CDeltaIn {
+  f32x4v k[RPL / 4], d[RPL / 4], q[RPL / 4], sc;
+  float v[CPL];
+};
+
+// ONE: every sequence brings one row (tiles of one token, little LDS, so that
+// many blocks share a CU).  VEC: all rows allow loads of four numbers.
+// Addresses beyond a tile's rows or a head's channels are clamped to its last
+// ones and the numbers dropped, so that the loads of a tile are one straight
+// run with nothing waiting between them.
+template <typename T, int RPL, int CPL, int NW, bool ONE, bool VEC>
+__global__ __launch_bounds__(64 * NW, ONE ? CDELTA_WAVES : 1) void channel_delta_kernel(
     T* __restrict__ out, float* __restrict__ out32, const T* __restrict__ q,
     const T* __restrict__ k, const T* __restrict__ v,
     const T* __restrict__ bl, const T* __restrict__ zl,
@@ -47,20 +64,20 @@ __global__ __launch_bounds__(64 * NW) void channel_delta_kernel(
     const float* __restrict__ a_log, const float* __restrict__ norm_w,
     float* __restrict__ state, const int* __restrict__ cu_q,
     const int* __restrict__ state_slot, int H, int G, int Dk, int Dv,
-    float q_scale, float key_eps, float eps, bool veck, bool vecv,
-    bool vecg) {
+    float q_scale, float key_eps, float eps) {
   constexpr int DKP = 8 * RPL;              // key rows incl. padding
   constexpr int CW = 8 * CPL;               // columns of a wave
   constexpr int COLS = NW * CW;
   constexpr int THREADS = 64 * NW;
-  constexpr int TT = cdelta_tile(DKP, COLS);
+  constexpr int TT = ONE ? 1 : cdelta_tile(DKP, COLS);
   constexpr int KU = TT * DKP / 4;          // four-number units of a tile
   constexpr int VU = TT * COLS / 4;
   constexpr int NIT = (KU + THREADS - 1) / THREADS;
   constexpr int NVI = (VU + THREADS - 1) / THREADS;
   constexpr int EC = COLS / 8;              // a lane's columns in the norm pass
   static_assert(TT <= 8 * NW, "one pass of eight lanes per token");
-  __shared__ f32x4v q_s[KU], k_s[KU], d_s[KU], v_s[VU], o_s[VU];
+  __shared__ f32x4v q_s[KU], k_s[KU], d_s[KU], v_s[VU];
+  __shared__ f32x4v o_s[VU + NW * 16 * CPL];   // + where the copies go
   __shared__ f32x4v sc_s[TT];               // 1/|k|, scale/|q|, q.k, beta
 
   const int cblocks = (Dv + COLS - 1) / COLS;
@@ -81,56 +98,84 @@ __global__ __launch_bounds__(64 * NW) void channel_delta_kernel(
   // row i of a lane: four consecutive rows per eight-lane stripe
   auto row_of = [&](int i) { return ((i >> 2) * 8 + rg) * 4 + (i & 3); };
   float* S = state + ((long)state_slot[b] * H + h) * Dk * Dv;
+  constexpr bool PAIR = VEC && CPL == 2;    // columns come in aligned pairs
   float s[CPL][RPL];
 #pragma unroll
-  for (int i = 0; i < RPL; ++i)
+  for (int i = 0; i < RPL; ++i) {
+    const int row = min(row_of(i), Dk - 1);
+    if (PAIR) {
+      const float2 x = *reinterpret_cast<const float2*>(
+          S + (long)row * Dv + min(col, Dv - 2));
+      s[0][i] = x.x;
+      s[CPL - 1][i] = x.y;
+    } else {
 #pragma unroll
-    for (int c = 0; c < CPL; ++c)
-      s[c][i] = (col + c < Dv && row_of(i) < Dk)
-                    ? S[(long)row_of(i) * Dv + col + c] : 0.f;
-  const float A = expf(a_log[h]);
+      for (int c = 0; c < CPL; ++c)
+        s[c][i] = S[(long)row * Dv + min(col + c, Dv - 1)];
+    }
+  }
+  const float A2 = -1.4426950408889634f * expf(a_log[h]);
   const int tn = wid * 8 + cl;              // my token in the norm passes
   const int ec0 = rg * EC;                  // ... and my first column there
-  float nw[EC];
+  auto out_col = [&](int e) {               // VEC: Dv is a multiple of four
+    return min(ec0 + 4 * e, Dv - (VEC ? 4 : 1));
+  };
+  Raw4<float> nw[EC / 4];
 #pragma unroll
-  for (int e = 0; e < EC; ++e)
-    nw[e] = (out && ec0 + e < Dv) ? norm_w[ec0 + e] : 0.f;
+  for (int e = 0; e < EC / 4; ++e)
+    nw[e].template load<VEC>(norm_w + out_col(e), Dv - out_col(e));
 
-  f32x4v rq[NIT], rk[NIT], rz[NIT], rv[NVI], gt[EC / 4];
-  float rb = 0.f;
+  // staging: my four channels (columns) of every TPK-th (TPV-th) token
+  constexpr int TPK = THREADS / (DKP / 4), TPV = THREADS / (COLS / 4);
+  static_assert(THREADS % (DKP / 4) == 0 && THREADS % (COLS / 4) == 0, "");
+  const int kt = tid / (DKP / 4), kr = (tid % (DKP / 4)) * 4;
+  const int vt = tid / (COLS / 4), vc = (tid % (COLS / 4)) * 4;
+  const int krl = max(min(kr, Dk - 4), 0);  // VEC: Dk and Dv are multiples
+  const int kra = VEC ? krl : min(kr, Dk - 1);                   // of four
+  const int vca = VEC ? min(cb0 + vc, Dv - 4) : min(cb0 + vc, Dv - 1);
+  const bool kok = kr < Dk;
+  Raw4<float> bias;
+  bias.template load<VEC>(dt_bias + h * Dk + kra, Dk - kra);
+
+  Raw4<T> rq[NIT], rk[NIT], rz[NIT], rv[NVI], gt[EC / 4];
+  T rb;
   auto fetch = [&](int n0) {
-    const int cnt = q1 - n0 < TT ? q1 - n0 : TT;
+    const int last = min(q1 - n0, TT) - 1;
 #pragma unroll
     for (int it = 0; it < NIT; ++it) {
-      if (it * THREADS * 4 >= cnt * DKP) break;      // block-uniform
-      const int u = tid + it * THREADS;
-      const int t = u / (DKP / 4), r = (u % (DKP / 4)) * 4;
-      const bool ok = t < cnt && r < Dk;
-      const f32x4v z4 = {{0.f, 0.f, 0.f, 0.f}};
-      rq[it] = z4; rk[it] = z4; rz[it] = z4;
-      if (ok) {
-        const long n = n0 + t;
-        rq[it] = load4(q + n * ldq + hk + r, Dk - r, veck);
-        rk[it] = load4(k + n * ldk + hk + r, Dk - r, veck);
-        rz[it] = load4(zl + n * ldz + h * Dk + r, Dk - r, veck);
-        const f32x4v bi = load4(dt_bias + h * Dk + r, Dk - r, veck);
-#pragma unroll
-        for (int e = 0; e < 4; ++e) rz[it].v[e] += bi.v[e];
-      }
+      const long n = n0 + min(kt + it * TPK, last);
+      rq[it].template load<VEC>(q + n * ldq + hk + kra, Dk - kra);
+      rk[it].template load<VEC>(k + n * ldk + hk + kra, Dk - kra);
+      rz[it].template load<VEC>(zl + n * ldz + h * Dk + kra, Dk - kra);
     }
 #pragma unroll
     for (int it = 0; it < NVI; ++it) {
-      if (it * THREADS * 4 >= cnt * COLS) break;
-      const int u = tid + it * THREADS;
-      const int t = u / (COLS / 4), c = cb0 + (u % (COLS / 4)) * 4;
-      if (t < cnt && c < Dv)
-        rv[it] = load4(v + (long)(n0 + t) * ldv + h * Dv + c, Dv - c, vecv);
-      else
-        rv[it] = {{0.f, 0.f, 0.f, 0.f}};
+      const long n = n0 + min(vt + it * TPV, last);
+      rv[it].template load<VEC>(v + n * ldv + h * Dv + vca, Dv - vca);
     }
-    rb = tn < cnt ? ldf(bl + (long)(n0 + tn) * ldb + h) : 0.f;
+    const long n = n0 + min(tn, last);
+    rb = bl[n * ldb + h];
+#pragma unroll
+    for (int e = 0; e < EC / 4; ++e)
+      gt[e].template load<VEC>(gate + n * ldg + h * Dv + out_col(e),
+                               Dv - out_col(e));
   };
   fetch(q0);
+  // the state is needed in the first walk only once: wait for it here, or
+  // every walk would also wait for the next tile's words
+  __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+  for (int i = 0; i < RPL; ++i)
+#pragma unroll
+    for (int c = 0; c < CPL; ++c) {
+      if (col + c >= Dv || row_of(i) >= Dk) s[c][i] = 0.f;
+      if (!ONE) asm volatile("" : "+v"(s[c][i]));
+    }
+  // all eight lanes of a column hold its output: the first writes it to the
+  // tile, the others to words of their own (no branch in the walk)
+  float* o_at = reinterpret_cast<float*>(o_s) +
+                (rg == 0 ? wcol : TT * COLS + tid * CPL);
+  const int o_step = rg == 0 ? COLS : 0;
 
   for (int n0 = q0; n0 < q1; n0 += TT) {
     const int cnt = q1 - n0 < TT ? q1 - n0 : TT;
@@ -139,32 +184,30 @@ __global__ __launch_bounds__(64 * NW) void channel_delta_kernel(
     for (int it = 0; it < NIT; ++it) {
       const int u = tid + it * THREADS;
       if (u * 4 < cnt * DKP) {
-        q_s[u] = rq[it];
-        k_s[u] = rk[it];
-        f32x4v d;
+        const f32x4v z = rz[it].get(), bi = bias.get();
+        f32x4v d, qv = rq[it].get(), kv = rk[it].get();
 #pragma unroll
-        for (int e = 0; e < 4; ++e)
-          d.v[e] = expf(-A * softplusf_acc(rz[it].v[e]));
+        for (int e = 0; e < 4; ++e) {
+          d.v[e] = __builtin_amdgcn_exp2f(
+              A2 * softplusf_fast(z.v[e] + bi.v[e]));
+          if (!kok) qv.v[e] = kv.v[e] = 0.f;
+        }
+        q_s[u] = qv;
+        k_s[u] = kv;
         d_s[u] = d;
       }
     }
 #pragma unroll
     for (int it = 0; it < NVI; ++it) {
       const int u = tid + it * THREADS;
-      if (u * 4 < cnt * COLS) v_s[u] = rv[it];
+      if (u * 4 < cnt * COLS) v_s[u] = rv[it].get();
     }
-    const float bcur = rb;
-    __syncthreads();
-    if (out && tn < cnt) {                  // this tile's output gates
+    const float bcur = ldf(&rb);
+    Raw4<T> gc[EC / 4];
 #pragma unroll
-      for (int e = 0; e < EC / 4; ++e) {
-        const int c = ec0 + 4 * e;
-        gt[e] = c < Dv ? load4(gate + (long)(n0 + tn) * ldg + h * Dv + c,
-                               Dv - c, vecg)
-                       : f32x4v{{0.f, 0.f, 0.f, 0.f}};
-      }
-    }
-    if (n0 + TT < q1) fetch(n0 + TT);       // in flight during the walk
+    for (int e = 0; e < EC / 4; ++e) gc[e] = gt[e];
+    __syncthreads();
+    if (!ONE && n0 + TT < q1) fetch(n0 + TT);   // in flight during the walk
     if (tn < cnt) {                         // lengths, eight lanes per token
       float sq = 0.f, sk = 0.f, qk = 0.f;
 #pragma unroll
@@ -184,56 +227,77 @@ __global__ __launch_bounds__(64 * NW) void channel_delta_kernel(
       if (rg == 0) {
         const float iq = q_scale * rsqrtf(sq + key_eps);
         const float ik = rsqrtf(sk + key_eps);
-        sc_s[tn] = {{ik, iq, qk * ik * iq, sigmoidf_acc(bcur)}};
+        sc_s[tn] = {{ik, iq, qk * ik * iq, sigmoidf_fast(bcur)}};
       }
     }
     __syncthreads();
     if (wave_live) {
-      auto step = [&](int t) {
-        const f32x4v sc = sc_s[t];
-        float kk[RPL], p[CPL], o[CPL], vv[CPL];
+      using In = CDeltaIn<RPL, CPL>;
+      auto words = [&](In& in, int t) {
+        in.sc = sc_s[t];
         const float* vr = reinterpret_cast<const float*>(v_s) + t * COLS + wcol;
 #pragma unroll
-        for (int c = 0; c < CPL; ++c) {
-          p[c] = 0.f;
-          o[c] = 0.f;
-          vv[c] = vr[c];
-        }
+        for (int c = 0; c < CPL; ++c) in.v[c] = vr[c];
 #pragma unroll
         for (int j = 0; j < RPL / 4; ++j) {
           const int at = t * (DKP / 4) + j * 8 + rg;
-          const f32x4v kq = k_s[at], dq = d_s[at], qq = q_s[at];
-#pragma unroll
-          for (int e = 0; e < 4; ++e) {
-            kk[4 * j + e] = kq.v[e];
-#pragma unroll
-            for (int c = 0; c < CPL; ++c) {
-              const float x = s[c][4 * j + e] * dq.v[e];
-              s[c][4 * j + e] = x;
-              p[c] += x * kq.v[e];
-              o[c] += x * qq.v[e];
-            }
-          }
-        }
-        float* orow = reinterpret_cast<float*>(o_s) + t * COLS + wcol;
-#pragma unroll
-        for (int c = 0; c < CPL; ++c) {
-          p[c] = oct_sum(p[c]);
-          o[c] = oct_sum(o[c]);
-          const float u = sc.v[3] * (vv[c] - sc.v[0] * p[c]);
-          const float ku = sc.v[0] * u;
-#pragma unroll
-          for (int i = 0; i < RPL; ++i) s[c][i] += kk[i] * ku;
-          o[c] = sc.v[1] * o[c] + sc.v[2] * u;
-          if (rg == 0) orow[c] = o[c];
+          in.k[j] = k_s[at];
+          in.d[j] = d_s[at];
+          in.q[j] = q_s[at];
         }
       };
-      int t = 0;
-      for (; t + 2 <= cnt; t += 2) {
-        step(t);
-        step(t + 1);
+      auto step = [&](const In& in, int t) {
+        float p[CPL], o[CPL];
+#pragma unroll
+        for (int c = 0; c < CPL; ++c) p[c] = o[c] = 0.f;
+#pragma unroll
+        for (int i = 0; i < RPL; ++i)
+#pragma unroll
+          for (int c = 0; c < CPL; ++c) {
+            const float x = s[c][i] * in.d[i / 4].v[i % 4];
+            s[c][i] = x;
+            p[c] += x * in.k[i / 4].v[i % 4];
+            o[c] += x * in.q[i / 4].v[i % 4];
+          }
+#pragma unroll
+        for (int c = 0; c < CPL; ++c) p[c] = oct_sum(p[c]);
+#pragma unroll
+        for (int c = 0; c < CPL; ++c) {
+          const float u = in.sc.v[3] * (in.v[c] - in.sc.v[0] * p[c]);
+          const float ku = in.sc.v[0] * u;
+#pragma unroll
+          for (int i = 0; i < RPL; ++i) s[c][i] += in.k[i / 4].v[i % 4] * ku;
+          p[c] = u;
+        }
+#pragma unroll
+        for (int c = 0; c < CPL; ++c)
+          o_at[t * o_step + c] = in.sc.v[1] * oct_sum(o[c]) + in.sc.v[2] * p[c];
+      };
+      if (ONE) {
+        In in;
+        words(in, 0);
+        step(in, 0);
+      } else if (RPL <= 16) {
+        // the next token's words are read while this one is worked on
+        In a, b;
+        words(a, 0);
+        int t = 0;
+        for (; t + 2 <= cnt; t += 2) {
+          words(b, t + 1);
+          __builtin_amdgcn_sched_barrier(0);
+          step(a, t);
+          words(a, t + 2 < cnt ? t + 2 : t + 1);
+          __builtin_amdgcn_sched_barrier(0);
+          step(b, t + 1);
+        }
+        if (t < cnt) step(a, t);
+      } else {
+        for (int t = 0; t < cnt; ++t) {
+          In in;
+          words(in, t);
+          step(in, t);
+        }
       }
-      if (t < cnt) step(t);
     }
     __syncthreads();                        // head outputs are complete
     if (tn < cnt) {
@@ -252,11 +316,12 @@ __global__ __launch_bounds__(64 * NW) void channel_delta_kernel(
           const int c = ec0 + 4 * e;
           if (c >= Dv) continue;
           f32x4v y;
+          const f32x4v g4 = gc[e].get(), w4 = nw[e].get();
 #pragma unroll
           for (int x = 0; x < 4; ++x)
-            y.v[x] = ov[4 * e + x] * inv * nw[4 * e + x] *
-                     sigmoidf_acc(gt[e].v[x]);
-          store4(out + (n * H + h) * Dv + c, y, Dv - c, vecv);
+            y.v[x] = ov[4 * e + x] * inv * w4.v[x] *
+                     sigmoidf_fast(g4.v[x]);
+          store4(out + (n * H + h) * Dv + c, y, Dv - c, VEC);
         }
       } else {
 #pragma unroll
@@ -267,18 +332,24 @@ __global__ __launch_bounds__(64 * NW) void channel_delta_kernel(
     }
   }
 #pragma unroll
-  for (int i = 0; i < RPL; ++i)
+  for (int i = 0; i < RPL; ++i) {
+    if (row_of(i) >= Dk) continue;
+    float* at = S + (long)row_of(i) * Dv + col;
+    if (PAIR) {
+      if (col < Dv) *reinterpret_cast<float2*>(at) = {s[0][i], s[CPL - 1][i]};
+    } else {
 #pragma unroll
-    for (int c = 0; c < CPL; ++c)
-      if (col + c < Dv && row_of(i) < Dk)
-        S[(long)row_of(i) * Dv + col + c] = s[c][i];
+      for (int c = 0; c < CPL; ++c)
+        if (col + c < Dv) at[c] = s[c][i];
+    }
+  }
 }
 
 void seq_group_rmsnorm(torch::Tensor out, torch::Tensor y,
                        torch::Tensor weight, int64_t groups, double eps,
                        torch::Tensor gate, int64_t gate_act);
 
-template <typename T, int RPL, int CPL, int NW>
+template <typename T, int RPL, int CPL, int NW, bool ONE, bool VEC>
 static void cdelta_launch(torch::Tensor& out, torch::Tensor& q,
                           torch::Tensor& k, torch::Tensor& v,
                           torch::Tensor& bl, torch::Tensor& zl,
@@ -295,13 +366,8 @@ static void cdelta_launch(torch::Tensor& out, torch::Tensor& q,
   if (!fused)
     raw = torch::empty({q.size(0), (long)H * Dv},
                        q.options().dtype(torch::kFloat32));
-  const bool veck = rows_by4<T>(q, Dk) && rows_by4<T>(k, Dk) &&
-                    rows_by4<T>(zl, Dk) &&
-                    (uintptr_t)dt_bias.data_ptr() % 16 == 0;
-  const bool vecv = rows_by4<T>(v, Dv) && rows_by4<T>(out, Dv);
-  const bool vecg = rows_by4<T>(gate, Dv);
   auto stream = at::hip::getCurrentHIPStream();
-  hipLaunchKernelGGL((channel_delta_kernel<T, RPL, CPL, NW>),
+  hipLaunchKernelGGL((channel_delta_kernel<T, RPL, CPL, NW, ONE, VEC>),
       dim3((unsigned)(slot.numel() * H * cblocks)), dim3(64 * NW), 0, stream,
       fused ? (T*)out.data_ptr() : nullptr,
       fused ? nullptr : raw.data_ptr<float>(), (const T*)q.data_ptr(),
@@ -311,7 +377,7 @@ static void cdelta_launch(torch::Tensor& out, torch::Tensor& q,
       dt_bias.data_ptr<float>(), a_log.data_ptr<float>(),
       norm_w.data_ptr<float>(), state.data_ptr<float>(),
       cu_q.data_ptr<int>(), slot.data_ptr<int>(), H, G, Dk, Dv,
-      1.f / sqrtf((float)Dk), (float)key_eps, (float)eps, veck, vecv, vecg);
+      1.f / sqrtf((float)Dk), (float)key_eps, (float)eps);
   HIP_CHECK_KERNEL();
   if (!fused) seq_group_rmsnorm(out, raw, norm_w, H, eps, gate, 1);
 }
@@ -322,7 +388,7 @@ void seq_channel_delta(torch::Tensor out, torch::Tensor q, torch::Tensor k,
                        torch::Tensor a_log, torch::Tensor gate,
                        torch::Tensor norm_w, torch::Tensor state,
                        torch::Tensor cu_q, torch::Tensor state_slot,
-                       double key_eps, double eps) {
+                       double key_eps, double eps, int64_t max_rows) {
   CHECK_ROWS(q); CHECK_ROWS(k); CHECK_ROWS(v); CHECK_ROWS(b_lin);
   CHECK_ROWS(z_lin); CHECK_ROWS(gate);
   CHECK_F32(dt_bias); CHECK_F32(a_log); CHECK_F32(norm_w); CHECK_F32(state);
@@ -348,13 +414,25 @@ void seq_channel_delta(torch::Tensor out, torch::Tensor q, torch::Tensor k,
   TORCH_CHECK(Dk <= 512, "delta rule: key dim above 512 not supported");
   TORCH_CHECK(cu_q.numel() == state_slot.numel() + 1);
   if (N == 0 || state_slot.numel() == 0) return;
+#define CDELTA_ARGS                                                           \
+  (out, q, k, v, b_lin, z_lin, dt_bias, a_log, gate, norm_w, state, cu_q,     \
+   state_slot, key_eps, eps)
 #define CDELTA(RPLV, CPLV, NWV)                                               \
-  cdelta_launch<T, RPLV, CPLV, NWV>(out, q, k, v, b_lin, z_lin, dt_bias,      \
-      a_log, gate, norm_w, state, cu_q, state_slot, key_eps, eps)
+  do {                                                                        \
+    if (!vec) cdelta_launch<T, RPLV, CPLV, 8, false, false> CDELTA_ARGS;      \
+    else if (max_rows == 1)                                                   \
+      cdelta_launch<T, RPLV, CPLV, NWV, true, true> CDELTA_ARGS;              \
+    else cdelta_launch<T, RPLV, CPLV, NWV, false, true> CDELTA_ARGS;          \
+  } while (0)
 #define CDELTA_W(RPLV, CPLV)                                                  \
   do { if (Dv <= 32 * CPLV) CDELTA(RPLV, CPLV, 4);                            \
        else CDELTA(RPLV, CPLV, 8); } while (0)
   SEQ_DISPATCH_T(dt, {
+    const bool vec = rows_by4<T>(q, Dk) && rows_by4<T>(k, Dk) &&
+                     rows_by4<T>(z_lin, Dk) && rows_by4<T>(v, Dv) &&
+                     rows_by4<T>(gate, Dv) && rows_by4<T>(out, Dv) &&
+                     (uintptr_t)dt_bias.data_ptr() % 16 == 0 &&
+                     (uintptr_t)state.data_ptr() % 16 == 0;
     if (Dk <= 32) CDELTA_W(4, 2);
     else if (Dk <= 64) CDELTA_W(8, 2);
     else if (Dk <= 128) CDELTA_W(16, 2);
@@ -363,4 +441,5 @@ void seq_channel_delta(torch::Tensor out, torch::Tensor q, torch::Tensor k,
   });
 #undef CDELTA_W
 #undef CDELTA
+#undef CDELTA_ARGS
 }

@@ -248,6 +248,86 @@ __global__ __launch_bounds__(256) void gqa_prepare_headnorm_kernel(
   }
 }
 
+// The same for head sizes D = 4 * LPH with LPH a power of two and half a
+// multiple of four: LPH lanes hold a head, four consecutive numbers each, so
+// a wave works on 64/LPH heads at once; the token's cosines and sines are
+// taken once per block.  Grid (tokens, blocks of 4*hpw heads).
+template <typename T, int LPH>
+__global__ __launch_bounds__(256) void gqa_prepare_headnorm4_kernel(
+    T* __restrict__ q_out, const T* __restrict__ q, long ldq,
+    const T* __restrict__ k, long ldk, const T* __restrict__ v, long ldv,
+    const float* __restrict__ qn, const float* __restrict__ kn, float eps,
+    const float* __restrict__ inv_freq, int half, float amp,
+    const int* __restrict__ positions, T* __restrict__ cache,
+    const int* __restrict__ slot_mapping, int H, int G, int Dv, int hpw,
+    bool vecv) {
+  constexpr int D = 4 * LPH;
+  constexpr int HPI = 64 / LPH;         // heads of a wave at once
+  __shared__ f32x4v cs_s[LPH];          // cosines then sines, half each
+  __shared__ f32x4v xs_s[4][64];
+  const long n = blockIdx.x;
+  const int wid = threadIdx.x >> 6, lane = threadIdx.x & 63;
+  const int l = lane % LPH, i = 4 * l;
+  T* crow = cache + (long)slot_mapping[n] * (G * (D + Dv));
+  if ((int)threadIdx.x < half) {
+    const float ang = (float)positions[n] * inv_freq[threadIdx.x];
+    float* cs = reinterpret_cast<float*>(cs_s);
+    cs[threadIdx.x] = cosf(ang) * amp;
+    cs[half + threadIdx.x] = sinf(ang) * amp;
+  }
+  if (blockIdx.y == 0) {                // the values as they are
+    const T* vr = v + n * ldv;
+    T* vd = crow + G * D;
+    for (int u = threadIdx.x * 4; u < G * Dv; u += 1024)
+      store4(vd + u, load4(vr + u, G * Dv - u, vecv), G * Dv - u, vecv);
+  }
+  __syncthreads();
+  const bool lo = i < half, turned = i < 2 * half;
+  const int pl = lo ? l + half / 4 : l - half / 4;    // partner's place
+  const f32x4v one = {{1.f, 1.f, 1.f, 1.f}}, zero = {{0.f, 0.f, 0.f, 0.f}};
+  const f32x4v c = turned ? cs_s[lo ? l : l - half / 4] : one;
+  const f32x4v s = turned ? cs_s[lo ? l + half / 4 : l] : zero;
+  const float sign = lo ? -1.f : 1.f;
+  const int h0 = (blockIdx.y * 4 + wid) * hpw;
+  const int h1 = min(h0 + hpw, H + G);
+  f32x4v* xs = xs_s[wid] + lane - l;
+  for (int hb = h0; hb < h1; hb += HPI) {
+    const int hu = hb + lane / LPH;
+    const bool ok = hu < h1, isq = hu < H;
+    const T* src = isq ? q + n * ldq + (long)hu * D
+                       : k + n * ldk + (long)(hu - H) * D;
+    f32x4v x = ok ? load4(src + i, 4, true) : zero;
+    float ss = 0.f;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) ss += x.v[e] * x.v[e];
+    const float inv = rsqrtf(lanegroup_sum<LPH>(ss) / D + eps);
+    const f32x4v w = load4((isq ? qn : kn) + i, 4, true);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) x.v[e] *= inv * w.v[e];
+    xs[l] = x;
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+    const f32x4v p = turned ? xs[pl] : zero;
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+    f32x4v y;
+#pragma unroll
+    for (int e = 0; e < 4; ++e)
+      y.v[e] = x.v[e] * c.v[e] + sign * p.v[e] * s.v[e];
+    if (ok)
+      store4((isq ? q_out + (n * H + hu) * D : crow + (hu - H) * D) + i, y, 4,
+             true);
+  }
+}
+
+#define PREP4(LPHV)                                                           \
+  hipLaunchKernelGGL((gqa_prepare_headnorm4_kernel<T, LPHV>), grid,           \
+      dim3(256), 0, stream, (T*)q_out.data_ptr(), (const T*)q.data_ptr(),     \
+      q.stride(0), (const T*)k.data_ptr(), k.stride(0),                       \
+      (const T*)v.data_ptr(), v.stride(0), q_norm.data_ptr<float>(),          \
+      k_norm.data_ptr<float>(), (float)eps,                                   \
+      half ? inv_freq.data_ptr<float>() : nullptr, half, (float)amp,          \
+      positions.data_ptr<int>(), (T*)cache.data_ptr(),                        \
+      slot_mapping.data_ptr<int>(), (int)H, (int)G, (int)Dv, hpw, vecv)
+
 void seq_gqa_prepare_store(torch::Tensor q_out, torch::Tensor q,
                            torch::Tensor k, torch::Tensor v,
                            torch::Tensor q_norm, torch::Tensor k_norm,
@@ -295,6 +375,37 @@ void seq_gqa_prepare_store(torch::Tensor q_out, torch::Tensor q,
     TORCH_CHECK(has_v && !head_unit && !v_rot,
                 "per-head norm weights: values of their own, no other option");
     TORCH_CHECK(D <= 512, "head sizes above 512 are not supported");
+    const int lph = (int)(D / 4);
+    const auto fits = [](const torch::Tensor& t, size_t bytes) {
+      return (uintptr_t)t.data_ptr() % bytes == 0; };
+    bool by4 = D % 4 == 0 && half % 4 == 0 && lph <= 64 &&
+               (lph & (lph - 1)) == 0 && fits(q_norm, 16) && fits(k_norm, 16);
+    bool vecv = false;
+    SEQ_DISPATCH_T(ty, {
+      by4 = by4 && rows_by4<T>(q, D) && rows_by4<T>(k, D) &&
+            fits(q_out, 4 * sizeof(T)) && fits(cache, 4 * sizeof(T)) &&
+            (G * Dv) % 4 == 0;
+      vecv = by4 && rows_by4<T>(v, G * Dv); });
+    if (by4) {
+      // long steps: a block takes all heads of a token; short ones: as many
+      // waves as there are head groups
+      const int hpi = 64 / lph, qk = (int)(H + G);
+      const int groups = (qk + hpi - 1) / hpi;
+      const int hpw = (N >= 1024 ? (groups + 3) / 4 : 1) * hpi;
+      const dim3 grid(N, (qk + 4 * hpw - 1) / (4 * hpw));
+      SEQ_DISPATCH_T(ty, {
+        switch (lph) {
+          case 1: PREP4(1); break;
+          case 2: PREP4(2); break;
+          case 4: PREP4(4); break;
+          case 8: PREP4(8); break;
+          case 16: PREP4(16); break;
+          case 32: PREP4(32); break;
+          default: PREP4(64); break;
+        } });
+      HIP_CHECK_KERNEL();
+      return;
+    }
     // heads per wave: enough waves to fill the chip first
     const int heads = (int)(H + 2 * G);
     const int hpw = N >= 4096 ? 8 : N >= 1024 ? 4 : 1;

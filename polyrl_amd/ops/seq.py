@@ -275,7 +275,7 @@ def gla_scan(q, k, v, z_lin, z_bias, state, cu_q, state_slot,
 
 def channel_delta_scan(q, k, v, b_lin, z_lin, dt_bias, a_log, gate, norm_w,
                        state, cu_q, state_slot, key_eps: float, eps: float,
-                       out_dtype) -> torch.Tensor:
+                       out_dtype, max_rows: int = 0) -> torch.Tensor:
     """Gated delta rule with per-channel decays over packed rows; ``state``
     (slots, H, Dk, Dv) fp32 in place.  q, k (N, G*Dk): head h uses q/k head
     h // (H/G); both are made unit vectors x / sqrt(sum x^2 + key_eps), q is
@@ -283,7 +283,8 @@ def channel_delta_scan(q, k, v, b_lin, z_lin, dt_bias, a_log, gate, norm_w,
     g = exp(-exp(a_log) * softplus(z_lin + dt_bias)) per key channel,
     S <- g S, u = beta (v - S^T k), S <- S + k u^T, o = S^T q; returns
     o / rms_head(o) * norm_w * sigmoid(gate) (N, H*Dv), norm_w (Dv,) shared
-    by the heads.  Inputs may be column slices."""
+    by the heads.  Inputs may be column slices.  ``max_rows`` bounds the
+    rows of one sequence (0 = unknown)."""
     if q.is_cuda:
         slots, H, Dk, Dv = state.shape
         out = torch.empty(q.shape[0], H * Dv, dtype=out_dtype,
@@ -291,7 +292,7 @@ def channel_delta_scan(q, k, v, b_lin, z_lin, dt_bias, a_log, gate, norm_w,
         if q.shape[0]:
             _ext().seq_channel_delta(out, q, k, v, b_lin, z_lin, dt_bias,
                                      a_log, gate, norm_w, state, cu_q,
-                                     state_slot, key_eps, eps)
+                                     state_slot, key_eps, eps, max_rows)
         return out
     return R.channel_delta_scan(q, k, v, b_lin, z_lin, dt_bias, a_log, gate,
                                 norm_w, state, cu_q, state_slot, key_eps,
@@ -299,20 +300,21 @@ def channel_delta_scan(q, k, v, b_lin, z_lin, dt_bias, a_log, gate, norm_w,
 
 
 def selective_scan(x, dt_lin, dt_bias, Bm, Cm, a_log, d_skip, z, state, cu_q,
-                   state_slot, out=None,
-                   out_scale: float = 1.0) -> torch.Tensor:
+                   state_slot, out=None, out_scale: float = 1.0,
+                   max_rows: int = 0) -> torch.Tensor:
     """Selective scan over packed rows; ``state`` (slots, C, Ns) fp32 in
     place.  dt = softplus(dt_lin + dt_bias) per channel;
     S <- exp(-exp(a_log) dt) S + dt x B^T, y = S C + d_skip x; returns
     y * silu(z) * out_scale (N, C) in ``out`` (a column slice is allowed)
-    or a new tensor.  Inputs may be column slices."""
+    or a new tensor.  Inputs may be column slices.  ``max_rows`` bounds the
+    rows of one sequence (0 = unknown)."""
     if x.is_cuda:
         if out is None:
             out = torch.empty(x.shape, dtype=x.dtype, device=x.device)
         if x.shape[0]:
             _ext().seq_selective_scan(out, x, dt_lin, dt_bias, Bm, Cm, a_log,
                                       d_skip, z, state, cu_q, state_slot,
-                                      out_scale)
+                                      out_scale, max_rows)
         return out
     return R.selective_scan(x, dt_lin, dt_bias, Bm, Cm, a_log, d_skip, z,
                             state, cu_q, state_slot, out, out_scale)

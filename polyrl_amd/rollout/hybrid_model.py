@@ -208,7 +208,7 @@ class ChannelDeltaMixer(_Part):
             low.narrow(1, 0, self.nz), self.dt_bias, self.a_log,
             low.narrow(1, self.nz, self.nv), self.norm,
             states.tensors[(li, "S")], bt.cu_q, bt.state_slot, s.key_eps,
-            model.cfg.norm_eps, h.dtype)
+            model.cfg.norm_eps, h.dtype, max_rows=bt.max_q)
         return _mm(y, self.wo)
 
 
@@ -262,7 +262,7 @@ class SelectiveScanMixer(_Part):
             x, dt, self.dt_b, dbc.narrow(1, R, N), dbc.narrow(1, R + N, N),
             self.a_log, self.d, proj.narrow(1, C, C),
             states.tensors[(li, self.key + "S")], bt.cu_q, bt.state_slot,
-            out=out, out_scale=scale)
+            out=out, out_scale=scale, max_rows=bt.max_q)
 
     def forward(self, h, bt, li, model, cache, states):
         return _mm(self.mix(_mm(h, self.w_in), bt, li, model, cache, states),

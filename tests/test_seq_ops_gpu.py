@@ -795,7 +795,8 @@ def test_softcap_logits(dt):
 @pytest.mark.parametrize("dt", DTYPES)
 @pytest.mark.parametrize("H,G,Dk,Dv,lens", [
     (4, 2, 12, 8, [5, 1, 40]), (1, 1, 3, 5, [2, 33]), (3, 1, 33, 64, [65, 1]),
-    (2, 2, 64, 64, [1, 1, 1]), (2, 2, 64, 64, [31, 32, 33, 100]),
+    (2, 2, 64, 64, [1, 1, 1]), (3, 1, 30, 100, [1, 1]),
+    (2, 1, 130, 150, [1, 1, 1]), (1, 1, 300, 9, [1]), (2, 2, 64, 64, [31, 32, 33, 100]),
     (2, 1, 64, 128, [70, 3]), (1, 1, 128, 128, [50, 1]),
     (2, 1, 20, 150, [9, 40]), (1, 1, 200, 24, [30]), (1, 1, 256, 70, [20]),
     (1, 1, 300, 40, [21, 1]), (2, 2, 512, 64, [11])])
@@ -817,7 +818,8 @@ def test_channel_delta_scan(dt, H, G, Dk, Dv, lens):
         return mod.channel_delta_scan(
             x[:, :nk], x[:, nk:2 * nk], x[:, 2 * nk:2 * nk + nv],
             x[:, 2 * nk + nv:2 * nk + nv + H], lo[:, :nz], dtb.to(d),
-            alog.to(d), lo[:, nz:], nw.to(d), s, c, sl, 1e-6, 1e-5, dt)
+            alog.to(d), lo[:, nz:], nw.to(d), s, c, sl, 1e-6, 1e-5, dt,
+            **({"max_rows": max(lens)} if d == DEV else {}))
     s0, s1 = st.clone(), st.clone().to(DEV)
     want, got = go(R, "cpu", s0), go(seq, DEV, s1)
     torch.testing.assert_close(s1.cpu(), s0, rtol=1e-4, atol=1e-5)
@@ -850,7 +852,7 @@ def test_selective_scan(dt, C, Ns, R_, lens):
                                   c, sl, out_scale=0.7, **kw)
     s0, s1 = st.clone(), st.clone().to(DEV)
     want = go(R, "cpu", s0)
-    got = go(seq, DEV, s1, out=out[:, 12:12 + C])
+    got = go(seq, DEV, s1, out=out[:, 12:12 + C], max_rows=max(lens))
     torch.testing.assert_close(s1.cpu(), s0, rtol=1e-4, atol=1e-5)
     torch.testing.assert_close(
         got.cpu().float(), want.float(),
