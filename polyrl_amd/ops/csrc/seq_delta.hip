@@ -37,11 +37,6 @@ constexpr int cdelta_tile(int dkp, int cols) {
   return fit < 32 ? fit : 32;
 }
 
-// waves per SIMD that single-token steps are compiled for
-#ifndef CDELTA_WAVES
-#define CDELTA_WAVES 4
-#endif
-
 // a token's words of one lane
 template <int RPL, int CPL>
 struct CDeltaIn {
@@ -50,12 +45,13 @@ struct CDeltaIn {
 };
 
 // ONE: every sequence brings one row (tiles of one token, little LDS, so that
-// many blocks share a CU).  VEC: all rows allow loads of four numbers.
+// many blocks share a CU; with four columns per lane a wave reads and writes
+// whole 128-byte lines of the state, which is what such a step is bound by).  VEC: all rows allow loads of four numbers.
 // Addresses beyond a tile's rows or a head's channels are clamped to its last
 // ones and the numbers dropped, so that the loads of a tile are one straight
 // run with nothing waiting between them.
 template <typename T, int RPL, int CPL, int NW, bool ONE, bool VEC>
-__global__ __launch_bounds__(64 * NW, ONE ? CDELTA_WAVES : 1) void channel_delta_kernel(
+__global__ __launch_bounds__(64 * NW, ONE && RPL <= 8 ? 4 : 1) void channel_delta_kernel(
     T* __restrict__ out, float* __restrict__ out32, const T* __restrict__ q,
     const T* __restrict__ k, const T* __restrict__ v,
     const T* __restrict__ bl, const T* __restrict__ zl,
@@ -98,16 +94,17 @@ __global__ __launch_bounds__(64 * NW, ONE ? CDELTA_WAVES : 1) void channel_delta
   // row i of a lane: four consecutive rows per eight-lane stripe
   auto row_of = [&](int i) { return ((i >> 2) * 8 + rg) * 4 + (i & 3); };
   float* S = state + ((long)state_slot[b] * H + h) * Dk * Dv;
-  constexpr bool PAIR = VEC && CPL == 2;    // columns come in aligned pairs
+  // VEC: a lane's columns exist together and are aligned to their number
+  struct alignas(4 * CPL) Cols { float x[CPL]; };
   float s[CPL][RPL];
 #pragma unroll
   for (int i = 0; i < RPL; ++i) {
     const int row = min(row_of(i), Dk - 1);
-    if (PAIR) {
-      const float2 x = *reinterpret_cast<const float2*>(
-          S + (long)row * Dv + min(col, Dv - 2));
-      s[0][i] = x.x;
-      s[CPL - 1][i] = x.y;
+    if (VEC) {
+      const Cols x = *reinterpret_cast<const Cols*>(
+          S + (long)row * Dv + min(col, Dv - CPL));
+#pragma unroll
+      for (int c = 0; c < CPL; ++c) s[c][i] = x.x[c];
     } else {
 #pragma unroll
       for (int c = 0; c < CPL; ++c)
@@ -335,8 +332,11 @@ __global__ __launch_bounds__(64 * NW, ONE ? CDELTA_WAVES : 1) void channel_delta
   for (int i = 0; i < RPL; ++i) {
     if (row_of(i) >= Dk) continue;
     float* at = S + (long)row_of(i) * Dv + col;
-    if (PAIR) {
-      if (col < Dv) *reinterpret_cast<float2*>(at) = {s[0][i], s[CPL - 1][i]};
+    if (VEC) {
+      Cols x;
+#pragma unroll
+      for (int c = 0; c < CPL; ++c) x.x[c] = s[c][i];
+      if (col < Dv) *reinterpret_cast<Cols*>(at) = x;
     } else {
 #pragma unroll
       for (int c = 0; c < CPL; ++c)
@@ -417,27 +417,31 @@ void seq_channel_delta(torch::Tensor out, torch::Tensor q, torch::Tensor k,
 #define CDELTA_ARGS                                                           \
   (out, q, k, v, b_lin, z_lin, dt_bias, a_log, gate, norm_w, state, cu_q,     \
    state_slot, key_eps, eps)
-#define CDELTA(RPLV, CPLV, NWV)                                               \
+// CPLV / NWV: columns per lane and waves of portions, CPL1 / NW1 of single
+// tokens
+#define CDELTA(RPLV, CPLV, NWV, CPL1, NW1)                                    \
   do {                                                                        \
     if (!vec) cdelta_launch<T, RPLV, CPLV, 8, false, false> CDELTA_ARGS;      \
     else if (max_rows == 1)                                                   \
-      cdelta_launch<T, RPLV, CPLV, NWV, true, true> CDELTA_ARGS;              \
+      cdelta_launch<T, RPLV, CPL1, NW1, true, true> CDELTA_ARGS;              \
     else cdelta_launch<T, RPLV, CPLV, NWV, false, true> CDELTA_ARGS;          \
   } while (0)
-#define CDELTA_W(RPLV, CPLV)                                                  \
-  do { if (Dv <= 32 * CPLV) CDELTA(RPLV, CPLV, 4);                            \
-       else CDELTA(RPLV, CPLV, 8); } while (0)
+#define CDELTA_W(RPLV, CPLV, CPL1)                                            \
+  do {                                                                        \
+    if (Dv <= 64) CDELTA(RPLV, CPLV, 8 / CPLV, CPL1, 8 / CPL1);               \
+    else CDELTA(RPLV, CPLV, 8, CPL1, 16 / CPL1);                              \
+  } while (0)
   SEQ_DISPATCH_T(dt, {
     const bool vec = rows_by4<T>(q, Dk) && rows_by4<T>(k, Dk) &&
                      rows_by4<T>(z_lin, Dk) && rows_by4<T>(v, Dv) &&
                      rows_by4<T>(gate, Dv) && rows_by4<T>(out, Dv) &&
                      (uintptr_t)dt_bias.data_ptr() % 16 == 0 &&
                      (uintptr_t)state.data_ptr() % 16 == 0;
-    if (Dk <= 32) CDELTA_W(4, 2);
-    else if (Dk <= 64) CDELTA_W(8, 2);
-    else if (Dk <= 128) CDELTA_W(16, 2);
-    else if (Dk <= 256) CDELTA_W(32, 1);
-    else CDELTA(64, 1, 8);
+    if (Dk <= 32) CDELTA_W(4, 2, 4);
+    else if (Dk <= 64) CDELTA_W(8, 2, 4);
+    else if (Dk <= 128) CDELTA_W(16, 2, 4);
+    else if (Dk <= 256) CDELTA_W(32, 1, 1);
+    else CDELTA(64, 1, 8, 1, 8);
   });
 #undef CDELTA_W
 #undef CDELTA
