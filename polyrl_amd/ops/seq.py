@@ -1,11 +1,13 @@
 """Sequence-mixer ops for hybrid decoders: fp32-residual norms (plain and
 offset weights, fused joints, scaled branches, the gated layer-norm joint of
-parallel layers), the composed embedding (scaled row + hashed pair row +
-sinusoid), stateful causal convolutions, the generalised delta rule, gated
-linear attention, the selective state-space scan, the real-gated linear
-recurrence, windowed or causal latent attention with an optional softmax
-sink, grouped-query (window or causal; softmax or sigmoid weights) attention
-over paged K/V rows, and table-routed or router-chosen expert feed-forwards.
+parallel layers, the post-norm joint), the composed embedding (scaled row +
+hashed pair row + sinusoid), stateful causal convolutions, the generalised
+delta rule, the gated delta rule with per-channel decays, gated linear
+attention, the selective scans (per head and per channel), the real-gated
+linear recurrence, windowed or causal latent attention with an optional softmax
+sink, grouped-query (window, chunked or causal; softmax or sigmoid weights)
+attention over paged K/V rows, and table-routed or router-chosen expert
+feed-forwards.
 
 Same policy as the rest of ``polyrl_amd.ops``: on a HIP device the in-tree
 extension is REQUIRED (csrc/seq_*.hip, templated on the activation type:
