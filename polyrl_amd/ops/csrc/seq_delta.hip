@@ -46,12 +46,14 @@ struct CDeltaIn {
 
 // ONE: every sequence brings one row (tiles of one token, little LDS, so that
 // many blocks share a CU; with four columns per lane a wave reads and writes
-// whole 128-byte lines of the state, which is what such a step is bound by).  VEC: all rows allow loads of four numbers.
+// whole 128-byte lines of the state, which is what such a step is bound by).
+// VEC: all rows allow loads of four numbers.
 // Addresses beyond a tile's rows or a head's channels are clamped to its last
 // ones and the numbers dropped, so that the loads of a tile are one straight
 // run with nothing waiting between them.
 template <typename T, int RPL, int CPL, int NW, bool ONE, bool VEC>
-__global__ __launch_bounds__(64 * NW, ONE && RPL <= 8 ? 4 : 1) void channel_delta_kernel(
+__global__ __launch_bounds__(64 * NW, ONE && RPL <= 8 ? 4 : 1)
+void channel_delta_kernel(
     T* __restrict__ out, float* __restrict__ out32, const T* __restrict__ q,
     const T* __restrict__ k, const T* __restrict__ v,
     const T* __restrict__ bl, const T* __restrict__ zl,
