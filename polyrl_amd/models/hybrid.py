@@ -1,10 +1,11 @@
 """Configuration of hybrid decoders: a stack whose layers each pick one
-sequence mixer (recurrent, state-space, gated linear attention, a real-gated
-linear recurrence, latent attention, grouped-query attention, or two of
-them side by side) and one feed-forward (dense, table-routed experts, router-chosen experts, or none).
+sequence mixer (recurrent, state-space, gated linear attention, linear
+attention with a fixed decay, a real-gated linear recurrence, latent
+attention, grouped-query attention, or two of them side by side) and one feed-forward (dense, table-routed experts, router-chosen experts, or none).
 
 The Bizusun design is the first family described this way, Kuforax the
-second, Vurivik the third, Nasipel the fourth, Puvapel the fifth.
+second, Vurivik the third, Nasipel the fourth, Puvapel the fifth, Redirax
+the sixth.
 Everything that can differ between two models of a family is a field here and is read from
 the checkpoint's ``config.json``; constants that the design fixes (the decay
 constant of the delta rule, its key epsilon) are defaults of the mixer
@@ -63,12 +64,27 @@ class SelectiveScanSpec:
 @dataclass
 class ParallelMixerSpec:
     """Two mixers side by side on the same input:
-    ``left_scale * left(h) + right_scale * right(h)``."""
+    ``left_scale * left(h) + right_scale * right(h)``.  With ``out_norm``
+    each result is first RMS-normed over the model width with a weight of
+    its own (tensors 'left.out' / 'right.out'); one scale serves both."""
     left: object
     right: object
     left_scale: float = 1.0
     right_scale: float = 1.0
+    out_norm: bool = False
     kind: str = "parallel"
+
+
+@dataclass
+class LightningSpec:
+    """Linear attention with one fixed decay per head: q, k and v pass SiLU,
+    ``S <- decay S + k v^T``, ``o = S^T q``; the row of all heads is
+    RMS-normed together and multiplied by ``sigmoid(W_g h)``."""
+    heads: int
+    dim: int
+    vdim: int
+    decay: List[float]
+    kind: str = "lightning"
 
 
 @dataclass
@@ -159,7 +175,8 @@ class RopeSpec:
     ``factor`` > 1 switches on YaRN: pairs that turn fewer than
     ``slow`` times within ``original`` positions have their frequency divided
     by ``factor``, pairs that turn more than ``fast`` times keep it, a linear
-    ramp joins the two, and cos/sin are scaled by ``amp_slope*ln(factor)+1``."""
+    ramp joins the two, and cos/sin are scaled by ``amp_slope*ln(factor)+1``.
+    ``linear``: every frequency is divided by ``factor`` and nothing else."""
     dims: int
     base: float = 10000.0
     factor: float = 1.0
@@ -168,11 +185,14 @@ class RopeSpec:
     slow: float = 1.0
     amp_slope: float = 0.1
     interleaved: bool = False
+    linear: bool = False
 
     def inv_freq_and_amp(self):
         """(per-pair frequencies as Python floats, cos/sin amplitude)."""
         dims, half = self.dims, self.dims // 2
         f = [self.base ** (-2.0 * i / dims) for i in range(half)]
+        if self.linear:
+            return [x / self.factor for x in f], 1.0
         if self.factor == 1.0 or self.original <= 0:
             return f, 1.0
 
@@ -220,8 +240,9 @@ class WindowAttnSpec:
     head with one weight row shared by the heads, before the rotation
     (``head_norm``), attention confined to chunks of ``chunk`` positions
     counted from the sequence's start (``chunk`` > 0: key j is seen from p
-    when floor(j / chunk) = floor(p / chunk)), and a fixed sink of score 0,
-    i.e. one added to the softmax denominator (``unit_sink``)."""
+    when floor(j / chunk) = floor(p / chunk)), a fixed sink of score 0,
+    i.e. one added to the softmax denominator (``unit_sink``), and a bias on
+    the output projection (``o_bias``, tensor 'o.b')."""
     heads: int
     kv_heads: int
     dim: int
@@ -248,6 +269,7 @@ class WindowAttnSpec:
     head_norm: bool = False
     chunk: int = 0
     unit_sink: bool = False
+    o_bias: bool = False
     kind: str = "attention"
 
     def bucket_of_distance(self) -> List[int]:
@@ -280,15 +302,25 @@ class FFSpec:
     shared_ff: int = 0
     weight_eps: float = 1e-20
     # routed_moe: the router's scores are a softmax over the experts or each
-    # logit's own sigmoid; a group's score is the sum of its best
+    # logit's own sigmoid, or the logits themselves, the weights being the
+    # softmax over the chosen ones ("logits"); a group's score is the sum of its best
     # ``group_top`` choice scores; the normalised weights are multiplied by
     # ``route_scale``; experts are W_down gelu(W_up h) ("gelu") or
-    # W_down (silu(W_gate h) * W_up h) ("silu_gated")
+    # W_down (silu(W_gate h) * W_up h) ("silu_gated") or the gated form with
+    # the "clamped" activation below ("clamped_gated"); the shared expert has
+    # the same form with a limit of its own
     router_act: str = "softmax"
     group_top: int = 1
     route_scale: float = 1.0
     expert_act: str = "gelu"
-    # dense: "silu" is silu(gate) * up; "clamped" is g * sigmoid(slope * g)
+    shared_limit: float = 0.0
+    # routed_moe: the router's correction is a bias of its projection (tensor
+    # 'router.b' instead of 'correction'); the shared expert is multiplied by
+    # the sigmoid of one number per token (tensor 'shared.sg')
+    router_bias: bool = False
+    shared_gate: bool = False
+    # dense: "silu" is silu(gate) * up; "relu" is max(gate, 0) * up;
+    # "clamped" is g * sigmoid(slope * g)
     # * (u + shift) with g = min(gate, limit), u = clamp(up, -limit, limit)
     act: str = "silu"
     limit: float = 0.0
@@ -309,8 +341,11 @@ class BigramSpec:
 
 @dataclass
 class HybridLayerSpec:
+    """``weights_of``: the layer that owns this one's tensors (mixer,
+    feed-forward, norms); its cache rows and states are its own."""
     mixer: object
     ff: Optional[FFSpec]
+    weights_of: Optional[int] = None
 
 
 @dataclass
@@ -333,11 +368,17 @@ class HybridConfig:
     # weights and m = ``residual_mult``.  "parallel": both sublayers read
     # the same stream, x += mixer(norm1(x)) + ff(norm2(x)).  "postnorm":
     # sublayers read the stream itself, x += norm1(mixer(x)),
-    # x += norm2(ff(x)).
+    # x += norm2(ff(x)).  "streams": ``streams`` copies of the stream; a
+    # sublayer reads u = sum_s in[s] x_s through its norm and every copy
+    # becomes x_t <- sum_s mix[s, t] x_s + out[t] * y (tensors 'hc1.*',
+    # 'hc2.*'); the stack ends with their sum.
     layer_style: str = "canon"
     # "rms": x / sqrt(mean(x^2) + eps) * w.  "layer": (x - mean) /
-    # sqrt(var + eps) * w (no bias); parallel layers only.
+    # sqrt(var + eps) * w (no bias); parallel layers only.  "tanh":
+    # tanh(alpha * x) * w + b with a scalar alpha (tensors '<name>.alpha',
+    # '<name>.b'); streams layers only.
     norm_kind: str = "rms"
+    streams: int = 1
     # every sublayer's result is multiplied by sigmoid(W h + b) of the
     # sublayer's own input h (tensors 'rg1', 'rg1.b', 'rg2', 'rg2.b')
     gated_residual: bool = False
@@ -399,9 +440,12 @@ class HybridConfig:
         assert m.heads % m.kv_heads == 0 and m.window >= 1
         if m.rope is not None:
             assert m.rope.dims % 2 == 0 and m.rope.dims <= m.dim
-            if m.rope.interleaved:
-                raise ValueError(f"layer {li}: grouped-query "
-                                 "attention rotates halves")
+            if m.rope.interleaved and (
+                    m.qk_norm or m.head_norm or m.head_unit_norm or
+                    m.value_rope_base > 0 or m.values_from_keys):
+                raise ValueError(f"layer {li}: interleaved pairs do not "
+                                 "combine with query/key norms or rotated "
+                                 "or shared values")
         assert m.weights in ("softmax", "sigmoid")
         if m.weights == "sigmoid" and (m.sink or m.bias_far > 0):
             raise ValueError(f"layer {li}: a sink or a distance "
@@ -422,6 +466,12 @@ class HybridConfig:
         if m.unit_sink and (m.sink or m.weights == "sigmoid"):
             raise ValueError(f"layer {li}: one sink, softmax weights")
 
+    @staticmethod
+    def _check_lightning(m):
+        assert m.heads > 0 and m.dim > 0 and m.vdim > 0
+        if len(m.decay) != m.heads:
+            raise ValueError("linear attention: one decay per head")
+
     def validate(self):
         for li, L in enumerate(self.layers):
             m = L.mixer
@@ -441,7 +491,7 @@ class HybridConfig:
                 assert m.heads % m.kv_heads == 0 and m.conv >= 1
             if m.kind == "parallel":
                 for part in (m.left, m.right):
-                    if part.kind not in ("attention", "mamba"):
+                    if part.kind not in ("attention", "mamba", "lightning"):
                         raise ValueError(f"layer {li}: {part.kind} cannot "
                                          "be one of two mixers")
                     if getattr(part, "bias_far", 0) > 0:
@@ -449,8 +499,22 @@ class HybridConfig:
                                          "side-by-side mixers")
                     if part.kind == "attention":
                         self._check_attention(li, part)
-                    else:
+                    elif part.kind == "mamba":
                         assert part.inner > 0 and part.conv >= 1
+                    else:
+                        self._check_lightning(part)
+                if m.out_norm:
+                    if self.layer_style != "streams":
+                        raise ValueError(f"layer {li}: normed side-by-side "
+                                         "outputs are joined by the streams "
+                                         "style")
+                    assert m.left_scale == m.right_scale
+                elif any(getattr(p, "o_bias", False)
+                         for p in (m.left, m.right)):
+                    raise ValueError(f"layer {li}: an output bias in "
+                                     "side-by-side mixers needs out_norm")
+            if m.kind == "lightning":
+                self._check_lightning(m)
             if m.kind == "rglru":
                 assert m.width % m.blocks == 0 and m.conv >= 1
             if m.kind == "latent_attention":
@@ -463,8 +527,8 @@ class HybridConfig:
             if m.kind == "attention":
                 self._check_attention(li, m)
             if L.ff is not None and L.ff.kind == "dense":
-                assert L.ff.act in ("silu", "clamped")
-                assert L.ff.act == "silu" or L.ff.limit > 0
+                assert L.ff.act in ("silu", "relu", "clamped")
+                assert L.ff.act != "clamped" or L.ff.limit > 0
             if L.ff is not None and L.ff.kind == "moe":
                 assert 0 < L.ff.top <= L.ff.experts
             if L.ff is not None and L.ff.kind == "routed_moe":
@@ -473,10 +537,32 @@ class HybridConfig:
                 assert total % f.group_count == 0
                 assert 0 < f.group_keep <= f.group_count
                 assert 0 < f.top <= f.group_keep * (total // f.group_count)
-                assert f.router_act in ("softmax", "sigmoid")
-                assert f.expert_act in ("gelu", "silu_gated")
+                assert f.router_act in ("softmax", "sigmoid", "logits")
+                assert f.expert_act in ("gelu", "silu_gated",
+                                        "clamped_gated")
+                if f.expert_act == "clamped_gated":
+                    assert f.limit > 0 and (not f.shared_ff or
+                                            f.shared_limit > 0)
+                assert not f.shared_gate or f.shared_ff > 0
                 assert f.group_top >= 1
-        assert self.norm_kind == "rms" or self.layer_style == "parallel"
+            j = L.weights_of
+            if j is not None:
+                if not 0 <= j < len(self.layers) or \
+                        self.layers[j].weights_of is not None:
+                    raise ValueError(f"layer {li}: weights_of must name a "
+                                     "layer with tensors of its own")
+                own = self.layers[j]
+                if (L.mixer, L.ff) != (own.mixer, own.ff):
+                    raise ValueError(f"layer {li} differs from layer {j}, "
+                                     "whose weights it uses")
+        if self.layer_style == "streams":
+            assert self.streams >= 1 and self.norm_kind == "tanh"
+            if any(L.ff is not None and L.ff.kind == "moe"
+                   for L in self.layers):
+                raise ValueError("table-routed experts write one stream")
+        else:
+            assert self.streams == 1 and self.norm_kind != "tanh"
+        assert self.norm_kind != "layer" or self.layer_style == "parallel"
         assert not self.gated_residual or self.layer_style == "parallel"
         if (self.loop_reinject or self.loop_step) and not self.loop:
             raise ValueError("pass inputs need a looped span")
@@ -1119,6 +1205,150 @@ def puvapel_preset(width: int, layers: int, vocab: int = 32000,
                         norm_offset=1.0, logit_softcap=30.0).validate()
 
 
+def _owner_of(layers: List[dict], li: int) -> Optional[int]:
+    """The layer at the end of a chain of 'weights_of' entries."""
+    j, seen = layers[li].get("weights_of"), {li}
+    while j is not None and layers[j].get("weights_of") is not None:
+        if j in seen:
+            raise ValueError(f"layer {li}: weights_of runs in a circle")
+        seen.add(j)
+        j = layers[j]["weights_of"]
+    return None if j is None else int(j)
+
+
+def _redirax_mixer_from_json(kind: str, m: dict) -> ParallelMixerSpec:
+    """Redirax's one mixer: causal grouped-query attention with biases and
+    interleaved, linearly scaled rotation beside linear attention with fixed
+    decays; half the sum of the two normed results."""
+    if kind != "parallel":
+        raise ValueError(f"unknown mixer type {kind!r}")
+    a, r = m["left"], m["right"]
+    rope = _rope_from_json(a.get("rot"), interleaved=True)
+    if rope is not None:
+        rope.linear = True
+    return ParallelMixerSpec(
+        left=WindowAttnSpec(
+            heads=int(a["heads"]), kv_heads=int(a["kv_heads"]),
+            dim=int(a["dim"]), vdim=int(a["vdim"]), window=UNBOUNDED,
+            scale=float(a["scale"]), rope=rope, qkv_bias=True, o_bias=True),
+        right=LightningSpec(heads=int(r["heads"]), dim=int(r["dim"]),
+                            vdim=int(r["vdim"]),
+                            decay=[float(x) for x in r["decay"]]),
+        left_scale=0.5, right_scale=0.5, out_norm=True)
+
+
+def _redirax_ff_from_json(f: Optional[dict]) -> Optional[FFSpec]:
+    if f is None:
+        return None
+    if f["kind"] == "dense":
+        return FFSpec(kind="dense", ff=int(f["ff"]), act="relu")
+    if f["kind"] == "moe":
+        s = f.get("shared") or {}
+        return FFSpec(kind="routed_moe", ff=int(f["expert"]["ff"]),
+                      experts=int(f["router"]["experts"]),
+                      top=int(f["router"]["top"]), weight_eps=0.0,
+                      router_act="logits", router_bias=True,
+                      expert_act="clamped_gated",
+                      limit=float(f["expert"]["limit"]),
+                      shared_ff=int(s.get("ff", 0)),
+                      shared_limit=float(s.get("limit", 0.0)),
+                      shared_gate=bool(s))
+    raise ValueError(f"unknown feed-forward kind {f['kind']!r}")
+
+
+def redirax_config_from_json(d: dict) -> HybridConfig:
+    """Read a Redirax ``config.json`` (already parsed)."""
+    layers = [HybridLayerSpec(_redirax_mixer_from_json(L["type"], L["mixer"]),
+                              _redirax_ff_from_json(L.get("mlp")),
+                              weights_of=_owner_of(d["layers"], li))
+              for li, L in enumerate(d["layers"])]
+    return HybridConfig(
+        arch="redirax", vocab_size=int(d["vocab"]),
+        hidden_size=int(d["width"]), layers=layers,
+        norm_eps=float(d["norm"]["eps"]), canon_taps=1, token_side_dim=0,
+        layer_style="streams", norm_kind="tanh",
+        streams=int(d.get("streams", 1)),
+        logit_softcap=float(d.get("logit_softcap") or 0.0)).validate()
+
+
+def redirax_config_to_json(cfg: HybridConfig) -> dict:
+    """Inverse of :func:`redirax_config_from_json` (checkpoint export)."""
+    layers = []
+    for L in cfg.layers:
+        a, r, f = L.mixer.left, L.mixer.right, L.ff
+        left = {"heads": a.heads, "kv_heads": a.kv_heads, "dim": a.dim,
+                "vdim": a.vdim, "scale": a.scale}
+        if a.rope is not None:
+            left["rot"] = {"base": a.rope.base, "dims": a.rope.dims,
+                           "scaling": {"factor": a.rope.factor}}
+        fj = None
+        if f is not None and f.kind == "dense":
+            fj = {"kind": "dense", "ff": f.ff}
+        elif f is not None:
+            fj = {"kind": "moe", "expert": {"ff": f.ff, "limit": f.limit},
+                  "router": {"experts": f.experts, "top": f.top}}
+            if f.shared_ff:
+                fj["shared"] = {"ff": f.shared_ff, "limit": f.shared_limit}
+        out = {"type": "parallel", "mixer": {
+            "left": left, "right": {"heads": r.heads, "dim": r.dim,
+                                    "vdim": r.vdim, "decay": list(r.decay)}},
+               "mlp": fj}
+        if L.weights_of is not None:
+            out["weights_of"] = L.weights_of
+        layers.append(out)
+    return {"architecture": "Redirax", "vocab": cfg.vocab_size,
+            "width": cfg.hidden_size, "layers": layers,
+            "norm": {"eps": cfg.norm_eps}, "streams": cfg.streams,
+            "logit_softcap": cfg.logit_softcap}
+
+
+def redirax_preset(width: int, layers: int, vocab: int = 32000,
+                   heads: int = 16, kv_heads: int = 4, right_heads: int = 0,
+                   experts: int = 16, top: int = 2, expert_ff: int = 0,
+                   shared_ff: int = 0, dense_ff: int = 0, streams: int = 2,
+                   shared_from: Optional[int] = None) -> HybridConfig:
+    """A Redirax stack of realistic layer sizes (random weights): the first
+    layer is dense, the others have routed clamped experts with a gated
+    shared expert; layers from ``shared_from`` on use the weights of layer
+    ``shared_from - 1``.  The linear attention's decays run from 0.9 to
+    0.999 over its heads."""
+    hd = width // heads
+    rh = right_heads or heads
+    expert_ff = expert_ff or max(64, width // 64 * 64)
+    out = []
+    for li in range(layers):
+        mixer = ParallelMixerSpec(
+            left=WindowAttnSpec(
+                heads=heads, kv_heads=kv_heads, dim=hd, vdim=hd,
+                window=UNBOUNDED, scale=1.0 / math.sqrt(hd),
+                rope=RopeSpec(dims=hd, base=10000.0, factor=2.0,
+                              interleaved=True, linear=True),
+                qkv_bias=True, o_bias=True),
+            right=LightningSpec(
+                heads=rh, dim=width // rh, vdim=width // rh,
+                decay=[1.0 - 0.1 * 0.01 ** (i / max(rh - 1, 1))
+                       for i in range(rh)]),
+            left_scale=0.5, right_scale=0.5, out_norm=True)
+        if li == 0:
+            ff = FFSpec("dense", dense_ff or top * expert_ff + shared_ff,
+                        act="relu")
+        else:
+            ff = FFSpec("routed_moe", expert_ff, experts, top, weight_eps=0.0,
+                        router_act="logits", router_bias=True,
+                        expert_act="clamped_gated", limit=7.0,
+                        shared_ff=shared_ff, shared_limit=5.0,
+                        shared_gate=shared_ff > 0)
+        own = None
+        if shared_from is not None and li >= shared_from:
+            own = shared_from - 1
+        out.append(HybridLayerSpec(mixer, ff, weights_of=own))
+    return HybridConfig(arch="redirax", vocab_size=vocab, hidden_size=width,
+                        layers=out, norm_eps=1e-5, canon_taps=1,
+                        token_side_dim=0, layer_style="streams",
+                        norm_kind="tanh", streams=streams,
+                        logit_softcap=30.0).validate()
+
+
 def read_config_dir(path: str):
     """Model config from a checkpoint folder's ``config.json``.  The
     ``architecture`` key names the family; HF-style folders
@@ -1136,6 +1366,8 @@ def read_config_dir(path: str):
         return nasipel_config_from_json(d)
     if arch == "Puvapel":
         return puvapel_config_from_json(d)
+    if arch == "Redirax":
+        return redirax_config_from_json(d)
     mt = d.get("model_type")
     if mt in ("llama", "qwen2"):
         from .registry import DecoderConfig

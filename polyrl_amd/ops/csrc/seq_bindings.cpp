@@ -124,20 +124,53 @@ void seq_gqa_window_attention_mfma(
     int64_t q_temp_every, double softcap, torch::Tensor head_bias,
     bool sigmoid_weights, torch::Tensor v_inv_freq, int64_t chunk,
     double out_scale);
+void seq_gqa_prepare_plain(torch::Tensor q_out, torch::Tensor q,
+                           torch::Tensor k, torch::Tensor v,
+                           torch::Tensor bias, torch::Tensor inv_freq,
+                           double amp, torch::Tensor positions,
+                           torch::Tensor cache, torch::Tensor slot_mapping,
+                           int64_t H, int64_t G, int64_t D, int64_t Dv,
+                           bool interleaved);
+void seq_lightning_scan(torch::Tensor out, torch::Tensor q, torch::Tensor k,
+                        torch::Tensor v, torch::Tensor decay,
+                        torch::Tensor state, torch::Tensor cu_q,
+                        torch::Tensor state_slot, int64_t max_rows);
+void seq_streams_open(torch::Tensor xs, torch::Tensor h, torch::Tensor table,
+                      torch::Tensor tokens, torch::Tensor w_in,
+                      torch::Tensor alpha, torch::Tensor w, torch::Tensor b);
+void seq_streams_join(torch::Tensor out, torch::Tensor xs, torch::Tensor a,
+                      torch::Tensor bias_a, torch::Tensor wa, torch::Tensor b,
+                      torch::Tensor bias_b, torch::Tensor wb, double scale,
+                      double eps, torch::Tensor w_mix, torch::Tensor w_out,
+                      torch::Tensor w_in, torch::Tensor alpha,
+                      torch::Tensor nw, torch::Tensor nb);
+void seq_tanh_norm(torch::Tensor out, torch::Tensor x, torch::Tensor alpha,
+                   torch::Tensor w, torch::Tensor b);
 void seq_moe_route(torch::Tensor idx, torch::Tensor w, torch::Tensor logits,
                    torch::Tensor correction, int64_t groups, int64_t keep,
                    int64_t act, int64_t group_top);
 void seq_moe_routed_ffn(torch::Tensor y, torch::Tensor act, torch::Tensor h,
                         torch::Tensor idx, torch::Tensor w_up,
-                        torch::Tensor w_down, bool gated);
+                        torch::Tensor w_down, bool gated, double limit,
+                        double slope, double shift);
 void seq_moe_weighted_combine(torch::Tensor out, torch::Tensor ys,
                               torch::Tensor idx, torch::Tensor w,
                               torch::Tensor h, torch::Tensor shared,
-                              int64_t E, double weight_eps, double scale);
+                              int64_t E, double weight_eps, double scale,
+                              torch::Tensor shared_gate);
 
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("seq_gqa_prepare_store", &seq_gqa_prepare_store,
         "whole-row q/k norm + partial rotation + K/V cache rows");
+  m.def("seq_gqa_prepare_plain", &seq_gqa_prepare_plain,
+        "projection biases + rotation + K/V cache rows, no norms");
+  m.def("seq_lightning_scan", &seq_lightning_scan,
+        "linear attention with fixed decays (fp32 state, in place)");
+  m.def("seq_streams_open", &seq_streams_open,
+        "residual streams from embedding rows + first tanh norm");
+  m.def("seq_streams_join", &seq_streams_join,
+        "residual streams mixed anew with a sublayer's result + tanh norm");
+  m.def("seq_tanh_norm", &seq_tanh_norm, "tanh(alpha x) w + b");
   m.def("seq_gqa_window_attention", &seq_gqa_window_attention,
         "grouped-query window attention over paged K/V rows (any dtype)");
   m.def("seq_gqa_window_attention_mfma", &seq_gqa_window_attention_mfma,
@@ -175,7 +208,7 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
         "RoPE (halves or interleaved pairs) on a slice of each head, in place");
   m.def("seq_latent_kv_store", &seq_latent_kv_store,
         "norm + rotate + write latent cache rows");
-  m.def("seq_act_mul", &seq_act_mul, "silu*b / sigmoid*b / tanh / gelu / clamped gated unit");
+  m.def("seq_act_mul", &seq_act_mul, "silu*b / sigmoid*b / tanh / gelu / clamped gated unit / relu*b");
   m.def("seq_gelu_mul_rows", &seq_gelu_mul_rows,
         "gelu_tanh(gate) * table rows gathered by token");
   m.def("seq_moe_combine", &seq_moe_combine,

@@ -27,6 +27,8 @@
 // head): every query and key head is divided by its own root mean square
 // AFTER the rotation (no weight), and every value head is rotated over all
 // its entries by its position (pairs (m, m + Dv/2)) before it is cached.
+// gqa_prepare_plain_kernel: biases on the projections and a rotation of
+// neighbouring pairs (2i, 2i + 1) or of halves, without norms.
 // Further options of the attention kernels: scores capped as
 // cap * tanh(score / cap), a number per head added to the capped score, and
 // weights sigmoid(score) per visible key with no normalisation over the
@@ -318,6 +320,133 @@ __global__ __launch_bounds__(256) void gqa_prepare_headnorm4_kernel(
   }
 }
 
+// No norms: one block per token adds the projection biases, turns the first
+// 2*half entries of every query and key head, pairs (2i, 2i + 1) or
+// (i, i + half), and writes queries and cache row.  The token's cosines and
+// sines are taken once.  VEC: four consecutive numbers per thread and step.
+template <typename T, bool VEC>
+__global__ __launch_bounds__(256) void gqa_prepare_plain_kernel(
+    T* __restrict__ q_out, const T* __restrict__ q, long ldq,
+    const T* __restrict__ k, long ldk, const T* __restrict__ v, long ldv,
+    const float* __restrict__ bias, const float* __restrict__ inv_freq,
+    int half, float amp, const int* __restrict__ positions,
+    T* __restrict__ cache, const int* __restrict__ slot_mapping, int H, int G,
+    int D, int Dv, bool interleaved) {
+  extern __shared__ float cs[];         // [half cosines | half sines]
+  constexpr int E = VEC ? 4 : 1;
+  const long n = blockIdx.x;
+  const float pos = (float)positions[n];
+  for (int i = threadIdx.x; i < half; i += 256) {
+    const float ang = pos * inv_freq[i];
+    cs[i] = cosf(ang) * amp;
+    cs[half + i] = sinf(ang) * amp;
+  }
+  __syncthreads();
+  const int nq = H * D, nk = G * D, nv = G * Dv;
+  T* crow = cache + (long)slot_mapping[n] * (nk + nv);
+  for (int u = threadIdx.x * E; u < nq + nk + nv; u += 256 * E) {
+    const bool isq = u < nq, isv = u >= nq + nk;
+    const T* src = isq ? q + n * ldq : isv ? v + n * ldv : k + n * ldk;
+    const float* bs = bias ? bias + (isq ? 0 : isv ? nq + nk : nq) : nullptr;
+    const int at = isq ? u : isv ? u - nq - nk : u - nq;
+    T* dst = isq ? q_out + n * nq + at : crow + (isv ? nk + at : at);
+    auto get = [&](int i) {             // E numbers from place i, with bias
+      f32x4v x = load4(src + i, E, VEC);
+      if (bs) {
+        const f32x4v c = load4(bs + i, E, VEC);
+#pragma unroll
+        for (int e = 0; e < E; ++e) x.v[e] += c.v[e];
+      }
+      return x;
+    };
+    f32x4v x = get(at);
+    const int d = isv ? 0 : at % D;
+    if (!isv && d < 2 * half) {
+      if (!interleaved) {
+        const bool lo = d < half;
+        const f32x4v y = get(lo ? at + half : at - half);
+        const float sign = lo ? -1.f : 1.f;
+        const int i = lo ? d : d - half;
+#pragma unroll
+        for (int e = 0; e < E; ++e)
+          x.v[e] = x.v[e] * cs[i + e] + sign * y.v[e] * cs[half + i + e];
+      } else if (VEC) {
+#pragma unroll
+        for (int e = 0; e < 4; e += 2) {
+          const int i = (d + e) / 2;
+          if (i < half) {
+            const float a = x.v[e], b = x.v[e + 1];
+            x.v[e] = a * cs[i] - b * cs[half + i];
+            x.v[e + 1] = b * cs[i] + a * cs[half + i];
+          }
+        }
+      } else {
+        const f32x4v y = get(d & 1 ? at - 1 : at + 1);
+        const float sign = d & 1 ? 1.f : -1.f;
+        x.v[0] = x.v[0] * cs[d / 2] + sign * y.v[0] * cs[half + d / 2];
+      }
+    }
+    store4(dst, x, E, VEC);
+  }
+}
+
+void seq_gqa_prepare_plain(torch::Tensor q_out, torch::Tensor q,
+                           torch::Tensor k, torch::Tensor v,
+                           torch::Tensor bias, torch::Tensor inv_freq,
+                           double amp, torch::Tensor positions,
+                           torch::Tensor cache, torch::Tensor slot_mapping,
+                           int64_t H, int64_t G, int64_t D, int64_t Dv,
+                           bool interleaved) {
+  CHECK_ROWS(q); CHECK_ROWS(k); CHECK_ROWS(v);
+  CHECK_I32(positions); CHECK_I32(slot_mapping);
+  const long N = q.size(0);
+  const int half = inv_freq.defined() ? (int)inv_freq.numel() : 0;
+  const bool has_b = bias.defined() && bias.numel() > 0;
+  TORCH_CHECK(H > 0 && G > 0 && H % G == 0 && D > 0 && Dv > 0);
+  TORCH_CHECK(q.size(1) == H * D && k.size(0) == N && k.size(1) == G * D &&
+              v.size(0) == N && v.size(1) == G * Dv);
+  TORCH_CHECK(2 * half <= D, "rotated entries exceed the head size");
+  auto ty = q.scalar_type();
+  TORCH_CHECK(k.scalar_type() == ty && v.scalar_type() == ty &&
+              cache.scalar_type() == ty && q_out.scalar_type() == ty);
+  if (half) CHECK_F32(inv_freq);
+  if (has_b) {
+    CHECK_F32(bias);
+    TORCH_CHECK(bias.numel() == (H + G) * D + G * Dv, "projection biases");
+  }
+  TORCH_CHECK(cache.is_cuda() && cache.is_contiguous() && cache.dim() == 3 &&
+              cache.size(2) == G * (D + Dv), "cache row must be G*(D+Dv)");
+  TORCH_CHECK(q_out.is_cuda() && q_out.is_contiguous() &&
+              q_out.numel() == N * H * D);
+  TORCH_CHECK(positions.numel() == N && slot_mapping.numel() == N);
+  if (N == 0) return;
+  auto stream = at::hip::getCurrentHIPStream();
+  const size_t bytes = 2 * half * sizeof(float);
+  TORCH_CHECK(bytes <= 60 * 1024, "rotated entries above 15360");
+  SEQ_DISPATCH_T(ty, {
+    const auto fits = [](const torch::Tensor& t, size_t b) {
+      return (uintptr_t)t.data_ptr() % b == 0; };
+    const bool vec = D % 4 == 0 && Dv % 4 == 0 &&
+                     (interleaved || half % 4 == 0) && rows_by4<T>(q, D) &&
+                     rows_by4<T>(k, D) && rows_by4<T>(v, Dv) &&
+                     fits(q_out, 4 * sizeof(T)) && fits(cache, 4 * sizeof(T)) &&
+                     (!has_b || fits(bias, 16));
+#define PLAIN_LAUNCH(VECV)                                                    \
+    hipLaunchKernelGGL((gqa_prepare_plain_kernel<T, VECV>), dim3(N),          \
+        dim3(256), bytes, stream, (T*)q_out.data_ptr(),                       \
+        (const T*)q.data_ptr(), q.stride(0), (const T*)k.data_ptr(),          \
+        k.stride(0), (const T*)v.data_ptr(), v.stride(0),                     \
+        has_b ? bias.data_ptr<float>() : nullptr,                             \
+        half ? inv_freq.data_ptr<float>() : nullptr, half, (float)amp,        \
+        positions.data_ptr<int>(), (T*)cache.data_ptr(),                      \
+        slot_mapping.data_ptr<int>(), (int)H, (int)G, (int)D, (int)Dv,        \
+        interleaved)
+    if (vec) PLAIN_LAUNCH(true);
+    else PLAIN_LAUNCH(false);
+  });
+  HIP_CHECK_KERNEL();
+}
+
 #define PREP4(LPHV)                                                           \
   hipLaunchKernelGGL((gqa_prepare_headnorm4_kernel<T, LPHV>), grid,           \
       dim3(256), 0, stream, (T*)q_out.data_ptr(), (const T*)q.data_ptr(),     \
@@ -518,11 +647,11 @@ struct Vec16<float> {
 // their key/value group's rows in cache when H/G >= 4).  Keys are walked 64
 // at a time in two phases: lane = key for the scores (each lane reads its
 // key row against the query in LDS), then lane = value entry for the
-// weighted sum (weights and row numbers from LDS).  When a value row is
-// ``lpr`` 16-byte pieces with lpr a power of two, lpr lanes read one row and
-// the wave reads 64/lpr rows per load; the lane groups' partial sums meet in
-// a shuffle reduction at the end.  Otherwise (lpr = 0) the wave reads one
-// value row per key.  The waves never meet at a block barrier.
+// weighted sum (weights and row numbers from LDS).  When a value row is made
+// of at most 64 16-byte pieces, ``lpr`` lanes (their number rounded up to a
+// power of two) read one row and the wave reads 64/lpr rows per load; the
+// lane groups' partial sums meet in a shuffle reduction at the end.
+// Otherwise (lpr = 0) the wave reads one value row per key.  The waves never meet at a block barrier.
 template <typename T, int NCH>
 __global__ __launch_bounds__(256) void gqa_attn_kernel(
     T* __restrict__ out,                // (N, H*Dv), row stride ldo
@@ -605,7 +734,7 @@ __global__ __launch_bounds__(256) void gqa_attn_kernel(
 #pragma unroll 4
       for (int jj0 = 0; jj0 < cntk; jj0 += kper) {
         const int jj = jj0 + kgrp;
-        if (jj < cntk) {
+        if (jj < cntk && dcol < Dv) {
           const float pj = ps[jj];
           float vv[EPL];
           Vec16<T>::load(cache + (long)ss[jj] * row + voff + dcol, vv);
@@ -635,7 +764,7 @@ __global__ __launch_bounds__(256) void gqa_attn_kernel(
     for (int k = 0; k < EPL; ++k)
       for (int off = lpr; off < 64; off <<= 1)
         ov[k] += __shfl_xor(ov[k], off, WAVE_SIZE);
-    if (lane < lpr) {
+    if (lane < lpr && dcol < Dv) {
 #pragma unroll
       for (int k = 0; k < EPL; ++k) {
         if (out32) out32[(n * H + h) * Dv + dcol + k] = ov[k] * inv;
@@ -759,9 +888,10 @@ void seq_gqa_window_attention(torch::Tensor out, torch::Tensor q,
   // 16-byte row loads need every head's keys to start on a 16-byte border
   const int per16 = q.scalar_type() == torch::kBFloat16 ? 8 : 4;
   const bool vec = D % per16 == 0 && Dv % per16 == 0;
-  // lanes per value row of 16-byte pieces, when that is a power of two <= 64
-  int lpr = vec ? (int)(Dv / per16) : 0;
-  if (lpr > 64 || (lpr & (lpr - 1))) lpr = 0;
+  // lanes per value row of 16-byte pieces: a power of two <= 64
+  int lpr = 0;
+  if (vec && Dv / per16 <= 64)
+    for (lpr = 1; lpr < Dv / per16; lpr <<= 1) {}
   auto stream = at::hip::getCurrentHIPStream();
   SEQ_DISPATCH_T(q.scalar_type(), {
     switch (nch) {

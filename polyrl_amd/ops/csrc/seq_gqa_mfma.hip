@@ -21,7 +21,8 @@
 // fp32 into a separate buffer for the pass that turns rotated values back.
 // The next tiles are fetched into registers while the current ones are
 // multiplied.
-// K-tile bytes are XOR-swizzled by row inside each 64-byte chunk.
+// K-tile bytes are XOR-swizzled by row inside each 64-byte chunk.  Key and
+// value head sizes are apart (KS and KV chunks of 32), up to 256 each.
 //
 // Grid: one dimension.  Workgroups go to the 8 XCDs in turn (id mod 8), each
 // with an L2 of its own, so the id is taken apart as XCD = id % 8 and, inside
@@ -58,7 +59,7 @@ DEV_INLINE int gtile_off(int row, int byte_col) {
   return row * (KS * 64) + (byte_col ^ ((row & 3) << 4));
 }
 
-template <int KS>
+template <int KS, int KV>
 __global__ __launch_bounds__(256) void gqa_attn_mfma_kernel(
     bf16_t* __restrict__ out,            // (N, H*Dv), row stride ldo
     const bf16_t* __restrict__ q,        // (N, H*D)
@@ -73,10 +74,9 @@ __global__ __launch_bounds__(256) void gqa_attn_mfma_kernel(
     const float* __restrict__ sink, float qt_coef, int qt_every, float cap,
     const float* __restrict__ hbias, bool sigm, float* __restrict__ out32,
     int chunk, long ldo, float out_scale) {
-  constexpr int DKP = KS * 32;           // padded head size in LDS
-  constexpr int NVT = KS * 2;            // 16-wide output tiles
-  __shared__ __attribute__((aligned(16))) bf16_t Ks[GKV * DKP];
-  __shared__ __attribute__((aligned(16))) bf16_t Vs[GKV * DKP];
+  constexpr int NVT = KV * 2;            // 16-wide output tiles
+  __shared__ __attribute__((aligned(16))) bf16_t Ks[GKV * KS * 32];
+  __shared__ __attribute__((aligned(16))) bf16_t Vs[GKV * KV * 32];
   __shared__ __attribute__((aligned(16))) bf16_t Ps[4][16 * GKV];
   __shared__ float rel_s[GQA_MAX_REL];
 
@@ -157,25 +157,48 @@ __global__ __launch_bounds__(256) void gqa_attn_mfma_kernel(
   auto tile_t0 = [&](int ti) { return ti < nkt ? ti * GKV : kmin + (ti - nkt) * GKV; };
   auto tile_jmax = [&](int ti) { return ti < nkt ? nk - 1 : pmax; };
 
-  constexpr int NV = (GKV * KS * 4 + 255) / 256;
-  i32x4_t prek[NV], prev[NV];
+  constexpr int NK = (GKV * KS * 4 + 255) / 256;
+  constexpr int NV = (GKV * KV * 4 + 255) / 256;
+  i32x4_t prek[NK], prev[NV];
   auto fetch = [&](int ti) {
     const int t0 = tile_t0(ti), jmax = tile_jmax(ti);
+    const i32x4_t z = {0, 0, 0, 0};
+    auto row_of = [&](int j) {
+      return cache + ((long)ptab[j / page_size] * page_size + j % page_size) * row;
+    };
+    if (KS == KV) {                      // a thread's key and value rows agree
+#pragma unroll
+      for (int i = 0; i < NK; ++i) {
+        const int v = threadIdx.x + i * 256;
+        const int col = (v % (KS * 4)) * 8;
+        const int j = t0 + v / (KS * 4);
+        prek[i] = z;
+        prev[i] = z;
+        if (v < GKV * KS * 4 && j <= jmax) {
+          const bf16_t* base = row_of(j);
+          if (col < D) prek[i] = *reinterpret_cast<const i32x4_t*>(base + koff + col);
+          if (col < Dv) prev[i] = *reinterpret_cast<const i32x4_t*>(base + voff + col);
+        }
+      }
+      return;
+    }
+#pragma unroll
+    for (int i = 0; i < NK; ++i) {
+      const int v = threadIdx.x + i * 256;
+      const int col = (v % (KS * 4)) * 8;
+      const int j = t0 + v / (KS * 4);
+      prek[i] = z;
+      if (v < GKV * KS * 4 && j <= jmax && col < D)
+        prek[i] = *reinterpret_cast<const i32x4_t*>(row_of(j) + koff + col);
+    }
 #pragma unroll
     for (int i = 0; i < NV; ++i) {
       const int v = threadIdx.x + i * 256;
-      const int kr = v / (KS * 4);
-      const int col = (v % (KS * 4)) * 8;
-      const int j = t0 + kr;
-      const i32x4_t z = {0, 0, 0, 0};
-      prek[i] = z;
+      const int col = (v % (KV * 4)) * 8;
+      const int j = t0 + v / (KV * 4);
       prev[i] = z;
-      if (v < GKV * KS * 4 && j <= jmax) {
-        const long slot = (long)ptab[j / page_size] * page_size + j % page_size;
-        const bf16_t* base = cache + slot * row;
-        if (col < D) prek[i] = *reinterpret_cast<const i32x4_t*>(base + koff + col);
-        if (col < Dv) prev[i] = *reinterpret_cast<const i32x4_t*>(base + voff + col);
-      }
+      if (v < GKV * KV * 4 && j <= jmax && col < Dv)
+        prev[i] = *reinterpret_cast<const i32x4_t*>(row_of(j) + voff + col);
     }
   };
   const int ntiles = nkt + nwt;
@@ -185,16 +208,20 @@ __global__ __launch_bounds__(256) void gqa_attn_mfma_kernel(
     const int t0 = tile_t0(ti), jmax = tile_jmax(ti);
     // ---- registers -> LDS tiles, then request the next tiles ------------
 #pragma unroll
+    for (int i = 0; i < NK; ++i) {
+      const int v = threadIdx.x + i * 256;
+      if (v < GKV * KS * 4)
+        *reinterpret_cast<i32x4_t*>(
+            reinterpret_cast<char*>(Ks) +
+            gtile_off<KS>(v / (KS * 4), (v % (KS * 4)) * 16)) = prek[i];
+    }
+#pragma unroll
     for (int i = 0; i < NV; ++i) {
       const int v = threadIdx.x + i * 256;
-      if (v < GKV * KS * 4) {
-        const int kr = v / (KS * 4);
-        const int col = (v % (KS * 4)) * 8;
-        *reinterpret_cast<i32x4_t*>(reinterpret_cast<char*>(Ks) +
-                                    gtile_off<KS>(kr, col * 2)) = prek[i];
-        *reinterpret_cast<i32x4_t*>(reinterpret_cast<char*>(Vs) +
-                                    gtile_off<KS>(kr, col * 2)) = prev[i];
-      }
+      if (v < GKV * KV * 4)
+        *reinterpret_cast<i32x4_t*>(
+            reinterpret_cast<char*>(Vs) +
+            gtile_off<KV>(v / (KV * 4), (v % (KV * 4)) * 16)) = prev[i];
     }
     __syncthreads();
     if (ti + 1 < ntiles) fetch(ti + 1);
@@ -282,7 +309,7 @@ __global__ __launch_bounds__(256) void gqa_attn_mfma_kernel(
         for (int j = 0; j < 8; ++j)
           bv[j] = *reinterpret_cast<const __bf16*>(
               reinterpret_cast<const char*>(Vs) +
-              gtile_off<KS>(lhi * 8 + j, d2));
+              gtile_off<KV>(lhi * 8 + j, d2));
         o_acc[nt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pa, bv, o_acc[nt],
                                                             0, 0, 0);
       }
@@ -334,8 +361,9 @@ void seq_rotate_back_heads(torch::Tensor out, torch::Tensor x,
                            torch::Tensor inv_freq, torch::Tensor positions,
                            torch::Tensor gate, int64_t H);
 
-#define GQA_MFMA_LAUNCH(KSV)                                                  \
-  hipLaunchKernelGGL((gqa_attn_mfma_kernel<KSV>), grid, dim3(256), 0, stream, \
+#define GQA_MFMA_LAUNCH(KSV, KVV)                                             \
+  hipLaunchKernelGGL((gqa_attn_mfma_kernel<KSV, KVV>), grid, dim3(256), 0,    \
+      stream,                                                                 \
       (bf16_t*)out.data_ptr(), (const bf16_t*)q.data_ptr(),                   \
       (const bf16_t*)cache.data_ptr(), page_table.data_ptr<int>(),            \
       (int)page_table.size(1), seq_of_tok.data_ptr<int>(),                    \
@@ -370,8 +398,9 @@ void seq_gqa_window_attention_mfma(
   TORCH_CHECK(tile_n0.numel() == tile_cnt.numel());
   const bool has_rel = rel.defined() && rel.numel() > 0;
   const bool has_gate = gate.defined() && gate.numel() > 0;
-  const int ks = (int)((std::max(D, Dv) + 31) / 32);
-  if (q.scalar_type() != torch::kBFloat16 || D % 8 || Dv % 8 || ks > 4 ||
+  const int ks = (int)((D + 31) / 32), kv = (int)((Dv + 31) / 32);
+  if (q.scalar_type() != torch::kBFloat16 || D % 8 || Dv % 8 ||
+      std::max(ks, kv) > 8 ||
       (has_rel && rel.size(0) > GQA_MAX_REL)) {
     seq_gqa_window_attention(out, q, cache, page_table, seq_of_tok, positions,
                              H, G, D, Dv, window, keep_first, rel,
@@ -403,11 +432,18 @@ void seq_gqa_window_attention_mfma(
   TORCH_CHECK(rounds * GQA_XCDS * (H / G) < (1L << 31), "grid too large");
   const dim3 grid((unsigned)(rounds * GQA_XCDS * (H / G)));
   auto stream = at::hip::getCurrentHIPStream();
-  switch (ks) {
-    case 1: GQA_MFMA_LAUNCH(1); break;
-    case 2: GQA_MFMA_LAUNCH(2); break;
-    case 3: GQA_MFMA_LAUNCH(3); break;
-    default: GQA_MFMA_LAUNCH(4); break;
+  switch (std::max(ks, kv)) {
+    case 1: GQA_MFMA_LAUNCH(1, 1); break;
+    case 2: GQA_MFMA_LAUNCH(2, 2); break;
+    case 3: GQA_MFMA_LAUNCH(3, 3); break;
+    case 4: GQA_MFMA_LAUNCH(4, 4); break;
+    case 5: case 6:
+      if (ks <= 3) GQA_MFMA_LAUNCH(3, 6);
+      else GQA_MFMA_LAUNCH(6, 6);
+      break;
+    default:
+      if (ks <= 4) GQA_MFMA_LAUNCH(4, 8);
+      else GQA_MFMA_LAUNCH(8, 8);
   }
   HIP_CHECK_KERNEL();
   if (v_rot) seq_rotate_back_heads(out, sums, v_inv_freq, positions, gate, H);

@@ -12,6 +12,8 @@
 //
 //   ACT 1 : act[slot, j] = silu(x_t . Wg[e][j]) * (x_t . Wu[e][j])   (gated)
 //   ACT 2 : act[slot, j] = gelu_erf(x_t . Wu[e][j])                  (plain)
+//   ACT 3 : act[slot, j] = g * sigmoid(slope g) * (u + shift) with
+//           g = min(x_t . Wg, limit), u = clamp(x_t . Wu, +-limit)    (gated)
 //   ACT 0 : y[slot, n]   = act[slot] . Wd[e][n]
 // slot = t * top + choice, e = table[token_t][choice], or, for experts
 // chosen by a router, e = slot_expert[slot] (an index >= the number of
@@ -38,8 +40,8 @@ __global__ __launch_bounds__(256) void moe_table_gemm_kernel(
     const int* __restrict__ table,      // (V, top)
     const int* __restrict__ slot_expert,   // (B*top,) or null (use the table)
     const bf16_t* __restrict__ w,       // (E, Nw, K): Nw = 2*Nout if gated
-    int B, int top, int K, int Nout) {
-  constexpr bool GATED = ACT == 1;
+    int B, int top, int K, int Nout, float limit, float slope, float shift) {
+  constexpr bool GATED = ACT == 1 || ACT == 3;
   constexpr bool BYTOKEN = ACT != 0;    // x rows by token, else by slot
   __shared__ int slots[MOE_MAX_SLOTS];
   __shared__ int count;
@@ -87,8 +89,14 @@ __global__ __launch_bounds__(256) void moe_table_gemm_kernel(
     for (int r = 0; r < 4; ++r) {
       const int ri = c0 + lhi * 4 + r;
       if (ri < cnt && nok) {
-        const float v = ACT == 1 ? siluf_acc(acc[r]) * acc2[r]
-                      : ACT == 2 ? gelu_erff_acc(acc[r]) : acc[r];
+        float v = acc[r];
+        if (ACT == 1) v = siluf_acc(acc[r]) * acc2[r];
+        if (ACT == 2) v = gelu_erff_acc(acc[r]);
+        if (ACT == 3) {
+          const float g = fminf(acc[r], limit);
+          const float u = fminf(fmaxf(acc2[r], -limit), limit);
+          v = g * sigmoidf_acc(slope * g) * (u + shift);
+        }
         out[(long)slots[ri] * Nout + n] = f2bf(v);
       }
     }
@@ -128,23 +136,26 @@ void seq_moe_table_ffn(torch::Tensor y, torch::Tensor act, torch::Tensor h,
                      (const bf16_t*)h.data_ptr(), h.stride(0),
                      (const long*)tokens.data_ptr<int64_t>(),
                      table.data_ptr<int>(), (const int*)nullptr,
-                     (const bf16_t*)w_gu.data_ptr(), B, top, W, ff);
+                     (const bf16_t*)w_gu.data_ptr(), B, top, W, ff, 0.f,
+                     0.f, 0.f);
   hipLaunchKernelGGL((moe_table_gemm_kernel<0>), dim3((W + 63) / 64, E),
                      dim3(256), 0, stream, (bf16_t*)y.data_ptr(),
                      (const bf16_t*)act.data_ptr(), (long)ff,
                      (const long*)tokens.data_ptr<int64_t>(),
                      table.data_ptr<int>(), (const int*)nullptr,
-                     (const bf16_t*)w_down.data_ptr(), B, top, ff, W);
+                     (const bf16_t*)w_down.data_ptr(), B, top, ff, W, 0.f,
+                     0.f, 0.f);
   HIP_CHECK_KERNEL();
 }
 
 // y (B*top, width) = router-chosen experts on h (B, width), plain
 // (gelu(W_up h), w_up (E, ff, W)) or gated (silu(W_gate h) * W_up h, w_up
-// (E, 2*ff, W) with the gate rows first); fills ``act`` (B*top, ff) on the
-// way.  Rows of identity experts stay unwritten.
+// (E, 2*ff, W) with the gate rows first; limit > 0: the clamped form); fills
+// ``act`` (B*top, ff) on the way.  Rows of identity experts stay unwritten.
 void seq_moe_routed_ffn(torch::Tensor y, torch::Tensor act, torch::Tensor h,
                         torch::Tensor idx, torch::Tensor w_up,
-                        torch::Tensor w_down, bool gated) {
+                        torch::Tensor w_down, bool gated, double limit,
+                        double slope, double shift) {
   CHECK_I32(idx);
   TORCH_CHECK(h.is_cuda() && h.dim() == 2 && h.stride(1) == 1 &&
               h.scalar_type() == torch::kBFloat16);
@@ -157,6 +168,7 @@ void seq_moe_routed_ffn(torch::Tensor y, torch::Tensor act, torch::Tensor h,
   const int top = idx.size(1);
   const int E = w_up.size(0), ff = w_up.size(1) / (gated ? 2 : 1);
   TORCH_CHECK(!gated || w_up.size(1) % 2 == 0);
+  TORCH_CHECK(limit >= 0 && (gated || limit == 0), "clamped experts are gated");
   TORCH_CHECK(w_up.size(2) == W && w_down.size(0) == E &&
               w_down.size(1) == W && w_down.size(2) == ff);
   TORCH_CHECK(W % 32 == 0 && ff % 32 == 0 && h.stride(0) % 8 == 0,
@@ -168,38 +180,35 @@ void seq_moe_routed_ffn(torch::Tensor y, torch::Tensor act, torch::Tensor h,
               y.size(0) == (long)B * top && y.size(1) == W);
   if (B == 0 || E == 0) return;
   auto stream = at::hip::getCurrentHIPStream();
-  if (gated)
-    hipLaunchKernelGGL((moe_table_gemm_kernel<1>), dim3((ff + 63) / 64, E),
-                       dim3(256), 0, stream, (bf16_t*)act.data_ptr(),
-                       (const bf16_t*)h.data_ptr(), h.stride(0),
-                       (const long*)nullptr, (const int*)nullptr,
-                       idx.data_ptr<int>(), (const bf16_t*)w_up.data_ptr(), B,
-                       top, W, ff);
-  else
-    hipLaunchKernelGGL((moe_table_gemm_kernel<2>), dim3((ff + 63) / 64, E),
-                       dim3(256), 0, stream, (bf16_t*)act.data_ptr(),
-                       (const bf16_t*)h.data_ptr(), h.stride(0),
-                       (const long*)nullptr, (const int*)nullptr,
-                       idx.data_ptr<int>(), (const bf16_t*)w_up.data_ptr(), B,
-                       top, W, ff);
+  const float lim = (float)limit, sl = (float)slope, sh = (float)shift;
+#define MOE_UP(ACTV)                                                          \
+  hipLaunchKernelGGL((moe_table_gemm_kernel<ACTV>), dim3((ff + 63) / 64, E),  \
+                     dim3(256), 0, stream, (bf16_t*)act.data_ptr(),           \
+                     (const bf16_t*)h.data_ptr(), h.stride(0),                \
+                     (const long*)nullptr, (const int*)nullptr,               \
+                     idx.data_ptr<int>(), (const bf16_t*)w_up.data_ptr(), B,  \
+                     top, W, ff, lim, sl, sh)
+  if (!gated) MOE_UP(2);
+  else if (lim > 0.f) MOE_UP(3);
+  else MOE_UP(1);
   hipLaunchKernelGGL((moe_table_gemm_kernel<0>), dim3((W + 63) / 64, E),
                      dim3(256), 0, stream, (bf16_t*)y.data_ptr(),
                      (const bf16_t*)act.data_ptr(), (long)ff,
                      (const long*)nullptr, (const int*)nullptr,
                      idx.data_ptr<int>(), (const bf16_t*)w_down.data_ptr(), B,
-                     top, ff, W);
+                     top, ff, W, 0.f, 0.f, 0.f);
   HIP_CHECK_KERNEL();
 }
 
 // ------------------------------------------------------------------ router
 // One wave per token, four tokens a block.  s = softmax(logits) over all E
-// router outputs, or (act 1) the logistic function of every logit;
-// choice = s + correction; experts form ``groups`` equal groups of
+// router outputs, or (act 1) the logistic function of every logit, or (act 2)
+// the logit itself; choice = s + correction; experts form ``groups`` equal groups of
 // neighbours, a group's score is the sum of its ``gtop`` largest choices,
 // and only the ``keep`` groups with the largest score stay eligible (the
 // others count as minus infinity); the ``top`` largest eligible choices
 // win, ties to the lower index.  Writes the indices and the UNcorrected s
-// at them.
+// at them, or (act 2) exp(choice - best choice).
 constexpr int ROUTE_MAX_E = 512;
 
 DEV_INLINE void wave_argmax(float& v, int& i) {
@@ -229,9 +238,9 @@ __global__ __launch_bounds__(256) void moe_route_kernel(
   float* c = c_sh[wid];
   float* gb = g_sh[wid];
   const float* z = logits + n * ldl;
-  if (act == 1) {
+  if (act >= 1) {
     for (int e = lane; e < E; e += 64) {
-      const float p = sigmoidf_acc(z[e]);
+      const float p = act == 1 ? sigmoidf_acc(z[e]) : z[e];
       s[e] = p;
       c[e] = p + correction[e];
     }
@@ -299,6 +308,7 @@ __global__ __launch_bounds__(256) void moe_route_kernel(
       if (gb[e / per] != INFINITY) c[e] = -INFINITY;
     __syncthreads();
   }
+  float best = 0.f;                   // the first pick is the largest
   for (int r = 0; r < top; ++r) {
     float bv = -INFINITY;
     int bi = 0x7fffffff;
@@ -311,10 +321,11 @@ __global__ __launch_bounds__(256) void moe_route_kernel(
     }
     wave_argmax(bv, bi);
     if (bi == 0x7fffffff) bi = 0;     // fewer eligible experts than top
+    if (r == 0) best = bv;
     if (lane == 0) {
       if (live) {
         idx[n * top + r] = bi;
-        wout[n * top + r] = s[bi];
+        wout[n * top + r] = act == 2 ? expf(bv - best) : s[bi];
       }
       c[bi] = -INFINITY;
     }
@@ -337,7 +348,7 @@ void seq_moe_route(torch::Tensor idx, torch::Tensor w, torch::Tensor logits,
   TORCH_CHECK(E >= 1 && E <= ROUTE_MAX_E, "router outputs above 512");
   TORCH_CHECK(correction.numel() == E && top >= 1 && top <= E);
   TORCH_CHECK(groups >= 1 && E % groups == 0 && keep >= 1 && keep <= groups);
-  TORCH_CHECK((act == 0 || act == 1) && group_top >= 1);
+  TORCH_CHECK(act >= 0 && act <= 2 && group_top >= 1);
   if (N == 0) return;
   auto stream = at::hip::getCurrentHIPStream();
   hipLaunchKernelGGL(moe_route_kernel, dim3((N + 3) / 4), dim3(256), 0, stream,
@@ -349,13 +360,14 @@ void seq_moe_route(torch::Tensor idx, torch::Tensor w, torch::Tensor logits,
 }
 
 // out[n, d] = sum_k w'[n,k] * (idx[n,k] < E ? ys[n*top+k, d] : h[n, d])
-//             (+ shared[n, d]),  w' = scale * w / (sum_k w + weight_eps)
+//             (+ shared[n, d] [* sigmoid(sgate[n])]),  w' = scale * w / (sum_k w + weight_eps)
 template <typename T>
 __global__ void moe_weighted_combine_kernel(
     T* __restrict__ out, const T* __restrict__ ys, const int* __restrict__ idx,
     const float* __restrict__ w, const T* __restrict__ h, long ldh,
     const T* __restrict__ shared, long lds_, int top, int E, float weight_eps,
-    long rows, int D, float scale) {
+    long rows, int D, float scale, const float* __restrict__ sgate,
+    long ldsg) {
   long i = (long)blockIdx.x * blockDim.x + threadIdx.x;
   const long stride = (long)gridDim.x * blockDim.x;
   for (; i < rows * D; i += stride) {
@@ -370,7 +382,10 @@ __global__ void moe_weighted_combine_kernel(
                                            : ldf(h + n * ldh + d);
       acc += w[n * top + k] * inv * v;
     }
-    if (shared) acc += ldf(shared + n * lds_ + d);
+    if (shared) {
+      const float sv = ldf(shared + n * lds_ + d);
+      acc += sgate ? sv * sigmoidf_acc(sgate[n * ldsg]) : sv;
+    }
     stf(out + i, acc);
   }
 }
@@ -378,7 +393,8 @@ __global__ void moe_weighted_combine_kernel(
 void seq_moe_weighted_combine(torch::Tensor out, torch::Tensor ys,
                               torch::Tensor idx, torch::Tensor w,
                               torch::Tensor h, torch::Tensor shared,
-                              int64_t E, double weight_eps, double scale) {
+                              int64_t E, double weight_eps, double scale,
+                              torch::Tensor shared_gate) {
   CHECK_I32(idx);
   CHECK_F32(w);
   CHECK_ROWS(h);
@@ -398,6 +414,12 @@ void seq_moe_weighted_combine(torch::Tensor out, torch::Tensor ys,
     TORCH_CHECK(shared.size(0) == N && shared.size(1) == D &&
                 shared.scalar_type() == ty);
   }
+  const bool has_sg = shared_gate.defined() && shared_gate.numel() > 0;
+  if (has_sg)
+    TORCH_CHECK(has_shared && shared_gate.is_cuda() && shared_gate.dim() == 2 &&
+                shared_gate.size(0) == N && shared_gate.size(1) == 1 &&
+                shared_gate.scalar_type() == torch::kFloat32,
+                "shared gate: one fp32 number per token");
   if (N == 0) return;
   const long nblk = std::min<long>((N * D + 255) / 256, MAX_RESIDENT_BLOCKS * 4);
   auto stream = at::hip::getCurrentHIPStream();
@@ -406,6 +428,7 @@ void seq_moe_weighted_combine(torch::Tensor out, torch::Tensor ys,
       w.data_ptr<float>(), (const T*)h.data_ptr(), h.stride(0),
       has_shared ? (const T*)shared.data_ptr() : nullptr,
       has_shared ? shared.stride(0) : 0, top, (int)E, (float)weight_eps, N,
-      D, (float)scale); });
+      D, (float)scale, has_sg ? shared_gate.data_ptr<float>() : nullptr,
+      has_sg ? shared_gate.stride(0) : 0); });
   HIP_CHECK_KERNEL();
 }

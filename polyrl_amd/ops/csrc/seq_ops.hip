@@ -710,6 +710,7 @@ void seq_latent_kv_store(torch::Tensor dkv, int64_t rank, torch::Tensor norm_w,
 // mode 0: silu(a) * b   mode 1: sigmoid(a) * b   mode 2: tanh(a)
 // mode 3: gelu(a), the exact (erf) form
 // mode 4: g * sigmoid(p1 * g) * (u + p2), g = min(a, p0), u = clamp(b, +-p0)
+// mode 5: max(a, 0) * b
 template <typename T>
 __global__ void act_mul_kernel(T* __restrict__ out, const T* __restrict__ a,
                                long lda, const T* __restrict__ b, long ldb,
@@ -733,7 +734,8 @@ __global__ void act_mul_kernel(T* __restrict__ out, const T* __restrict__ a,
       v = g * sigmoidf_acc(p1 * g) * (u + p2);
     } else {
       const float bv = ldf(b + r * ldb + c);
-      v = (mode == 0 ? siluf_acc(av) : sigmoidf_acc(av)) * bv;
+      v = (mode == 5   ? fmaxf(av, 0.f)
+           : mode == 0 ? siluf_acc(av) : sigmoidf_acc(av)) * bv;
     }
     stf(out + i, v);
   }

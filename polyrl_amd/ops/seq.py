@@ -1,9 +1,10 @@
 """Sequence-mixer ops for hybrid decoders: fp32-residual norms (plain and
 offset weights, fused joints, scaled branches, the gated layer-norm joint of
-parallel layers, the post-norm joint), the composed embedding (scaled row +
+parallel layers, the post-norm joint, the joint of several residual streams),
+the composed embedding (scaled row +
 hashed pair row + sinusoid), stateful causal convolutions, the generalised
 delta rule, the gated delta rule with per-channel decays, gated linear
-attention, the selective scans (per head and per channel), the real-gated
+attention, linear attention with a fixed decay, the selective scans (per head and per channel), the real-gated
 linear recurrence, windowed or causal latent attention with an optional softmax
 sink, grouped-query (window, chunked or causal; softmax or sigmoid weights)
 attention over paged K/V rows, and table-routed or router-chosen expert
@@ -275,6 +276,78 @@ def gla_scan(q, k, v, z_lin, z_bias, state, cu_q, state_slot,
                       q_scale, inv_tau)
 
 
+def lightning_scan(q, k, v, decay, state, cu_q, state_slot,
+                   max_rows: int = 0) -> torch.Tensor:
+    """Linear attention with one fixed decay per head over packed rows;
+    ``state`` (slots, H, Dk, Dv) fp32 in place, ``decay`` (H,) fp32.  q, k
+    (N, H*Dk) and v (N, H*Dv) pass SiLU here; per head
+    S <- decay S + k v^T, o = S^T q.  Returns o as fp32 (N, H*Dv), not
+    normed.  Inputs may be column slices.  ``max_rows`` bounds the rows of
+    one sequence (0 = unknown): single tokens stream the state once, bf16
+    portions run chunk by chunk on the matrix cores."""
+    if q.is_cuda:
+        slots, H, Dk, Dv = state.shape
+        out = torch.empty(q.shape[0], H * Dv, dtype=torch.float32,
+                          device=q.device)
+        if q.shape[0]:
+            _ext().seq_lightning_scan(out, q, k, v, decay, state, cu_q,
+                                      state_slot, max_rows)
+        return out
+    return R.lightning_scan(q, k, v, decay, state, cu_q, state_slot)
+
+
+def tanh_norm(x, alpha, w, b, out_dtype) -> torch.Tensor:
+    """tanh(alpha * x) * w + b for fp32 rows x (N, D); alpha (1,), w and b
+    (D,) fp32."""
+    if x.is_cuda:
+        out = torch.empty(x.shape, dtype=out_dtype, device=x.device)
+        if x.shape[0]:
+            _ext().seq_tanh_norm(out, x, alpha, w, b)
+        return out
+    return R.tanh_norm(x, alpha, w, b, out_dtype)
+
+
+def streams_open(table, tokens, streams: int, nxt, out_dtype):
+    """``streams`` equal fp32 copies (N, streams, D) of each token's table
+    row, and the next sublayer's input: with ``nxt`` = (in (S,), alpha (1,),
+    w (D,), b (D,)) fp32 that is tanh(alpha u) * w + b of
+    u = sum_s in[s] x_s."""
+    if table.is_cuda:
+        N, D = tokens.shape[0], table.shape[1]
+        xs = torch.empty(N, streams, D, dtype=torch.float32,
+                         device=table.device)
+        h = torch.empty(N, D, dtype=out_dtype, device=table.device)
+        if N:
+            _ext().seq_streams_open(xs, h, table, tokens, *nxt)
+        return xs, h
+    return R.streams_open(table, tokens, streams, nxt, out_dtype)
+
+
+def streams_join(xs, branch, w_mix, w_out, nxt, out_dtype, eps: float):
+    """The joint behind a sublayer of a stack with several residual streams,
+    in one pass over the row: x_t <- sum_s w_mix[s, t] x_s + w_out[t] * y,
+    all from the old streams xs (N, S, D) fp32, in place; returns the next
+    sublayer's input (``nxt`` as in :func:`streams_open`) as out_dtype, or,
+    with ``nxt`` None, the fp32 sum of the new streams (xs is then left as it
+    was).  ``branch`` is y (N, D), or (a, bias_a, w_a, b, bias_b, w_b,
+    scale): y = scale * (rms(a + bias_a) * w_a + rms(b + bias_b) * w_b) with
+    rms(v) = v / sqrt(mean(v^2) + eps), biases optional, weights (D,) fp32."""
+    if xs.is_cuda:
+        N, S, D = xs.shape
+        out = torch.empty(N, D, dtype=torch.float32 if nxt is None
+                          else out_dtype, device=xs.device)
+        if N:
+            e = torch.Tensor()
+            o = lambda t: t if t is not None else e
+            pair = branch if isinstance(branch, tuple) else \
+                (branch, None, None, None, None, None, 1.0)
+            _ext().seq_streams_join(
+                out, xs, *[o(t) for t in pair[:6]], pair[6], eps, w_mix,
+                w_out, *(nxt if nxt is not None else (e, e, e, e)))
+        return out
+    return R.streams_join(xs, branch, w_mix, w_out, nxt, out_dtype, eps)
+
+
 def channel_delta_scan(q, k, v, b_lin, z_lin, dt_bias, a_log, gate, norm_w,
                        state, cu_q, state_slot, key_eps: float, eps: float,
                        out_dtype, max_rows: int = 0) -> torch.Tensor:
@@ -408,7 +481,8 @@ def latent_window_attention(q_lat, q_rot, cache, page_table, seq_of_tok,
 def gqa_prepare_store(q, k, v, q_norm, k_norm, eps: float, inv_freq,
                       amp: float, positions, cache, slot_mapping, H: int,
                       G: int, D: int, Dv: int, head_unit: bool = False,
-                      v_inv_freq=None) -> torch.Tensor:
+                      v_inv_freq=None, interleaved: bool = False,
+                      bias=None) -> torch.Tensor:
     """Queries and cache rows of grouped-query attention from a step's
     projections (column slices allowed).  Optional RMS norm over the WHOLE
     query row and the whole key row (weights q_norm / k_norm; weights of D
@@ -421,11 +495,21 @@ def gqa_prepare_store(q, k, v, q_norm, k_norm, eps: float, inv_freq,
     query and key head by its root mean square after the rotation (no
     weight); ``v_inv_freq`` (Dv/2,) rotates every value head over all its
     entries by its position (pairs (m, m + Dv/2)) before it is cached.
-    Returns the queries (N, H*D)."""
+    ``bias`` (H*D + G*D + G*Dv,) fp32 is added to the projections first;
+    ``interleaved`` turns the pairs (2i, 2i + 1) instead (neither combines
+    with norms or rotated values).  Returns the queries (N, H*D)."""
     if q.is_cuda:
         out = torch.empty(q.shape[0], H * D, dtype=q.dtype, device=q.device)
         if q.shape[0]:
             e = torch.Tensor()
+            if bias is not None or interleaved:
+                assert q_norm is None and not head_unit and \
+                    v_inv_freq is None and v is not None
+                _ext().seq_gqa_prepare_plain(
+                    out, q, k, v, bias if bias is not None else e,
+                    inv_freq if inv_freq is not None else e, amp, positions,
+                    cache, slot_mapping, H, G, D, Dv, interleaved)
+                return out
             _ext().seq_gqa_prepare_store(
                 out, q, k, v if v is not None else e,
                 q_norm if q_norm is not None else e,
@@ -436,7 +520,7 @@ def gqa_prepare_store(q, k, v, q_norm, k_norm, eps: float, inv_freq,
         return out
     return R.gqa_prepare_store(q, k, v, q_norm, k_norm, eps, inv_freq, amp,
                                positions, cache, slot_mapping, H, G, D, Dv,
-                               head_unit, v_inv_freq)
+                               head_unit, v_inv_freq, interleaved, bias)
 
 
 def gqa_window_attention(q, cache, page_table, seq_of_tok, positions, H: int,
@@ -499,10 +583,10 @@ def gqa_window_attention(q, cache, page_table, seq_of_tok, positions, H: int,
 
 def gqa_mfma_supported(q, D: int, Dv: int) -> bool:
     """The matrix-core kernel serves bf16 batches that hold a prompt
-    portion, with head sizes in multiples of 8 up to 128; everything else
+    portion, with head sizes in multiples of 8 up to 256; everything else
     (fp32, odd sizes, steps of single tokens) runs one wave per row."""
     return (q.dtype == torch.bfloat16 and D % 8 == 0 and Dv % 8 == 0
-            and D <= 128 and Dv <= 128)
+            and D <= 256 and Dv <= 256)
 
 
 def moe_route(logits, correction, top: int, groups: int, keep: int,
@@ -513,14 +597,18 @@ def moe_route(logits, correction, top: int, groups: int, keep: int,
     neighbours, a group's score is the sum of its ``group_top`` largest
     choice scores, only the ``keep`` groups with the largest score stay
     eligible; the ``top`` largest eligible choice scores win.  Returns
-    (index int32 (N, top), s at those indices fp32 (N, top))."""
+    (index int32 (N, top), s at those indices fp32 (N, top)).  With
+    ``act="logits"`` s is the logit itself, ``correction`` a bias on it, and
+    the returned weights are exp(choice - largest choice): their shares are
+    the softmax over the chosen logits.  ``logits`` may be a column slice."""
     if logits.is_cuda:
         N = logits.shape[0]
         idx = torch.empty(N, top, dtype=torch.int32, device=logits.device)
         w = torch.empty(N, top, dtype=torch.float32, device=logits.device)
         if N:
             _ext().seq_moe_route(idx, w, logits, correction, groups, keep,
-                                 {"softmax": 0, "sigmoid": 1}[act], group_top)
+                                 {"softmax": 0, "sigmoid": 1, "logits": 2}[act],
+                                 group_top)
         return idx, w
     return R.moe_route(logits, correction, top, groups, keep, act, group_top)
 
@@ -540,26 +628,33 @@ def moe_routed_ffn_supported(h, top: int, ff: int) -> bool:
     return moe_table_ffn_supported(h, top, ff)
 
 
-def moe_routed_ffn(h, idx, w_up, w_down, gated: bool = False) -> torch.Tensor:
+def moe_routed_ffn(h, idx, w_up, w_down, gated: bool = False,
+                   clamp: Optional[tuple] = None) -> torch.Tensor:
     """Router-chosen experts: row t*top+k of the result is expert
     idx[t, k] applied to h[t]; rows whose index is >= E (identity experts)
     are left unwritten.  Plain experts: W_down gelu_erf(W_up h) with w_up
     (E, ff, W); ``gated``: W_down (silu(W_gate h) * W_up h) with w_up
-    (E, 2*ff, W) holding gate rows then up rows.  w_down (E, W, ff)."""
+    (E, 2*ff, W) holding gate rows then up rows; with ``clamp`` = (limit,
+    slope, shift) the gated activation is :func:`clamped_glu`'s.  w_down
+    (E, W, ff)."""
     if h.is_cuda:
         N, top = idx.shape
         y = torch.empty(N * top, h.shape[1], dtype=h.dtype, device=h.device)
         act = torch.empty(N * top, w_down.shape[2], dtype=h.dtype,
                           device=h.device)
-        _ext().seq_moe_routed_ffn(y, act, h, idx, w_up, w_down, gated)
+        lim, slope, shift = clamp or (0.0, 0.0, 0.0)
+        _ext().seq_moe_routed_ffn(y, act, h, idx, w_up, w_down, gated, lim,
+                                  slope, shift)
         return y
-    return R.moe_routed_ffn(h, idx, w_up, w_down, gated)
+    return R.moe_routed_ffn(h, idx, w_up, w_down, gated, clamp)
 
 
 def moe_weighted_combine(ys, idx, w, h, shared, E: int, weight_eps: float,
-                         out_dtype, scale: float = 1.0) -> torch.Tensor:
+                         out_dtype, scale: float = 1.0,
+                         shared_gate=None) -> torch.Tensor:
     """y[n] = sum_k w'[n,k] * (ys[n*top+k] if idx[n,k] < E else h[n])
-    [+ shared[n]] with w' = scale * w / (sum_k w + weight_eps), fp32
+    [+ shared[n], times sigmoid(shared_gate[n]) when a gate (N, 1) fp32 is
+    given (a column slice is allowed)] with w' = scale * w / (sum_k w + weight_eps), fp32
     sums."""
     if ys.is_cuda:
         out = torch.empty(h.shape, dtype=out_dtype, device=h.device)
@@ -567,10 +662,11 @@ def moe_weighted_combine(ys, idx, w, h, shared, E: int, weight_eps: float,
             _ext().seq_moe_weighted_combine(
                 out, ys, idx, w, h,
                 shared if shared is not None else torch.Tensor(), E,
-                weight_eps, scale)
+                weight_eps, scale,
+                shared_gate if shared_gate is not None else torch.Tensor())
         return out
     return R.moe_weighted_combine(ys, idx, w, h, shared, E, weight_eps,
-                                  out_dtype, scale)
+                                  out_dtype, scale, shared_gate)
 
 
 def silu_mul_any(gate, up):
@@ -581,6 +677,16 @@ def silu_mul_any(gate, up):
             _ext().seq_act_mul(out, gate, up, 0, 0.0, 0.0, 0.0)
         return out
     return R.silu_mul_any(gate, up)
+
+
+def relu_glu(gate, up):
+    """max(gate, 0) * up for bf16 or fp32 (row-strided views allowed)."""
+    if gate.is_cuda:
+        out = torch.empty(gate.shape, dtype=gate.dtype, device=gate.device)
+        if gate.shape[0]:
+            _ext().seq_act_mul(out, gate, up, 5, 0.0, 0.0, 0.0)
+        return out
+    return R.relu_glu(gate, up)
 
 
 def clamped_glu(gate, up, limit: float, slope: float, shift: float):

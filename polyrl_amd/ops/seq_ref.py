@@ -186,6 +186,66 @@ def gla_scan(q, k, v, z_lin, z_bias, state, cu_q, state_slot, q_scale,
     return out
 
 
+def lightning_scan(q, k, v, decay, state, cu_q, state_slot):
+    slots, H, Dk, Dv = state.shape
+    N = q.shape[0]
+
+    def silu(x, d):
+        x = x.float()
+        return (x * torch.sigmoid(x)).reshape(N, H, d)
+    qf, kf, vf = silu(q, Dk), silu(k, Dk), silu(v, Dv)
+    dec = decay.float().view(H, 1, 1)
+    out = torch.empty(N, H * Dv, dtype=torch.float32, device=q.device)
+    cu = cu_q.tolist()
+    for b, slot in enumerate(state_slot.tolist()):
+        S = state[slot]                                  # (H, Dk, Dv)
+        for n in range(cu[b], cu[b + 1]):
+            S = dec * S + kf[n].unsqueeze(-1) * vf[n].unsqueeze(1)
+            out[n] = torch.einsum("hk,hkv->hv", qf[n], S).reshape(-1)
+        state[slot] = S
+    return out
+
+
+def tanh_norm(x, alpha, w, b, out_dtype):
+    return (torch.tanh(alpha.float() * x.float()) * w.float()
+            + b.float()).to(out_dtype)
+
+
+def _streams_read(xs, nxt, out_dtype):
+    w_in, alpha, w, b = nxt
+    u = torch.einsum("s,nsd->nd", w_in.float(), xs)
+    return tanh_norm(u, alpha, w, b, out_dtype)
+
+
+def streams_open(table, tokens, streams, nxt, out_dtype):
+    x = table[tokens.long()].float()
+    xs = x.unsqueeze(1).repeat(1, streams, 1)
+    return xs, _streams_read(xs, nxt, out_dtype)
+
+
+def streams_join(xs, branch, w_mix, w_out, nxt, out_dtype, eps):
+    if isinstance(branch, tuple):
+        a, bias_a, wa, b, bias_b, wb, scale = branch
+
+        def unit(t, bias, w):
+            t = t.float() if bias is None else t.float() + bias.float()
+            return t * torch.rsqrt(t.pow(2).mean(-1, keepdim=True) + eps) \
+                * w.float()
+        y = (unit(a, bias_a, wa) + unit(b, bias_b, wb)) * scale
+    else:
+        y = branch.float()
+    new = torch.einsum("st,nsd->ntd", w_mix.float(), xs) \
+        + w_out.float().view(1, -1, 1) * y.unsqueeze(1)
+    if nxt is None:
+        return new.sum(1)
+    xs.copy_(new)
+    return _streams_read(xs, nxt, out_dtype)
+
+
+def relu_glu(gate, up):
+    return (gate.float().clamp(min=0) * up.float()).to(gate.dtype)
+
+
 def clamped_glu(gate, up, limit, slope, shift):
     g = gate.float().clamp(max=limit)
     u = up.float().clamp(-limit, limit)
@@ -302,10 +362,14 @@ def gelu_erf(x):
 
 def gqa_prepare_store(q, k, v, q_norm, k_norm, eps, inv_freq, amp, positions,
                       cache, slot_mapping, H, G, D, Dv, head_unit=False,
-                      v_inv_freq=None):
+                      v_inv_freq=None, interleaved=False, bias=None):
     N = q.shape[0]
     qf, kf = q.float(), k.float()
     vf = kf if v is None else v.float()
+    if bias is not None:
+        bf = bias.float()
+        a, b = H * D, (H + G) * D
+        qf, kf, vf = qf + bf[:a], kf + bf[a:b], vf + bf[b:]
     if q_norm is not None and q_norm.numel() == D:      # per head
         def unit(x, n, w):
             x = x.reshape(N, n, D)
@@ -319,7 +383,11 @@ def gqa_prepare_store(q, k, v, q_norm, k_norm, eps, inv_freq, amp, positions,
             * k_norm.float()
     qf, kf = qf.reshape(N, H, D).clone(), kf.reshape(N, G, D).clone()
     half = 0 if inv_freq is None else inv_freq.numel()
-    if half:
+    if half and interleaved:
+        for t in (qf, kf):
+            t[..., :2 * half] = _rotate(t[..., :2 * half], positions,
+                                        inv_freq, amp, True)
+    elif half:
         ang = positions.float().unsqueeze(-1) * inv_freq.float()
         c = (torch.cos(ang) * amp).unsqueeze(1)
         s = (torch.sin(ang) * amp).unsqueeze(1)
@@ -393,8 +461,9 @@ def gqa_window_attention(q, cache, page_table, seq_of_tok, positions, H, G,
 
 def moe_route(logits, correction, top, groups, keep, act="softmax",
               group_top=1):
-    s = torch.softmax(logits.float(), -1) if act == "softmax" \
-        else torch.sigmoid(logits.float())
+    z = logits.float()
+    s = torch.softmax(z, -1) if act == "softmax" \
+        else torch.sigmoid(z) if act == "sigmoid" else z
     choice = s + correction.float()
     N, E = s.shape
     if groups > 1:
@@ -405,11 +474,13 @@ def moe_route(logits, correction, top, groups, keep, act="softmax",
         open_.scatter_(1, kept, True)
         choice = choice.masked_fill(
             ~open_.repeat_interleave(E // groups, 1), float("-inf"))
-    idx = choice.topk(top, -1).indices
+    best, idx = choice.topk(top, -1)
+    if act == "logits":
+        return idx.int(), torch.exp(best - best[:, :1])
     return idx.int(), s.gather(1, idx)
 
 
-def moe_routed_ffn(h, idx, w_up, w_down, gated=False):
+def moe_routed_ffn(h, idx, w_up, w_down, gated=False, clamp=None):
     N, top = idx.shape
     E = w_up.shape[0]
     y = torch.zeros(N * top, h.shape[1], dtype=h.dtype, device=h.device)
@@ -421,7 +492,8 @@ def moe_routed_ffn(h, idx, w_up, w_down, gated=False):
         a = h[sl // top] @ w_up[e].t()
         if gated:
             ff = w_down.shape[2]
-            a = silu_mul_any(a[:, :ff], a[:, ff:])
+            a = clamped_glu(a[:, :ff], a[:, ff:], *clamp) if clamp \
+                else silu_mul_any(a[:, :ff], a[:, ff:])
         else:
             a = gelu_erf(a)
         y[sl] = a @ w_down[e].t()
@@ -429,7 +501,7 @@ def moe_routed_ffn(h, idx, w_up, w_down, gated=False):
 
 
 def moe_weighted_combine(ys, idx, w, h, shared, E, weight_eps, out_dtype,
-                         scale=1.0):
+                         scale=1.0, shared_gate=None):
     N, top = idx.shape
     wn = w.float() / (w.float().sum(-1, keepdim=True) + weight_eps) * scale
     rows = ys.float().view(N, top, -1)
@@ -437,7 +509,10 @@ def moe_weighted_combine(ys, idx, w, h, shared, E, weight_eps, out_dtype,
     rows = torch.where(ident, h.float().unsqueeze(1).expand_as(rows), rows)
     y = (rows * wn.unsqueeze(-1)).sum(1)
     if shared is not None:
-        y = y + shared.float()
+        sh = shared.float()
+        if shared_gate is not None:
+            sh = sh * torch.sigmoid(shared_gate.float()).view(N, 1)
+        y = y + sh
     return y.to(out_dtype)
 
 

@@ -478,7 +478,7 @@ class Engine:
         cfg_style = self.model.cfg.layer_style
         self.enable_hybrid_graphs = (
             str(dev) != "cpu"
-            and cfg_style in ("prenorm", "parallel", "postnorm")
+            and cfg_style in ("prenorm", "parallel", "postnorm", "streams")
             and bool(int(__import__("os").environ.get(
                 "POLYRL_HIP_GRAPHS", "1"))))
         self._graph_seen: Dict[int, int] = {}

@@ -269,11 +269,63 @@ class SelectiveScanMixer(_Part):
                    self.wo)
 
 
+class LightningMixer(_Part):
+    """Linear attention with fixed decays (models.hybrid.LightningSpec): one
+    fused projection for queries, keys, values and the output gate; the scan
+    applies the SiLUs and keeps one fp32 (dim, vdim) state per head and
+    sequence; the norm over the row of all heads and the sigmoid gate are
+    one kernel.  ``w_in`` / ``wo`` may be slices of another mixer's."""
+
+    @staticmethod
+    def sizes(s):
+        """(rows of the input projection, columns of the output one)."""
+        return 2 * s.heads * (s.dim + s.vdim), s.heads * s.vdim
+
+    def __init__(self, spec, width, device, dtype, w_in=None, wo=None):
+        self.spec = s = spec
+        self.nk, self.nv = s.heads * s.dim, s.heads * s.vdim
+        z = lambda *a, dt=dtype: torch.empty(*a, device=device, dtype=dt)
+        self.w_in = w_in if w_in is not None else \
+            z(2 * (self.nk + self.nv), width)
+        self.wo = wo if wo is not None else z(width, self.nv)
+        self.norm = z(self.nv, dt=torch.float32)
+        self.decay = torch.tensor(s.decay, dtype=torch.float32,
+                                  device=device)
+
+    def named(self, p):
+        a, b = 2 * self.nk, 2 * self.nk + self.nv
+        return {p + "q": self.w_in[:self.nk], p + "k": self.w_in[self.nk:a],
+                p + "v": self.w_in[a:b], p + "g": self.w_in[b:],
+                p + "norm": self.norm, p + "o": self.wo}
+
+    def state_shapes(self):
+        s = self.spec
+        return {"S": (s.heads, s.dim, s.vdim)}
+
+    def mix(self, proj, bt, li, model, cache, states, out=None, scale=1.0):
+        assert out is None and scale == 1.0
+        nk, nv = self.nk, self.nv
+        o = seq.lightning_scan(
+            proj.narrow(1, 0, nk), proj.narrow(1, nk, nk),
+            proj.narrow(1, 2 * nk, nv), self.decay,
+            states.tensors[(li, self.key + "S")], bt.cu_q, bt.state_slot,
+            max_rows=bt.max_q)
+        return seq.group_rmsnorm(o, self.norm, 1, model.cfg.norm_eps,
+                                 proj.dtype,
+                                 gate=proj.narrow(1, 2 * nk + nv, nv))
+
+    def forward(self, h, bt, li, model, cache, states):
+        return _mm(self.mix(_mm(h, self.w_in), bt, li, model, cache, states),
+                   self.wo)
+
+
 class ParallelMixer(_Part):
     """Two mixers side by side (models.hybrid.ParallelMixerSpec): one fused
     input projection, and one output product over both results, which the
     mixers' last kernels write next to each other already multiplied by
-    their scales."""
+    their scales.  With ``out_norm`` the two output products stay apart and
+    the result is the tuple that :func:`ops.seq.streams_join` norms and adds
+    (projection biases join in the cache writer, the output bias there)."""
 
     def __init__(self, spec, width, device, dtype):
         self.spec = s = spec
@@ -282,17 +334,29 @@ class ParallelMixer(_Part):
             cr.sizes(s.right)
         self.w_in = torch.empty(self.rl + self.rr, width, device=device,
                                 dtype=dtype)
-        self.wo = torch.empty(width, self.cl + self.cr, device=device,
-                              dtype=dtype)
+        wl = wr = None                 # output products of their own
+        self.norm_l = self.norm_r = None
+        if s.out_norm:
+            f32 = torch.float32
+            self.norm_l = torch.empty(width, device=device, dtype=f32)
+            self.norm_r = torch.empty(width, device=device, dtype=f32)
+        else:
+            self.wo = torch.empty(width, self.cl + self.cr, device=device,
+                                  dtype=dtype)
+            wl, wr = self.wo[:, :self.cl], self.wo[:, self.cl:]
         self.left = cl(s.left, width, device, dtype, w_in=self.w_in[:self.rl],
-                       wo=self.wo[:, :self.cl])
+                       wo=wl)
         self.right = cr(s.right, width, device, dtype,
-                        w_in=self.w_in[self.rl:], wo=self.wo[:, self.cl:])
+                        w_in=self.w_in[self.rl:], wo=wr)
         self.left.key, self.right.key = "left.", "right."
 
     def named(self, p):
-        return {**self.left.named(p + "left."),
-                **self.right.named(p + "right.")}
+        out = {**self.left.named(p + "left."),
+               **self.right.named(p + "right.")}
+        if self.norm_l is not None:
+            out[p + "left.out"], out[p + "right.out"] = self.norm_l, \
+                self.norm_r
+        return out
 
     def cache_row(self):
         rows = [m.cache_row() for m in (self.left, self.right)]
@@ -305,6 +369,14 @@ class ParallelMixer(_Part):
 
     def forward(self, h, bt, li, model, cache, states):
         proj = _mm(h, self.w_in)
+        if self.norm_l is not None:
+            yl, yr = (_mm(m.mix(proj.narrow(1, at, n), bt, li, model, cache,
+                                states), m.wo)
+                      for m, at, n in ((self.left, 0, self.rl),
+                                       (self.right, self.rl, self.rr)))
+            return (yl, getattr(self.left, "b_o", None), self.norm_l,
+                    yr, getattr(self.right, "b_o", None), self.norm_r,
+                    self.spec.left_scale)
         y = torch.empty(h.shape[0], self.cl + self.cr, device=h.device,
                         dtype=h.dtype)
         self.left.mix(proj.narrow(1, 0, self.rl), bt, li, model, cache,
@@ -643,10 +715,16 @@ class WindowAttnMixer(_Part):
         self.nv = 0 if s.values_from_keys else s.kv_heads * s.vdim
         self.ng = s.heads if s.head_gate else 0
         self.row = s.kv_heads * (s.dim + s.vdim)
-        # (the head gate has no bias: its entries stay zero)
+        # biases join in the product (the head gate has none: its entries
+        # stay zero), or, on a slice of another mixer's product, in the cache
+        # writer
         self.w_in, self.b_in = (w_in, None) if w_in is not None else \
             self._with_tail(self.nq + self.nk + self.nv + self.ng, tail,
                             width, device, dtype, s.qkv_bias)
+        self.b_store = z(self.nq + self.nk + self.nv, dt=f32) \
+            if s.qkv_bias and w_in is not None else None
+        self.b_o = z(width, dt=f32 if w_in is not None else dtype) \
+            if s.o_bias else None
         self.sink = z(s.heads, dt=f32) if s.sink else None
         self.unit_sink = torch.zeros(s.heads, device=device, dtype=f32) \
             if s.unit_sink else None
@@ -666,6 +744,7 @@ class WindowAttnMixer(_Part):
             f, self.amp = s.rope.inv_freq_and_amp()
             self.inv_freq = torch.tensor(f, dtype=torch.float64).float() \
                 .to(device)
+        self.interleaved = s.rope is not None and s.rope.interleaved
         self.rel = self.dist_bucket = None
         if s.bias_far > 0:
             self.rel = z(int(s.bias_rows), s.heads, dt=f32)
@@ -687,10 +766,13 @@ class WindowAttnMixer(_Part):
         if self.rel is not None:
             out[p + "rel"] = self.rel
         if s_bias:
-            out[p + "q.b"] = self.b_in[:a]
-            out[p + "k.b"] = self.b_in[a:b]
+            bias = self.b_in if self.b_store is None else self.b_store
+            out[p + "q.b"] = bias[:a]
+            out[p + "k.b"] = bias[a:b]
             if self.nv:
-                out[p + "v.b"] = self.b_in[b:b + self.nv]
+                out[p + "v.b"] = bias[b:b + self.nv]
+        if self.b_o is not None:
+            out[p + "o.b"] = self.b_o
         if self.sink is not None:
             out[p + "sink"] = self.sink
         if self.head_bias is not None:
@@ -712,7 +794,8 @@ class WindowAttnMixer(_Part):
     def forward(self, h, bt, li, model, cache, states):
         proj = _mm(h, self.w_in, self.b_in)
         self._split_tail(proj)
-        return _mm(self.mix(proj, bt, li, model, cache, states), self.wo)
+        return _mm(self.mix(proj, bt, li, model, cache, states), self.wo,
+                   self.b_o)
 
     def mix(self, proj, bt, li, model, cache, states, out=None, scale=1.0):
         s = self.spec
@@ -730,7 +813,8 @@ class WindowAttnMixer(_Part):
             self.q_norm, self.k_norm, model.cfg.norm_eps, self.inv_freq,
             self.amp, bt.positions, rows, bt.slot_mapping, s.heads,
             s.kv_heads, s.dim, s.vdim, head_unit=s.head_unit_norm,
-            v_inv_freq=self.v_inv_freq)
+            v_inv_freq=self.v_inv_freq, interleaved=self.interleaved,
+            bias=self.b_store)
         return seq.gqa_window_attention(
             q, rows, bt.page_table, bt.seq_of_tok, bt.positions, s.heads,
             s.kv_heads, s.dim, s.vdim, s.window, s.keep_first, self.rel,
@@ -746,8 +830,9 @@ class WindowAttnMixer(_Part):
 
 
 class DenseFF(_Part):
-    """Gated feed-forward, gate and up as one product: silu(gate) * up, or
-    the clamped form (models.hybrid.FFSpec.act); optional biases."""
+    """Gated feed-forward, gate and up as one product: silu(gate) * up,
+    relu(gate) * up or the clamped form (models.hybrid.FFSpec.act); optional
+    biases."""
 
     def __init__(self, spec, width, vocab, device, dtype):
         self.spec = spec
@@ -774,6 +859,8 @@ class DenseFF(_Part):
         gate, up = gu.narrow(1, 0, self.ff), gu.narrow(1, self.ff, self.ff)
         if f.act == "clamped":
             act = seq.clamped_glu(gate, up, f.limit, f.gate_slope, f.up_shift)
+        elif f.act == "relu":
+            act = seq.relu_glu(gate, up)
         else:
             act = seq.silu_mul_any(gate, up)
         # added by the caller's next norm
@@ -853,27 +940,36 @@ class TableMoE(_Part):
 
 class RoutedMoE(_Part):
     """Experts chosen by an fp32 router (softmax or per-logit sigmoid
-    scores) with a selection-only correction and group-limited choice;
-    experts W_down gelu(W_up h) or, gated, W_down (silu(W_gate h) * W_up h)
-    with the gate rows stored ahead of the up rows; trailing identity
-    experts return the input; a shared expert runs for every token.
-    Returns the sublayer output (N, width)."""
+    scores with a selection-only correction, or a softmax over the chosen
+    biased logits) and group-limited choice; experts W_down gelu(W_up h) or,
+    gated, W_down (silu(W_gate h) * W_up h) or the clamped form, with the
+    gate rows stored ahead of the up rows; trailing identity experts return
+    the input; a shared expert of the same form runs for every token,
+    optionally times the sigmoid of one number per token, whose projection
+    is the router's last row.  Returns the sublayer output (N, width)."""
 
     def __init__(self, spec, width, vocab, device, dtype):
         self.spec = f = spec
         self.E, self.top, self.ff = f.experts, f.top, f.ff
         z = lambda *a, dt=dtype: torch.empty(*a, device=device, dtype=dt)
         f32 = torch.float32
-        self.gated = f.expert_act == "silu_gated"
+        self.gated = f.expert_act != "gelu"
+        self.clamp = (f.limit, f.gate_slope, f.up_shift) \
+            if f.expert_act == "clamped_gated" else None
+        self.R = R = f.experts + f.identity         # router outputs
         self.w_up = z(f.experts, (2 if self.gated else 1) * f.ff, width)
         self.w_down = z(f.experts, width, f.ff)
-        self.router = z(f.experts + f.identity, width, dt=f32)
-        self.correction = z(f.experts + f.identity, dt=f32)
-        self.s_up = z(f.shared_ff, width) if f.shared_ff else None
+        self.router = z(R + (1 if f.shared_gate else 0), width, dt=f32)
+        self.correction = z(R, dt=f32)
+        self.s_up = z((2 if self.gated else 1) * f.shared_ff, width) \
+            if f.shared_ff else None
         self.s_down = z(width, f.shared_ff) if f.shared_ff else None
 
     def named(self, p):
-        out = {p + "router": self.router, p + "correction": self.correction}
+        f = self.spec
+        out = {p + "router": self.router[:self.R],
+               p + ("router.b" if f.router_bias else "correction"):
+               self.correction}
         for e in range(self.E):
             if self.gated:
                 out[f"{p}e{e}.gate"] = self.w_up[e, :self.ff]
@@ -882,8 +978,14 @@ class RoutedMoE(_Part):
                 out[f"{p}e{e}.up"] = self.w_up[e]
             out[f"{p}e{e}.down"] = self.w_down[e]
         if self.s_up is not None:
-            out[p + "shared.up"] = self.s_up
+            if self.gated:
+                out[p + "shared.gate"] = self.s_up[:f.shared_ff]
+                out[p + "shared.up"] = self.s_up[f.shared_ff:]
+            else:
+                out[p + "shared.up"] = self.s_up
             out[p + "shared.down"] = self.s_down
+        if f.shared_gate:
+            out[p + "shared.sg"] = self.router[self.R:]
         return out
 
     def experts_large(self, h, idx):
@@ -915,36 +1017,46 @@ class RoutedMoE(_Part):
         ys[order] = ys_sorted           # identity rows stay unread
         return ys
 
-    def _act(self, a):
+    def _act(self, a, limit=None):
         if self.gated:
-            return seq.silu_mul_any(a.narrow(1, 0, self.ff),
-                                    a.narrow(1, self.ff, self.ff))
+            ff = a.shape[1] // 2
+            gate, up = a.narrow(1, 0, ff), a.narrow(1, ff, ff)
+            if self.clamp is not None:
+                return seq.clamped_glu(
+                    gate, up, self.clamp[0] if limit is None else limit,
+                    *self.clamp[1:])
+            return seq.silu_mul_any(gate, up)
         return seq.gelu_erf(a)
 
     def forward(self, h, res, bt):
         f = self.spec
         logits = _mm(h.float(), self.router)
+        gate = logits.narrow(1, self.R, 1) if f.shared_gate else None
+        if gate is not None:
+            logits = logits.narrow(1, 0, self.R)
         idx, w = seq.moe_route(logits, self.correction, f.top, f.group_count,
                                f.group_keep, f.router_act, f.group_top)
         if h.shape[0] <= 256 and self.E and \
                 seq.moe_routed_ffn_supported(h, self.top, self.ff):
             ys = seq.moe_routed_ffn(h, idx, self.w_up, self.w_down,
-                                    self.gated)
+                                    self.gated, self.clamp)
         elif self.E:
             ys = self.experts_large(h, idx.long())
         else:
             ys = h.new_empty(h.shape[0] * f.top, h.shape[1])
         shared = None
         if self.s_up is not None:
-            shared = _mm(seq.gelu_erf(_mm(h, self.s_up)), self.s_down)
+            shared = _mm(self._act(_mm(h, self.s_up), f.shared_limit),
+                         self.s_down)
         return seq.moe_weighted_combine(ys, idx, w, h, shared, self.E,
-                                        f.weight_eps, h.dtype, f.route_scale)
+                                        f.weight_eps, h.dtype, f.route_scale,
+                                        gate)
 
 
 _MIXERS = {"general_delta": DeltaRuleMixer, "mamba2": SSMMixer,
            "gla": GLAMixer, "rglru": RGLRUMixer,
            "channel_delta": ChannelDeltaMixer, "mamba": SelectiveScanMixer,
-           "parallel": ParallelMixer,
+           "lightning": LightningMixer, "parallel": ParallelMixer,
            "latent_attention": LatentAttnMixer, "attention": WindowAttnMixer}
 _FFS = {"dense": DenseFF, "moe": TableMoE, "routed_moe": RoutedMoE}
 
@@ -1023,6 +1135,48 @@ class PostNormLayer:
         out.update(self.mixer.named(p + "mix."))
         if self.ff is not None:
             out[p + "norm2"] = self.norm2
+            out.update(self.ff.named(p + "mlp."))
+        return out
+
+
+class StreamsLayer:
+    """Several residual streams: a sublayer reads a mixture of them through
+    a tanh norm, and all streams are mixed anew with its result
+    (models.hybrid.HybridConfig, layer style "streams")."""
+
+    class Side:
+        """What one sublayer reads and writes the streams with."""
+
+        def __init__(self, width, streams, device):
+            z = lambda *a: torch.empty(*a, device=device, dtype=torch.float32)
+            self.alpha, self.w, self.b = z(1), z(width), z(width)
+            self.w_in, self.w_out = z(streams), z(streams)
+            self.w_mix = z(streams, streams)          # [from, to]
+
+        @property
+        def read(self):
+            return self.w_in, self.alpha, self.w, self.b
+
+        def named(self, norm, hc):
+            return {norm: self.w, norm + ".alpha": self.alpha,
+                    norm + ".b": self.b, hc + "in": self.w_in,
+                    hc + "out": self.w_out, hc + "mix": self.w_mix}
+
+    def __init__(self, cfg: HybridConfig, li: int, device, dtype):
+        L = cfg.layers[li]
+        W = cfg.hidden_size
+        self.mixer = _MIXERS[L.mixer.kind](L.mixer, W, device, dtype)
+        self.ff = None if L.ff is None else \
+            _FFS[L.ff.kind](L.ff, W, cfg.vocab_size, device, dtype)
+        self.side1 = self.Side(W, cfg.streams, device)
+        self.side2 = self.Side(W, cfg.streams, device) \
+            if self.ff is not None else None
+
+    def named(self, p: str) -> Dict[str, torch.Tensor]:
+        out = self.side1.named(p + "norm1", p + "hc1.")
+        out.update(self.mixer.named(p + "mix."))
+        if self.ff is not None:
+            out.update(self.side2.named(p + "norm2", p + "hc2."))
             out.update(self.ff.named(p + "mlp."))
         return out
 
@@ -1131,12 +1285,17 @@ class HybridInferenceModel:
         self.prenorm = cfg.layer_style == "prenorm"
         self.parallel = cfg.layer_style == "parallel"
         self.postnorm = cfg.layer_style == "postnorm"
-        layer_cls = SandwichLayer if self.sandwich else \
+        self.streams = cfg.layer_style == "streams"
+        layer_cls = StreamsLayer if self.streams else \
+            SandwichLayer if self.sandwich else \
             PreNormLayer if self.prenorm else \
             PostNormLayer if self.postnorm else \
             ParallelLayer if self.parallel else HybridLayer
-        self.layers = [layer_cls(cfg, li, device, dtype)
-                       for li in range(cfg.num_hidden_layers)]
+        owned = {li: layer_cls(cfg, li, device, dtype)
+                 for li, L in enumerate(cfg.layers) if L.weights_of is None}
+        # a layer without tensors of its own runs its owner's
+        self.layers = [owned[li if L.weights_of is None else L.weights_of]
+                       for li, L in enumerate(cfg.layers)]
         self.runs = cfg.run_order()
         W = cfg.hidden_size
         self.embed = torch.empty(cfg.vocab_size, W, device=device, dtype=dtype)
@@ -1165,7 +1324,14 @@ class HybridInferenceModel:
         if cfg.sin_pos_base > 0:
             self.pos_inv_freq = seq.sinusoid_inv_freq(W, cfg.sin_pos_base,
                                                       device)
-        for li, lw in enumerate(self.layers):
+        self.final_alpha = self.final_b = None
+        if cfg.norm_kind == "tanh":
+            self.final_alpha = torch.empty(1, device=device,
+                                           dtype=torch.float32)
+            self.final_b = torch.empty(W, device=device, dtype=torch.float32)
+            self._name_map["final.norm.alpha"] = self.final_alpha
+            self._name_map["final.norm.b"] = self.final_b
+        for li, lw in owned.items():
             self._name_map.update(lw.named(f"l{li}."))
         self.capture_layers: Optional[List[torch.Tensor]] = None
 
@@ -1196,12 +1362,12 @@ class HybridInferenceModel:
     def graph_safe_decode(self, B: int) -> bool:
         """Whether a decode step of B single tokens runs without a decision
         on the host (so it can be captured in a graph): pre-norm stacks
-        always; post-norm and parallel stacks when every routed feed-forward takes the
-        fused expert kernels (bf16, sizes in multiples of 32, a batch the
+        always; post-norm, parallel and streams stacks when every routed
+        feed-forward takes the fused expert kernels (bf16, sizes in multiples of 32, a batch the
         kernels' slot list holds)."""
         if self.prenorm:
             return True
-        if not self.parallel and not self.postnorm:
+        if not self.parallel and not self.postnorm and not self.streams:
             return False
         for L in self.layers:
             f = L.ff
@@ -1304,6 +1470,16 @@ class HybridInferenceModel:
                 buf.copy_(torch.randn(buf.shape, generator=g) - 3.0)
             elif self.parallel and name.endswith(".b"):
                 buf.copy_(torch.randn(buf.shape, generator=g) * 0.2)
+            elif self.streams and name.endswith(".alpha"):
+                buf.copy_(0.5 + torch.rand(buf.shape, generator=g) * 0.5)
+            elif self.streams and name.endswith(".b"):
+                buf.copy_(torch.randn(buf.shape, generator=g) * 0.1)
+            elif self.streams and name.endswith((".in", ".out")):
+                buf.copy_((1.0 / buf.numel() if name.endswith(".in") else 1.0)
+                          + torch.randn(buf.shape, generator=g) * 0.1)
+            elif self.streams and name.endswith(".mix"):
+                buf.copy_(torch.eye(buf.shape[0]) * 0.9
+                          + torch.randn(buf.shape, generator=g) * 0.1)
             elif name.endswith("mix.pb"):
                 buf.copy_(torch.randn(buf.shape, generator=g) * 0.5 - 4.0)
             elif (self.sandwich or self.postnorm) and name.endswith(
@@ -1359,6 +1535,8 @@ class HybridInferenceModel:
             return self._forward_parallel(bt, cache, states)
         if self.postnorm:
             return self._forward_postnorm(bt, cache, states)
+        if self.streams:
+            return self._forward_streams(bt, cache, states)
         cfg, dt = self.cfg, self.dtype
         eps = cfg.norm_eps
         res = self.embed[bt.tokens].float()
@@ -1435,6 +1613,34 @@ class HybridInferenceModel:
             if self.capture_layers is not None:
                 self.capture_layers.append(res.clone())
         return res
+
+    def _forward_streams(self, bt: HybridBatch, cache, states):
+        """Layer runs of the streams style: one fused pass behind every
+        sublayer mixes its result into all streams (N, S, width) fp32 and
+        writes the next sublayer's normed input; the last one returns the
+        sum of the streams."""
+        cfg, dt = self.cfg, self.dtype
+        subs = []                       # (run, run of a mixer?, sublayer, side)
+        for ri, li in enumerate(self.runs):
+            L = self.layers[li]
+            subs.append((ri, True, L.mixer, L.side1))
+            if L.ff is not None:
+                subs.append((ri, False, L.ff, L.side2))
+        if not subs:
+            return self.embed[bt.tokens].float() * cfg.streams
+        xs, h = seq.streams_open(self.embed, bt.tokens, cfg.streams,
+                                 subs[0][3].read, dt)
+        for i, (ri, is_mixer, sub, side) in enumerate(subs):
+            y = sub.forward(h, bt, ri, self, cache, states) if is_mixer else \
+                sub.forward(h, None, bt)
+            last = i + 1 == len(subs)
+            nxt = None if last else subs[i + 1][3].read
+            h = seq.streams_join(xs, y, side.w_mix, side.w_out, nxt, dt,
+                                 cfg.norm_eps)
+            if self.capture_layers is not None and \
+                    (last or subs[i + 1][1]):
+                self.capture_layers.append(h.clone() if last else xs.sum(1))
+        return h
 
     def embed_rows(self, bt: HybridBatch) -> torch.Tensor:
         """The fp32 embedding output of a packed batch: scaled table row,
@@ -1551,6 +1757,9 @@ class HybridInferenceModel:
             h = seq.gated_add_layernorm(
                 res_rows.contiguous(), None, None, None, None,
                 self.final_norm, None, self.cfg.norm_eps, self.dtype)[0]
+        elif self.cfg.norm_kind == "tanh":
+            h = seq.tanh_norm(res_rows.contiguous(), self.final_alpha,
+                              self.final_norm, self.final_b, self.dtype)
         else:
             h = seq.add_rmsnorm_f32res(res_rows.contiguous(), None,
                                        self.final_norm, self.cfg.norm_eps,
