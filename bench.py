@@ -133,8 +133,8 @@ def main():
                         "decode tokens/s of a hybrid decoder beside a dense "
                         "one of equal width and depth (registry names, "
                         "random weights), e.g. bizusun-1b:llama3-1b, "
-                        "vurivik-1b:llama3-1b, nasipel-1b:kuforax-1b or "
-                        "puvapel-1b:vurivik-1b")
+                        "vurivik-1b:llama3-1b, nasipel-1b:kuforax-1b, "
+                        "puvapel-1b:vurivik-1b or redirax-1b:kuforax-1b")
     p.add_argument("--engine-prefill", type=str, default="8x2048",
                    help="engine-compare prefill workload: prompts x length")
     p.add_argument("--engine-decode", type=str, default="64x128",

@@ -108,8 +108,26 @@ MODEL_CONFIGS = {
 
 def _hybrid_presets():
     from .hybrid import (bizusun_preset, kuforax_preset, nasipel_preset,
-                         puvapel_preset, vurivik_preset)
+                         puvapel_preset, redirax_preset, vurivik_preset)
     return {
+        # tiny stack for CPU unit tests / fast GPU smoke
+        "redirax-debug": lambda: redirax_preset(
+            width=64, layers=4, vocab=300, heads=4, kv_heads=2,
+            right_heads=2, experts=6, top=2, expert_ff=32, shared_ff=32,
+            streams=3, shared_from=3),
+        # bench pairs: beside kuforax-400m / -1b / -8b-l8 (equal width,
+        # depth, heads, vocabulary, expert count and choices, a shared expert
+        # in both; the gated experts' hidden size is set so that the
+        # parameter totals agree within 1.5 %)
+        "redirax-400m": lambda: redirax_preset(
+            width=1024, layers=12, vocab=32000, heads=16, kv_heads=4,
+            experts=8, top=2, expert_ff=1216, shared_ff=1216),
+        "redirax-1b": lambda: redirax_preset(
+            width=2048, layers=16, vocab=128256, heads=32, kv_heads=8,
+            experts=16, top=2, expert_ff=1600, shared_ff=1600),
+        "redirax-8b-l8": lambda: redirax_preset(
+            width=4096, layers=8, vocab=128256, heads=32, kv_heads=8,
+            experts=16, top=2, expert_ff=2368, shared_ff=2368),
         # tiny stack for CPU unit tests / fast GPU smoke
         "puvapel-debug": lambda: puvapel_preset(
             width=64, layers=3, vocab=300, heads=4, kv_heads=2, ff=96,

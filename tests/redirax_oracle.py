@@ -193,7 +193,7 @@ def random_weights(cfg, seed=0):
     Wd, V, S = int(cfg["width"]), int(cfg["vocab"]), int(cfg["streams"])
 
     def rnd(*shape, std=1.0, mean=0.0):
-        return (torch.randn(*shape, generator=g) * std + mean) \
+        return (torch.randn(shape, generator=g) * std + mean) \
             .bfloat16().float()
 
     def lin(o, i, gain=1.0):

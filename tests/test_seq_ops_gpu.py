@@ -917,3 +917,221 @@ def test_chunked_attention_with_head_norms(dt, H, G, D, Dv, half, chunk, lens,
             if dt == torch.bfloat16 else dict(rtol=1e-4, atol=1e-4)
         torch.testing.assert_close(got.cpu().float(), ref, **lim)
         assert not out[:, :8].any() and not out[:, 8 + H * Dv:].any()
+
+
+@pytest.mark.parametrize("dt", DTYPES)
+@pytest.mark.parametrize("S", [1, 2, 3, 4, 5, 9, 32])
+@pytest.mark.parametrize("D", [36, 37, 1028, 2048, 3000, 5000])
+def test_streams_join_open_and_tanh_norm(dt, S, D):
+    """The joint of several residual streams: a plain branch, a pair of
+    normed branches with and without biases (column slices too), the stack's
+    end, and the rows' start."""
+    N = 5
+    g = lambda t: None if t is None else t.to(DEV)
+    xs = rnd(N, S, D)
+    mix, w_out, w_in = rnd(S, S) * 0.4, rnd(S), rnd(S)
+    nxt = (w_in, rnd(1), rnd(D), rnd(D))
+    dn = tuple(map(g, nxt))
+    big = rnd(N, 2 * D + 3, dt=dt)
+    a, b = big[:, :D], big[:, D + 3:]
+    bg = g(big)
+    da, db = bg[:, :D], bg[:, D + 3:]
+    wa, wb, ba, bb = rnd(D), rnd(D), rnd(D), rnd(D)
+    lim = tol(dt)
+    for br, dbr in (((a), (da)),
+                    ((a, None, wa, b, None, wb, 0.5),
+                     (da, None, g(wa), db, None, g(wb), 0.5)),
+                    ((a, ba, wa, b, None, wb, 1.5),
+                     (da, g(ba), g(wa), db, None, g(wb), 1.5)),
+                    ((a, ba, wa, b, bb, wb, 0.7),
+                     (da, g(ba), g(wa), db, g(bb), g(wb), 0.7))):
+        x0, x1 = xs.clone(), xs.clone().to(DEV)
+        want = R.streams_join(x0, br, mix, w_out, nxt, dt, 1e-5)
+        got = seq.streams_join(x1, dbr, g(mix), g(w_out), dn, dt, 1e-5)
+        torch.testing.assert_close(x1.cpu(), x0, rtol=1e-4, atol=1e-4)
+        torch.testing.assert_close(
+            got.cpu().float(), want.float(), rtol=lim["rtol"],
+            atol=max(lim["atol"], 2e-4))
+        x2 = xs.clone().to(DEV)
+        end = seq.streams_join(x2, dbr, g(mix), g(w_out), None, dt, 1e-5)
+        assert end.dtype == torch.float32
+        torch.testing.assert_close(end.cpu(), x0.sum(1), rtol=1e-4, atol=1e-3)
+        torch.testing.assert_close(x2.cpu(), xs, rtol=0, atol=0)
+    table = rnd(11, D, dt=dt)
+    tokens = torch.tensor([3, 0, 10, 3, 7])
+    x0, h0 = R.streams_open(table, tokens, S, nxt, dt)
+    x1, h1 = seq.streams_open(g(table), g(tokens), S, dn, dt)
+    torch.testing.assert_close(x1.cpu(), x0, rtol=0, atol=0)
+    torch.testing.assert_close(h1.cpu().float(), h0.float(),
+                               rtol=lim["rtol"], atol=max(lim["atol"], 2e-4))
+    z = rnd(N, D)
+    torch.testing.assert_close(
+        seq.tanh_norm(g(z), *dn[1:], dt).cpu().float(),
+        R.tanh_norm(z, *nxt[1:], dt).float(), **lim)
+
+
+@pytest.mark.parametrize("dt", DTYPES)
+@pytest.mark.parametrize("H,Dk,Dv,lens", [
+    (2, 32, 64, [5, 1, 20]), (3, 10, 14, [40, 2]), (1, 7, 5, [9, 1]),
+    (2, 64, 68, [64, 65, 63, 1]), (2, 96, 128, [130, 1]),
+    (1, 128, 192, [200, 3, 129]), (2, 20, 40, [128]), (1, 130, 8, [70]),
+    (1, 300, 20, [33, 1]), (2, 512, 12, [6]), (4, 64, 64, [1, 1, 1, 1]),
+    (2, 33, 7, [1, 1]), (1, 500, 132, [1, 1]), (3, 4, 4, [300, 1]),
+])
+def test_lightning_scan(dt, H, Dk, Dv, lens):
+    """Single tokens, token by token and 64-token chunks on the matrix
+    cores: results and states, decays from zero to one, starting from
+    non-zero states in scattered slots."""
+    slots = [(3 * i + 1) % 7 for i in range(len(lens))]
+    bt = batch(lens, slots)
+    N = sum(lens)
+    pad = 4
+    big = rnd(N, pad + H * (2 * Dk + Dv), dt=dt)
+    dec = torch.tensor([0.0, 0.9, 1.0, 0.37][:H]) if H > 1 else \
+        torch.tensor([0.97])
+    st = rnd(7, H, Dk, Dv)
+
+    def go(mod, d, s, **kw):
+        c, sl, _ = bt[d]
+        x = big.to(d)
+        a, b = pad + H * Dk, pad + 2 * H * Dk
+        return mod.lightning_scan(x[:, pad:a], x[:, a:b], x[:, b:],
+                                  dec.to(d), s, c, sl, **kw)
+    s0 = st.clone()
+    want = go(R, "cpu", s0)
+    scale = float(want.abs().max())
+    for mr in {max(lens), 0}:
+        s1 = st.clone().to(DEV)
+        got = go(seq, DEV, s1, max_rows=mr)
+        lim = 1e-5 if dt == torch.float32 or max(lens) == 1 and mr == 1 \
+            else 1e-2
+        assert float((got.cpu() - want).abs().max()) < lim * scale
+        assert float((s1.cpu() - s0).abs().max()) < \
+            lim * float(s0.abs().max())
+
+
+def test_lightning_chunks_keep_fp32_states_and_scores():
+    """bf16 portions whose q, k and v are exact after SiLU (large whole
+    numbers): states with 16 significant bits, decayed keys and decayed
+    scores must come through the matrix cores with far less than a bf16
+    rounding."""
+    H, Dk, Dv, N = 2, 64, 64, 200
+    bt = batch([N], [0])
+    x = torch.randint(20, 28, (N, H * (2 * Dk + Dv))).to(torch.bfloat16)
+    dec = torch.tensor([0.83, 0.996])
+    st = rnd(1, H, Dk, Dv) * 1000 + 333.3
+
+    def go(mod, d, s):
+        c, sl, _ = bt[d]
+        y = x.to(d)
+        a, b = H * Dk, 2 * H * Dk
+        return mod.lightning_scan(y[:, :a], y[:, a:b], y[:, b:], dec.to(d), s,
+                                  c, sl)
+    s0, s1 = st.clone(), st.clone().to(DEV)
+    want = go(R, "cpu", s0)
+    got = go(seq, DEV, s1)
+    rel = (got.cpu() - want).abs() / want.abs()
+    assert float(rel.max()) < 3e-5
+    assert float(((s1.cpu() - s0).abs() / s0.abs()).max()) < 3e-5
+
+
+@pytest.mark.parametrize("dt", DTYPES)
+@pytest.mark.parametrize("H,G,D,Dv,half,inter,bias", [
+    (4, 2, 24, 40, 6, True, True), (4, 2, 24, 40, 5, True, True),
+    (3, 3, 11, 7, 3, True, True), (3, 1, 11, 7, 4, False, True),
+    (6, 3, 64, 64, 32, True, False), (8, 2, 32, 16, 16, False, True),
+    (2, 1, 48, 200, 0, True, True), (1, 1, 2, 1, 1, True, True),
+])
+def test_gqa_prepare_with_biases_and_pairs(dt, H, G, D, Dv, half, inter,
+                                           bias):
+    lens, starts, page = [5, 1, 3], [0, 370, 6], 4
+    cache, ptab, pos, sot, slot = _paged(lens, starts, page, G * (D + Dv), dt)
+    N = sum(lens)
+    for off in (0, 4, 3):
+        big = rnd(N, off + H * D + G * D + G * Dv + 5, dt=dt)
+        a, b = off + H * D, off + (H + G) * D
+        bs = rnd((H + G) * D + G * Dv) if bias else None
+        inv = torch.rand(half) if half else None
+        g = lambda t: None if t is None else t.to(DEV)
+        c0, c1 = cache.clone(), cache.clone().to(DEV)
+        cut = lambda t: (t[:, off:a], t[:, a:b], t[:, b:b + G * Dv])
+        want = R.gqa_prepare_store(*cut(big), None, None, 1e-5, inv, 1.07,
+                                   pos, c0, slot, H, G, D, Dv,
+                                   interleaved=inter, bias=bs)
+        got = seq.gqa_prepare_store(*cut(g(big)), None, None, 1e-5, g(inv),
+                                    1.07, g(pos), c1, g(slot), H, G, D, Dv,
+                                    interleaved=inter, bias=g(bs))
+        lim = dict(tol(dt))
+        lim["atol"] = max(lim["atol"], 1e-4)      # angles of hundreds
+        torch.testing.assert_close(got.cpu().float(), want.float(), **lim)
+        torch.testing.assert_close(c1.cpu().float(), c0.float(), **lim)
+
+
+@pytest.mark.parametrize("dt", DTYPES)
+@pytest.mark.parametrize("H,G,D,Dv,lens,starts", [
+    (4, 2, 96, 192, [70, 1, 130], [3, 300, 40]),
+    (2, 1, 128, 256, [40, 1], [10, 65]), (3, 3, 40, 168, [66, 2], [0, 9]),
+    (2, 2, 200, 48, [64, 5], [30, 0]), (1, 1, 256, 256, [65], [64]),
+    (8, 8, 160, 144, [33, 1], [20, 90]), (4, 1, 8, 24, [1, 1, 1], [0, 31, 200]),
+    (4, 2, 24, 48, [1, 1], [5, 70]), (2, 1, 16, 80, [9, 1], [55, 64]),
+])
+def test_causal_attention_with_large_and_uneven_head_sizes(dt, H, G, D, Dv,
+                                                           lens, starts):
+    page = 4
+    cache, ptab, pos, sot, slot = _paged(lens, starts, page, G * (D + Dv), dt)
+    q = rnd(sum(lens), H * D, dt=dt, scale=2.5)
+    scale = 1.0 / math.sqrt(D)
+    args = (H, G, D, Dv, 1 << 30, 0, None, None, None, scale, dt)
+    want = R.gqa_window_attention(q, cache, ptab, sot, pos, *args)
+    g = lambda t: t.to(DEV)
+    for tl in (None, seq.attention_tiles(lens, DEV)):
+        got = seq.gqa_window_attention(g(q), g(cache), g(ptab), g(sot),
+                                       g(pos), *args, tiles=tl)
+        torch.testing.assert_close(got.cpu().float(), want.float(), **tol(dt))
+
+
+@pytest.mark.parametrize("N,E,top", [(1, 4, 1), (37, 5, 3), (130, 16, 16),
+                                     (9, 300, 7)])
+def test_router_softmax_over_chosen_logits(N, E, top):
+    z = rnd(N, E + 3) * 3
+    bias = rnd(E)
+    zz = z[:, 1:1 + E]
+    i0, w0 = R.moe_route(zz, bias, top, 1, 1, "logits")
+    i1, w1 = seq.moe_route(z.to(DEV)[:, 1:1 + E], bias.to(DEV), top, 1, 1,
+                           "logits")
+    assert torch.equal(i1.cpu(), i0)
+    torch.testing.assert_close(w1.cpu(), w0, rtol=1e-5, atol=1e-6)
+    best = (zz + bias).topk(top, -1).values
+    torch.testing.assert_close(w0 / w0.sum(-1, keepdim=True),
+                               torch.softmax(best, -1), rtol=1e-5, atol=1e-6)
+
+
+@pytest.mark.parametrize("N,top,E", [(1, 2, 4), (37, 3, 5), (200, 4, 8)])
+def test_clamped_experts_and_gated_shared_expert(N, top, E):
+    dt = torch.bfloat16
+    Wd, ff = 96, 64
+    h = rnd(N, Wd, dt=dt)
+    idx = torch.stack([torch.randperm(E)[:top] for _ in range(N)]).int()
+    up, down = rnd(E, 2 * ff, Wd, dt=dt, scale=0.2), \
+        rnd(E, Wd, ff, dt=dt, scale=0.1)
+    clamp = (0.8, 1.702, 1.0)
+    ys0 = R.moe_routed_ffn(h, idx, up, down, True, clamp)
+    ys1 = seq.moe_routed_ffn(h.to(DEV), idx.to(DEV), up.to(DEV),
+                             down.to(DEV), True, clamp)
+    torch.testing.assert_close(ys1.cpu().float(), ys0.float(), **tol(dt))
+    w, shared, z = torch.rand(N, top), rnd(N, Wd, dt=dt), rnd(N, E + 1)
+    want = R.moe_weighted_combine(ys0, idx, w, h, shared, E, 0.0, dt,
+                                  shared_gate=z[:, E:])
+    got = seq.moe_weighted_combine(ys1, idx.to(DEV), w.to(DEV), h.to(DEV),
+                                   shared.to(DEV), E, 0.0, dt,
+                                   shared_gate=z.to(DEV)[:, E:])
+    torch.testing.assert_close(got.cpu().float(), want.float(), **tol(dt))
+
+
+@pytest.mark.parametrize("dt", DTYPES)
+def test_relu_glu(dt):
+    big = rnd(9, 70, dt=dt)
+    d = big.to(DEV)
+    torch.testing.assert_close(
+        seq.relu_glu(d[:, :33], d[:, 37:]).cpu().float(),
+        R.relu_glu(big[:, :33], big[:, 37:]).float(), **tol(dt))
