@@ -157,7 +157,11 @@ void seq_moe_weighted_combine(torch::Tensor out, torch::Tensor ys,
                               torch::Tensor idx, torch::Tensor w,
                               torch::Tensor h, torch::Tensor shared,
                               int64_t E, double weight_eps, double scale,
-                              torch::Tensor shared_gate);
+                              torch::Tensor shared_gate, torch::Tensor place);
+void seq_moe_router(torch::Tensor idx, torch::Tensor w, torch::Tensor extra,
+                    torch::Tensor h, torch::Tensor router,
+                    torch::Tensor correction, int64_t groups, int64_t keep,
+                    int64_t act, int64_t group_top);
 
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("seq_gqa_prepare_store", &seq_gqa_prepare_store,
@@ -177,6 +181,8 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
         "grouped-query window attention on the matrix cores (bf16)");
   m.def("seq_moe_route", &seq_moe_route,
         "softmax / sigmoid router with correction and group-limited top-k");
+  m.def("seq_moe_router", &seq_moe_router,
+        "router product and choice for batches of few tokens");
   m.def("seq_moe_routed_ffn", &seq_moe_routed_ffn,
         "router-chosen plain or gated experts for decode-sized bf16 batches");
   m.def("seq_gated_add_layernorm", &seq_gated_add_layernorm,

@@ -4,13 +4,21 @@
 // odd-size / single-token path.  A block is 4 waves x 16 rows: up to 64
 // consecutive tokens of one sequence for one query head.  Their
 // windows overlap, so the block walks the union of the visible keys in tiles
-// of 32 -- first the kept first tokens that lie before the union's window
+// of GKV -- first the kept first tokens that lie before the union's window
 // ([0, min(keep, kmin))), then [kmin, last position] -- and masks per
-// element: key j is live for the row at position p when j <= p and
-// (p - j < window or j < keep); with chunks a windowed key must also lie in
-// the row's own chunk of positions.  K and V tiles of the head's key/value group
-// come from the paged cache rows ([G*D keys | G*Dv values]) into LDS; QK^T
-// and P.V run on v_mfma_f32_16x16x32_bf16 with fp32 accumulators; scale, the
+// element, in tiles that need it: key j is live for the row at position p
+// when j <= p and (p - j < window or j < keep); with chunks a windowed key
+// must also lie in the row's own chunk of positions.
+//
+// K and V tiles of the head's key/value group come from the paged cache rows
+// ([G*D keys | G*Dv values]) into LDS, keys as they are (16-byte pieces
+// XOR-swizzled by row), values turned to [entry][key] in 4x4 pieces on the
+// way.  The wave computes the scores as K Q^T, so that a lane's accumulators
+// hold many keys of ONE row: the softmax needs two lane exchanges per tile,
+// and the weights, rounded to bf16, are at once the B operand of V^T P^T (the
+// order of keys inside a product's K index is free: both operands use the
+// order the accumulators have).  The output accumulates as [entry][row].
+// Products run on v_mfma_f32_16x16x32_bf16 with fp32 accumulators; scale, the
 // optional distance-bucket bias (this head's column of the table sits in
 // LDS), the online softmax and the sigmoid head gate are fp32; so are the
 // optional sink (the running maximum starts at the head's sink, the running
@@ -19,10 +27,9 @@
 // to the capped score, and weights sigmoid(score) per live key without any
 // normalisation over keys (no running maximum, no rescaling); head sums as
 // fp32 into a separate buffer for the pass that turns rotated values back.
-// The next tiles are fetched into registers while the current ones are
-// multiplied.
-// K-tile bytes are XOR-swizzled by row inside each 64-byte chunk.  Key and
-// value head sizes are apart (KS and KV chunks of 32), up to 256 each.
+// The next tile's words are fetched into registers while the current one is
+// multiplied; the cache rows of the tile after that are looked up meanwhile.
+// Key and value head sizes are apart (KS and KV chunks of 32), up to 256 each.
 //
 // Grid: one dimension.  Workgroups go to the 8 XCDs in turn (id mod 8), each
 // with an L2 of its own, so the id is taken apart as XCD = id % 8 and, inside
@@ -50,7 +57,6 @@ typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8_t;
 typedef __attribute__((ext_vector_type(4))) float f32x4_t;
 typedef __attribute__((ext_vector_type(4))) int i32x4_t;
 
-constexpr int GKV = 32;          // keys per tile
 constexpr int GQA_MAX_REL = 256; // bias-table rows held in LDS
 constexpr int GQA_XCDS = 8;      // accelerator dies, each with its own L2
 
@@ -59,7 +65,7 @@ DEV_INLINE int gtile_off(int row, int byte_col) {
   return row * (KS * 64) + (byte_col ^ ((row & 3) << 4));
 }
 
-template <int KS, int KV>
+template <int KS, int KV, int GKV>
 __global__ __launch_bounds__(256) void gqa_attn_mfma_kernel(
     bf16_t* __restrict__ out,            // (N, H*Dv), row stride ldo
     const bf16_t* __restrict__ q,        // (N, H*D)
@@ -75,9 +81,11 @@ __global__ __launch_bounds__(256) void gqa_attn_mfma_kernel(
     const float* __restrict__ hbias, bool sigm, float* __restrict__ out32,
     int chunk, long ldo, float out_scale) {
   constexpr int NVT = KV * 2;            // 16-wide output tiles
+  constexpr int NKT = GKV / 16;          // 16-key score tiles
+  constexpr int VROW = GKV + 8;          // padded LDS row of one value entry
   __shared__ __attribute__((aligned(16))) bf16_t Ks[GKV * KS * 32];
-  __shared__ __attribute__((aligned(16))) bf16_t Vs[GKV * KV * 32];
-  __shared__ __attribute__((aligned(16))) bf16_t Ps[4][16 * GKV];
+  __shared__ __attribute__((aligned(16))) bf16_t Vt[KV * 32 * VROW];
+  __shared__ int slot_s[2][GKV];         // cache rows of a tile's keys
   __shared__ float rel_s[GQA_MAX_REL];
 
   const int lane = threadIdx.x & 63;
@@ -114,16 +122,29 @@ __global__ __launch_bounds__(256) void gqa_attn_mfma_kernel(
   const int nk = keep < kmin ? keep : kmin;      // kept keys before kmin
   const int nkt = (nk + GKV - 1) / GKV;          // their tiles
   const int nwt = (pmax - kmin) / GKV + 1;       // window tiles
-
+  const int ntiles = nkt + nwt;
+  // tile ti covers keys [t0, t0+GKV) up to jmax
+  auto tile_t0 = [&](int ti) { return ti < nkt ? ti * GKV : kmin + (ti - nkt) * GKV; };
+  auto tile_jmax = [&](int ti) { return ti < nkt ? nk - 1 : pmax; };
+  // cache row of a tile's key i (keys past the tile's last: that one)
+  auto slot_of = [&](int ti, int i) {
+    const int j = min(tile_t0(ti) + i, tile_jmax(ti));
+    return ptab[j / page_size] * page_size + j % page_size;
+  };
+  if (threadIdx.x < GKV) slot_s[0][threadIdx.x] = slot_of(0, threadIdx.x);
+  else if ((int)threadIdx.x < 2 * GKV && ntiles > 1)
+    slot_s[1][threadIdx.x - GKV] = slot_of(1, threadIdx.x - GKV);
   if (rel)
     for (int i = threadIdx.x; i < rel_rows; i += 256)
       rel_s[i] = rel[(long)i * H + h];
 
-  // ---- Q fragments (A layout): row l15 of this wave, k = ks*32 + lhi*8 ..
+  // ---- this lane's row: Q fragments (k = ks*32 + lhi*8 ..), its state -----
+  const int ri = wid * 16 + l15;
+  const bool rok = ri < cnt;
+  const int rpos = pos0 + ri, rlo = row_lo(rpos);
   bf16x8_t qfrag[KS];
   {
-    const int i = wid * 16 + l15;
-    const bf16_t* qp = q + ((long)(n0 + (i < cnt ? i : 0)) * H + h) * D;
+    const bf16_t* qp = q + ((long)(n0 + (rok ? ri : 0)) * H + h) * D;
     const i32x4_t zi = {0, 0, 0, 0};
 #pragma unroll
     for (int ks = 0; ks < KS; ++ks) {
@@ -134,83 +155,63 @@ __global__ __launch_bounds__(256) void gqa_attn_mfma_kernel(
   }
   const float hb = hbias ? hbias[h] : 0.f;
   const float inv_cap = cap > 0.f ? 1.f / cap : 0.f;
-  float m_run[4], l_run[4], rscale[4];
-  int rpos[4], rlo[4];
-  bool rok[4];
+  float rscale = scale;
+  if (qt_coef != 0.f)
+    rscale *= 1.f + qt_coef * logf((float)((rpos + 1) / qt_every + 1));
+  // running maximum of the row; each of its four lanes sums its own keys
+  float m_run = sink ? sink[h] : -1e30f;
+  float l_run = sink && lhi == 0 ? 1.f : 0.f;
   f32x4_t o_acc[NVT];
 #pragma unroll
-  for (int r = 0; r < 4; ++r) {
-    const int i = wid * 16 + lhi * 4 + r;
-    m_run[r] = sink ? sink[h] : -1e30f;
-    l_run[r] = sink ? 1.f : 0.f;
-    rpos[r] = pos0 + i;
-    rlo[r] = row_lo(rpos[r]);
-    rok[r] = i < cnt;
-    rscale[r] = scale;
-    if (qt_coef != 0.f)
-      rscale[r] *= 1.f + qt_coef * logf((float)((rpos[r] + 1) / qt_every + 1));
-  }
-#pragma unroll
   for (int nt = 0; nt < NVT; ++nt) o_acc[nt] = {0.f, 0.f, 0.f, 0.f};
+  // first and last position of the wave's rows (rows past cnt included: what
+  // they compute is dropped)
+  const int wp0 = pos0 + wid * 16, wp1 = wp0 + 15;
+  const int wlo = row_lo(wp1);
 
-  // tile ti covers keys [t0, t0+32) up to jmax
-  auto tile_t0 = [&](int ti) { return ti < nkt ? ti * GKV : kmin + (ti - nkt) * GKV; };
-  auto tile_jmax = [&](int ti) { return ti < nkt ? nk - 1 : pmax; };
-
-  constexpr int NK = (GKV * KS * 4 + 255) / 256;
-  constexpr int NV = (GKV * KV * 4 + 255) / 256;
-  i32x4_t prek[NK], prev[NV];
+  // ---- global -> registers: 16-byte key pieces, 4x4 value pieces ----------
+  constexpr int NKI = GKV * KS * 4;              // key pieces of a tile
+  constexpr int NK = (NKI + 255) / 256;
+  constexpr int KG = GKV / 4;                    // groups of four keys
+  constexpr int NVI = KG * KV * 8;               // value pieces of a tile
+  constexpr int NV = (NVI + 255) / 256;
+  i32x4_t prek[NK];
+  uint2 prev[NV][4];
   auto fetch = [&](int ti) {
-    const int t0 = tile_t0(ti), jmax = tile_jmax(ti);
-    const i32x4_t z = {0, 0, 0, 0};
-    auto row_of = [&](int j) {
-      return cache + ((long)ptab[j / page_size] * page_size + j % page_size) * row;
-    };
-    if (KS == KV) {                      // a thread's key and value rows agree
-#pragma unroll
-      for (int i = 0; i < NK; ++i) {
-        const int v = threadIdx.x + i * 256;
-        const int col = (v % (KS * 4)) * 8;
-        const int j = t0 + v / (KS * 4);
-        prek[i] = z;
-        prev[i] = z;
-        if (v < GKV * KS * 4 && j <= jmax) {
-          const bf16_t* base = row_of(j);
-          if (col < D) prek[i] = *reinterpret_cast<const i32x4_t*>(base + koff + col);
-          if (col < Dv) prev[i] = *reinterpret_cast<const i32x4_t*>(base + voff + col);
-        }
-      }
-      return;
-    }
+    const int last = tile_jmax(ti) - tile_t0(ti);   // last live key's place
+    const int* sl = slot_s[ti & 1];
 #pragma unroll
     for (int i = 0; i < NK; ++i) {
       const int v = threadIdx.x + i * 256;
-      const int col = (v % (KS * 4)) * 8;
-      const int j = t0 + v / (KS * 4);
-      prek[i] = z;
-      if (v < GKV * KS * 4 && j <= jmax && col < D)
-        prek[i] = *reinterpret_cast<const i32x4_t*>(row_of(j) + koff + col);
+      const int kr = v / (KS * 4), col = (v % (KS * 4)) * 8;
+      prek[i] = {0, 0, 0, 0};
+      if (v < NKI && kr <= last && col < D)
+        prek[i] = *reinterpret_cast<const i32x4_t*>(
+            cache + (long)sl[kr] * row + koff + col);
     }
 #pragma unroll
     for (int i = 0; i < NV; ++i) {
       const int v = threadIdx.x + i * 256;
-      const int col = (v % (KV * 4)) * 8;
-      const int j = t0 + v / (KV * 4);
-      prev[i] = z;
-      if (v < GKV * KV * 4 && j <= jmax && col < Dv)
-        prev[i] = *reinterpret_cast<const i32x4_t*>(row_of(j) + voff + col);
+      const int kg = v % KG * 4, col = v / KG * 4;
+#pragma unroll
+      for (int t = 0; t < 4; ++t) {
+        prev[i][t] = make_uint2(0u, 0u);
+        if (v < NVI && kg + t <= last && col < Dv)
+          prev[i][t] = *reinterpret_cast<const uint2*>(
+              cache + (long)sl[kg + t] * row + voff + col);
+      }
     }
   };
-  const int ntiles = nkt + nwt;
+  __syncthreads();                       // the first two tiles' rows
   fetch(0);
 
   for (int ti = 0; ti < ntiles; ++ti) {
     const int t0 = tile_t0(ti), jmax = tile_jmax(ti);
-    // ---- registers -> LDS tiles, then request the next tiles ------------
+    // ---- registers -> LDS tiles, then request the next tile ---------------
 #pragma unroll
     for (int i = 0; i < NK; ++i) {
       const int v = threadIdx.x + i * 256;
-      if (v < GKV * KS * 4)
+      if (v < NKI)
         *reinterpret_cast<i32x4_t*>(
             reinterpret_cast<char*>(Ks) +
             gtile_off<KS>(v / (KS * 4), (v % (KS * 4)) * 16)) = prek[i];
@@ -218,121 +219,153 @@ __global__ __launch_bounds__(256) void gqa_attn_mfma_kernel(
 #pragma unroll
     for (int i = 0; i < NV; ++i) {
       const int v = threadIdx.x + i * 256;
-      if (v < GKV * KV * 4)
-        *reinterpret_cast<i32x4_t*>(
-            reinterpret_cast<char*>(Vs) +
-            gtile_off<KV>(v / (KV * 4), (v % (KV * 4)) * 16)) = prev[i];
+      if (v < NVI) {
+        bf16_t* vt = Vt + v / KG * 4 * VROW + v % KG * 4;
+        const uint2* p = prev[i];
+        // entry e of the four keys, two per word
+        *reinterpret_cast<uint2*>(vt) = make_uint2(
+            __builtin_amdgcn_perm(p[1].x, p[0].x, 0x05040100u),
+            __builtin_amdgcn_perm(p[3].x, p[2].x, 0x05040100u));
+        *reinterpret_cast<uint2*>(vt + VROW) = make_uint2(
+            __builtin_amdgcn_perm(p[1].x, p[0].x, 0x07060302u),
+            __builtin_amdgcn_perm(p[3].x, p[2].x, 0x07060302u));
+        *reinterpret_cast<uint2*>(vt + 2 * VROW) = make_uint2(
+            __builtin_amdgcn_perm(p[1].y, p[0].y, 0x05040100u),
+            __builtin_amdgcn_perm(p[3].y, p[2].y, 0x05040100u));
+        *reinterpret_cast<uint2*>(vt + 3 * VROW) = make_uint2(
+            __builtin_amdgcn_perm(p[1].y, p[0].y, 0x07060302u),
+            __builtin_amdgcn_perm(p[3].y, p[2].y, 0x07060302u));
+      }
     }
     __syncthreads();
     if (ti + 1 < ntiles) fetch(ti + 1);
+    int next_slot = 0;                   // stored before the closing barrier
+    const bool look = threadIdx.x < GKV && ti + 2 < ntiles;
+    if (look) next_slot = slot_of(ti + 2, threadIdx.x);
 
-    // ---- S (16 rows x 32 keys) = Q K^T ----------------------------------
-    f32x4_t c[2];
+    // ---- S^T (GKV keys x 16 rows) = K Q^T; row l15, keys lhi*4 + r --------
+    float p[NKT][4];
 #pragma unroll
-    for (int nt = 0; nt < 2; ++nt) {
-      c[nt] = {0.f, 0.f, 0.f, 0.f};
-      const int kr = nt * 16 + l15;
+    for (int nt = 0; nt < NKT; ++nt) {
+      f32x4_t c = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
       for (int ks = 0; ks < KS; ++ks) {
-        const bf16x8_t bf = *reinterpret_cast<const bf16x8_t*>(
+        const bf16x8_t kf = *reinterpret_cast<const bf16x8_t*>(
             reinterpret_cast<const char*>(Ks) +
-            gtile_off<KS>(kr, (ks * 32 + lhi * 8) * 2));
-        c[nt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qfrag[ks], bf, c[nt],
-                                                        0, 0, 0);
+            gtile_off<KS>(nt * 16 + l15, (ks * 32 + lhi * 8) * 2));
+        c = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qfrag[ks], c, 0, 0, 0);
       }
+#pragma unroll
+      for (int r = 0; r < 4; ++r) p[nt][r] = c[r] * rscale;
     }
-    // ---- mask, bias, online softmax (C layout: row lhi*4+r, col l15) ----
-    float p[2][4], alpha[4];
+    // ---- bias, cap, mask ----------------------------------------------------
+    // (wave-uniform) every key of the tile is live for every row
+    const bool full = t0 + GKV - 1 <= min(wp0, jmax) && t0 >= wlo;
+    if (rel || cap > 0.f || hbias) {
 #pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      float s[2];
+      for (int nt = 0; nt < NKT; ++nt)
 #pragma unroll
-      for (int nt = 0; nt < 2; ++nt) {
-        const int j = t0 + nt * 16 + l15;
-        const int dist = rpos[r] - j;
-        const bool live = rok[r] && j <= jmax && dist >= 0 &&
-                          (j >= rlo[r] || j < keep);
-        float sv = c[nt][r] * rscale[r];
-        if (rel && live) sv += rel_s[dist_bucket[dist]];
-        if (cap > 0.f) sv = cap * tanhf_fast(sv * inv_cap);
-        sv += hb;
-        s[nt] = live ? sv : -1e30f;
+        for (int r = 0; r < 4; ++r) {
+          float sv = p[nt][r];
+          if (rel) {
+            const int dist = rpos - (t0 + nt * 16 + lhi * 4 + r);
+            if (dist >= 0 && dist < window) sv += rel_s[dist_bucket[dist]];
+          }
+          if (cap > 0.f) sv = cap * tanhf_fast(sv * inv_cap);
+          p[nt][r] = sv + hb;
+        }
+    }
+    if (!full) {
+#pragma unroll
+      for (int nt = 0; nt < NKT; ++nt)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int j = t0 + nt * 16 + lhi * 4 + r;
+          const bool live = j <= jmax && j <= rpos && (j >= rlo || j < keep);
+          if (!live) p[nt][r] = -1e30f;
+        }
+    }
+    // ---- weights --------------------------------------------------------------
+    if (sigm) {
+#pragma unroll
+      for (int nt = 0; nt < NKT; ++nt)
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          p[nt][r] = p[nt][r] > -1e29f ? sigmoidf_acc(p[nt][r]) : 0.f;
+    } else {
+      float mx = p[0][0];
+#pragma unroll
+      for (int nt = 0; nt < NKT; ++nt)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) mx = fmaxf(mx, p[nt][r]);
+      mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+      mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+      const float mn = fmaxf(m_run, mx);
+      if (__any(mn > m_run)) {           // some row's maximum moved
+        const float alpha = __expf(m_run - mn);
+        l_run *= alpha;
+#pragma unroll
+        for (int nt = 0; nt < NVT; ++nt)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) o_acc[nt][r] *= alpha;
+        m_run = mn;
       }
-      if (sigm) {
-        alpha[r] = 1.f;
-#pragma unroll
-        for (int nt = 0; nt < 2; ++nt)
-          p[nt][r] = s[nt] > -1e29f ? sigmoidf_acc(s[nt]) : 0.f;
-        continue;
-      }
-      float rm = fmaxf(s[0], s[1]);
-#pragma unroll
-      for (int off = 1; off < 16; off <<= 1)
-        rm = fmaxf(rm, __shfl_xor(rm, off, 64));
-      const float mn = fmaxf(m_run[r], rm);
-      alpha[r] = __expf(m_run[r] - mn);
-      m_run[r] = mn;
       float rs = 0.f;
 #pragma unroll
-      for (int nt = 0; nt < 2; ++nt) {
-        p[nt][r] = s[nt] > -1e29f ? __expf(s[nt] - mn) : 0.f;
-        rs += p[nt][r];
-      }
+      for (int nt = 0; nt < NKT; ++nt)
 #pragma unroll
-      for (int off = 1; off < 16; off <<= 1) rs += __shfl_xor(rs, off, 64);
-      l_run[r] = l_run[r] * alpha[r] + rs;
-    }
-    if (!sigm) {
-#pragma unroll
-      for (int nt = 0; nt < NVT; ++nt)
-#pragma unroll
-        for (int r = 0; r < 4; ++r) o_acc[nt][r] *= alpha[r];
+        for (int r = 0; r < 4; ++r) {
+          // (a row without a live key so far has m_run = -1e30)
+          const float e = __expf(p[nt][r] - m_run);
+          p[nt][r] = full || p[nt][r] > -1e29f ? e : 0.f;
+          rs += p[nt][r];
+        }
+      l_run += rs;
     }
 
-    // ---- P: C layout -> A layout through a wave-private LDS tile --------
-    bf16_t* ps = Ps[wid];
+    // ---- O^T += V^T P^T, keys in the accumulators' order ---------------------
 #pragma unroll
-    for (int nt = 0; nt < 2; ++nt)
+    for (int kb = 0; kb < NKT / 2; ++kb) {
+      bf16x8_t pb;
 #pragma unroll
-      for (int r = 0; r < 4; ++r)
-        ps[(lhi * 4 + r) * GKV + nt * 16 + l15] = f2bf(p[nt][r]);
-    const bf16x8_t pa =
-        *reinterpret_cast<const bf16x8_t*>(ps + l15 * GKV + lhi * 8);
-
-    // ---- O += P V --------------------------------------------------------
+      for (int j = 0; j < 4; ++j) {
+        pb[j] = (__bf16)p[2 * kb][j];
+        pb[4 + j] = (__bf16)p[2 * kb + 1][j];
+      }
 #pragma unroll
-    for (int nt = 0; nt < NVT; ++nt) {
-      if (nt * 16 < Dv) {
-        bf16x8_t bv;
-        const int d2 = (nt * 16 + l15) * 2;
-#pragma unroll
-        for (int j = 0; j < 8; ++j)
-          bv[j] = *reinterpret_cast<const __bf16*>(
-              reinterpret_cast<const char*>(Vs) +
-              gtile_off<KV>(lhi * 8 + j, d2));
-        o_acc[nt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pa, bv, o_acc[nt],
-                                                            0, 0, 0);
+      for (int nt = 0; nt < NVT; ++nt) {
+        if (nt * 16 < Dv) {
+          const bf16_t* vr = Vt + (nt * 16 + l15) * VROW + kb * 32 + lhi * 4;
+          const uint2 a = *reinterpret_cast<const uint2*>(vr);
+          const uint2 c = *reinterpret_cast<const uint2*>(vr + 16);
+          const i32x4_t av = {(int)a.x, (int)a.y, (int)c.x, (int)c.y};
+          o_acc[nt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+              __builtin_bit_cast(bf16x8_t, av), pb, o_acc[nt], 0, 0, 0);
+        }
       }
     }
+    if (look) slot_s[ti & 1][threadIdx.x] = next_slot;
     __syncthreads();   // every wave is done with the tiles before restaging
   }
 
+  l_run += __shfl_xor(l_run, 16, 64);
+  l_run += __shfl_xor(l_run, 32, 64);
+  if (!rok) return;
+  const long tok = n0 + ri;
+  float inv = (sigm ? 1.f : 1.f / l_run) * out_scale;
+  if (gate && !out32) inv *= sigmoidf_acc(bf2f(gate[tok * ldg + h]));
+  bf16_t* op = out + tok * ldo + h * Dv;
+  float* op32 = out32 ? out32 + (tok * H + h) * Dv : nullptr;
+  const bool by8 = ((uintptr_t)op & 7) == 0;
 #pragma unroll
-  for (int r = 0; r < 4; ++r) {
-    const int i = wid * 16 + lhi * 4 + r;
-    if (!rok[r]) continue;
-    const long tok = n0 + i;
-    float inv = (sigm ? 1.f : 1.f / l_run[r]) * out_scale;
-    if (gate && !out32) inv *= sigmoidf_acc(bf2f(gate[tok * ldg + h]));
-    bf16_t* op = out + tok * ldo + h * Dv;
-    float* op32 = out32 ? out32 + (tok * H + h) * Dv : nullptr;
+  for (int nt = 0; nt < NVT; ++nt) {
+    const int d = nt * 16 + lhi * 4;     // four entries; Dv is a multiple of 8
+    if (d < Dv) {
+      f32x4v o;
 #pragma unroll
-    for (int nt = 0; nt < NVT; ++nt) {
-      const int d = nt * 16 + l15;
-      if (d < Dv) {
-        if (op32) op32[d] = o_acc[nt][r] * inv;
-        else op[d] = f2bf(o_acc[nt][r] * inv);
-      }
+      for (int r = 0; r < 4; ++r) o.v[r] = o_acc[nt][r] * inv;
+      if (op32) store4(op32 + d, o, 4, true);
+      else store4(op + d, o, 4, by8);
     }
   }
 }
@@ -362,8 +395,9 @@ void seq_rotate_back_heads(torch::Tensor out, torch::Tensor x,
                            torch::Tensor gate, int64_t H);
 
 #define GQA_MFMA_LAUNCH(KSV, KVV)                                             \
-  hipLaunchKernelGGL((gqa_attn_mfma_kernel<KSV, KVV>), grid, dim3(256), 0,    \
-      stream,                                                                 \
+  hipLaunchKernelGGL(                                                         \
+      (gqa_attn_mfma_kernel<KSV, KVV, (KVV > 4 ? 32 : 64)>), grid, dim3(256), \
+      0, stream,                                                              \
       (bf16_t*)out.data_ptr(), (const bf16_t*)q.data_ptr(),                   \
       (const bf16_t*)cache.data_ptr(), page_table.data_ptr<int>(),            \
       (int)page_table.size(1), seq_of_tok.data_ptr<int>(),                    \

@@ -3,12 +3,14 @@
 // Routing is a table over token ids, so a block finds its expert's rows by
 // scanning the batch's (token, choice) slots itself: no host routing, no
 // sort, no gather copy, and the launch shape depends only on the batch size
-// (capturable in a graph).  Grid = (64-column tile, expert); a block whose
+// (capturable in a graph).  Grid = (16-column tile, expert); a block whose
 // expert got no row exits at once.  The op is weight-read bound at these
-// batch sizes (every live expert streams its matrices once per step), so a
-// wave just streams 16 weight rows with 16-byte loads straight into
-// v_mfma_f32_16x16x32_bf16 B fragments while the A fragments (<= 16 token
-// rows per pass) come from the activations; fp32 accumulation.
+// batch sizes (every live expert streams its matrices once per step), so the
+// four waves of a block take a quarter of the columns' K each and stream
+// their 16 weight rows with 16-byte loads, several k-steps in flight,
+// straight into v_mfma_f32_16x16x32_bf16 B fragments while the A fragments
+// come from the activations; the partial sums (fp32) meet in LDS.  Up to 64
+// token rows go along with one pass over the weights.
 //
 //   ACT 1 : act[slot, j] = silu(x_t . Wg[e][j]) * (x_t . Wu[e][j])   (gated)
 //   ACT 2 : act[slot, j] = gelu_erf(x_t . Wu[e][j])                  (plain)
@@ -32,6 +34,97 @@ typedef __attribute__((ext_vector_type(4))) int i32x4_t;
 
 constexpr int MOE_MAX_SLOTS = 1024;
 
+constexpr int MOE_COLS = 16;          // output columns of a block
+
+// RT row tiles of 16 (slots c0 .. c0 + 16*RT of this expert) against the
+// block's columns; U k-steps in flight per wave
+template <int ACT, int RT, int U>
+DEV_INLINE void moe_tile(bf16_t* __restrict__ out, const bf16_t* __restrict__ x,
+                         long ldx, const bf16_t* __restrict__ wrow,
+                         const bf16_t* __restrict__ wrow2, const int* slots,
+                         int cnt, int c0, int top, int K, int Nout, int n0,
+                         float limit, float slope, float shift, float* red) {
+  constexpr bool GATED = ACT == 1 || ACT == 3;
+  constexpr bool BYTOKEN = ACT != 0;  // x rows by token, else by slot
+  constexpr int NA = GATED ? 2 : 1;
+  const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
+  const int l15 = lane & 15, lhi = lane >> 4;
+  // this wave's k-steps: an even number, so that it reads whole 128-byte lines
+  const int steps = K / 32, per = (steps + 7) / 8 * 2;
+  const int s0 = wid * per, s1 = min(s0 + per, steps);
+  const bf16_t* xrow[RT];
+#pragma unroll
+  for (int t = 0; t < RT; ++t) {      // rows past cnt: any row, dropped below
+    const int slot = slots[min(c0 + t * 16 + l15, cnt - 1)];
+    xrow[t] = x + (long)(BYTOKEN ? slot / top : slot) * ldx + lhi * 8;
+  }
+  f32x4_t acc[NA][RT];
+#pragma unroll
+  for (int a = 0; a < NA; ++a)
+#pragma unroll
+    for (int t = 0; t < RT; ++t) acc[a][t] = {0.f, 0.f, 0.f, 0.f};
+  const i32x4_t zi = {0, 0, 0, 0};
+#pragma unroll 1
+  for (int s = s0; s < s1; s += U) {
+    i32x4_t b[U], b2[U], a[RT][U];
+#pragma unroll
+    for (int u = 0; u < U; ++u) {     // past the end: the last step again
+      const long o = (long)min(s + u, s1 - 1) * 32;
+      b[u] = *reinterpret_cast<const i32x4_t*>(wrow + o);
+      if (GATED) b2[u] = *reinterpret_cast<const i32x4_t*>(wrow2 + o);
+#pragma unroll
+      for (int t = 0; t < RT; ++t)
+        a[t][u] = *reinterpret_cast<const i32x4_t*>(xrow[t] + o);
+    }
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const bool on = s + u < s1;     // wave-uniform
+#pragma unroll
+      for (int t = 0; t < RT; ++t) {
+        const bf16x8_t av = __builtin_bit_cast(bf16x8_t, on ? a[t][u] : zi);
+        acc[0][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+            av, __builtin_bit_cast(bf16x8_t, b[u]), acc[0][t], 0, 0, 0);
+        if (GATED)
+          acc[NA - 1][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+              av, __builtin_bit_cast(bf16x8_t, b2[u]), acc[NA - 1][t], 0, 0, 0);
+      }
+    }
+  }
+  // C layout: row = lhi*4 + r, col = l15
+#pragma unroll
+  for (int a = 0; a < NA; ++a)
+#pragma unroll
+    for (int t = 0; t < RT; ++t)
+#pragma unroll
+      for (int r = 0; r < 4; ++r)
+        red[((wid * NA + a) * RT + t) * 256 + (lhi * 4 + r) * 16 + l15] =
+            acc[a][t][r];
+  __syncthreads();
+  const int n = n0 + threadIdx.x % 16;
+#pragma unroll
+  for (int t = 0; t < RT; ++t) {
+    const int ri = c0 + t * 16 + threadIdx.x / 16;
+    float v[NA];
+#pragma unroll
+    for (int a = 0; a < NA; ++a) {
+      v[a] = 0.f;
+#pragma unroll
+      for (int w = 0; w < 4; ++w)
+        v[a] += red[((w * NA + a) * RT + t) * 256 + threadIdx.x];
+    }
+    float y = v[0];
+    if (ACT == 1) y = siluf_acc(v[0]) * v[NA - 1];
+    if (ACT == 2) y = gelu_erff_acc(v[0]);
+    if (ACT == 3) {
+      const float g = fminf(v[0], limit);
+      const float u = fminf(fmaxf(v[NA - 1], -limit), limit);
+      y = g * sigmoidf_acc(slope * g) * (u + shift);
+    }
+    if (ri < cnt && n < Nout) out[(long)slots[ri] * Nout + n] = f2bf(y);
+  }
+  __syncthreads();                    // red may be written again
+}
+
 template <int ACT>
 __global__ __launch_bounds__(256) void moe_table_gemm_kernel(
     bf16_t* __restrict__ out,           // (B*top, Nout)
@@ -42,13 +135,10 @@ __global__ __launch_bounds__(256) void moe_table_gemm_kernel(
     const bf16_t* __restrict__ w,       // (E, Nw, K): Nw = 2*Nout if gated
     int B, int top, int K, int Nout, float limit, float slope, float shift) {
   constexpr bool GATED = ACT == 1 || ACT == 3;
-  constexpr bool BYTOKEN = ACT != 0;    // x rows by token, else by slot
   __shared__ int slots[MOE_MAX_SLOTS];
   __shared__ int count;
+  __shared__ float red[4 * (GATED ? 2 : 1) * 4 * 256];
   const int e = blockIdx.y;
-  const int lane = threadIdx.x & 63;
-  const int wid = threadIdx.x >> 6;
-  const int l15 = lane & 15, lhi = lane >> 4;
   if (threadIdx.x == 0) count = 0;
   __syncthreads();
   const int S = B * top;
@@ -61,46 +151,19 @@ __global__ __launch_bounds__(256) void moe_table_gemm_kernel(
   const int cnt = count;
   if (cnt == 0) return;
 
-  const int n = blockIdx.x * 64 + wid * 16 + l15;   // this lane's B column
-  const bool nok = n < Nout;
+  const int lane = threadIdx.x & 63;
+  const int n0 = blockIdx.x * MOE_COLS;
+  const int n = min(n0 + (lane & 15), Nout - 1);      // this lane's B column
   const long Nw = GATED ? 2L * Nout : Nout;
-  const bf16_t* wrow = w + ((long)e * Nw + (nok ? n : 0)) * K + lhi * 8;
-  const bf16_t* wrow2 = wrow + (long)Nout * K;       // up rows (gated)
-
-  for (int c0 = 0; c0 < cnt; c0 += 16) {
-    const int si = c0 + l15;
-    const int slot = si < cnt ? slots[si] : -1;
-    const bf16_t* xrow = x + (long)(slot < 0 ? 0 : (BYTOKEN ? slot / top : slot)) * ldx + lhi * 8;
-    f32x4_t acc = {0.f, 0.f, 0.f, 0.f}, acc2 = {0.f, 0.f, 0.f, 0.f};
-    const i32x4_t zi = {0, 0, 0, 0};
-    const bf16x8_t zero = __builtin_bit_cast(bf16x8_t, zi);
-#pragma unroll 4
-    for (int k0 = 0; k0 < K; k0 += 32) {
-      const bf16x8_t a = slot >= 0 ? *reinterpret_cast<const bf16x8_t*>(xrow + k0) : zero;
-      const bf16x8_t b = nok ? *reinterpret_cast<const bf16x8_t*>(wrow + k0) : zero;
-      acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, acc, 0, 0, 0);
-      if (GATED) {
-        const bf16x8_t b2 = nok ? *reinterpret_cast<const bf16x8_t*>(wrow2 + k0) : zero;
-        acc2 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b2, acc2, 0, 0, 0);
-      }
-    }
-    // C layout: row = lhi*4 + r (slot of the pass), col = l15
-#pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int ri = c0 + lhi * 4 + r;
-      if (ri < cnt && nok) {
-        float v = acc[r];
-        if (ACT == 1) v = siluf_acc(acc[r]) * acc2[r];
-        if (ACT == 2) v = gelu_erff_acc(acc[r]);
-        if (ACT == 3) {
-          const float g = fminf(acc[r], limit);
-          const float u = fminf(fmaxf(acc2[r], -limit), limit);
-          v = g * sigmoidf_acc(slope * g) * (u + shift);
-        }
-        out[(long)slots[ri] * Nout + n] = f2bf(v);
-      }
-    }
-  }
+  const bf16_t* wrow = w + ((long)e * Nw + n) * K + (lane >> 4) * 8;
+  const bf16_t* wrow2 = wrow + (long)Nout * K;        // up rows (gated)
+#define MOE_TILE(RTV, UV, C0)                                                 \
+  moe_tile<ACT, RTV, UV>(out, x, ldx, wrow, wrow2, slots, cnt, C0, top, K,    \
+                         Nout, n0, limit, slope, shift, red)
+  if (cnt <= 16) MOE_TILE(1, 8, 0);
+  else if (cnt <= 32) MOE_TILE(2, 4, 0);
+  else
+    for (int c0 = 0; c0 < cnt; c0 += 64) MOE_TILE(4, 4, c0);
 }
 
 // y (B*top, width) = table-routed experts on h (B, width); fills ``act``
@@ -131,14 +194,14 @@ void seq_moe_table_ffn(torch::Tensor y, torch::Tensor act, torch::Tensor h,
               y.size(0) == (long)B * top && y.size(1) == W);
   if (B == 0) return;
   auto stream = at::hip::getCurrentHIPStream();
-  hipLaunchKernelGGL((moe_table_gemm_kernel<1>), dim3((ff + 63) / 64, E),
+  hipLaunchKernelGGL((moe_table_gemm_kernel<1>), dim3((ff + MOE_COLS - 1) / MOE_COLS, E),
                      dim3(256), 0, stream, (bf16_t*)act.data_ptr(),
                      (const bf16_t*)h.data_ptr(), h.stride(0),
                      (const long*)tokens.data_ptr<int64_t>(),
                      table.data_ptr<int>(), (const int*)nullptr,
                      (const bf16_t*)w_gu.data_ptr(), B, top, W, ff, 0.f,
                      0.f, 0.f);
-  hipLaunchKernelGGL((moe_table_gemm_kernel<0>), dim3((W + 63) / 64, E),
+  hipLaunchKernelGGL((moe_table_gemm_kernel<0>), dim3((W + MOE_COLS - 1) / MOE_COLS, E),
                      dim3(256), 0, stream, (bf16_t*)y.data_ptr(),
                      (const bf16_t*)act.data_ptr(), (long)ff,
                      (const long*)tokens.data_ptr<int64_t>(),
@@ -182,8 +245,8 @@ void seq_moe_routed_ffn(torch::Tensor y, torch::Tensor act, torch::Tensor h,
   auto stream = at::hip::getCurrentHIPStream();
   const float lim = (float)limit, sl = (float)slope, sh = (float)shift;
 #define MOE_UP(ACTV)                                                          \
-  hipLaunchKernelGGL((moe_table_gemm_kernel<ACTV>), dim3((ff + 63) / 64, E),  \
-                     dim3(256), 0, stream, (bf16_t*)act.data_ptr(),           \
+  hipLaunchKernelGGL((moe_table_gemm_kernel<ACTV>),                           \
+                     dim3((ff + MOE_COLS - 1) / MOE_COLS, E), dim3(256), 0, stream, (bf16_t*)act.data_ptr(),           \
                      (const bf16_t*)h.data_ptr(), h.stride(0),                \
                      (const long*)nullptr, (const int*)nullptr,               \
                      idx.data_ptr<int>(), (const bf16_t*)w_up.data_ptr(), B,  \
@@ -191,7 +254,7 @@ void seq_moe_routed_ffn(torch::Tensor y, torch::Tensor act, torch::Tensor h,
   if (!gated) MOE_UP(2);
   else if (lim > 0.f) MOE_UP(3);
   else MOE_UP(1);
-  hipLaunchKernelGGL((moe_table_gemm_kernel<0>), dim3((W + 63) / 64, E),
+  hipLaunchKernelGGL((moe_table_gemm_kernel<0>), dim3((W + MOE_COLS - 1) / MOE_COLS, E),
                      dim3(256), 0, stream, (bf16_t*)y.data_ptr(),
                      (const bf16_t*)act.data_ptr(), (long)ff,
                      (const long*)nullptr, (const int*)nullptr,
@@ -223,21 +286,20 @@ DEV_INLINE void wave_argmax(float& v, int& i) {
   }
 }
 
-__global__ __launch_bounds__(256) void moe_route_kernel(
-    int* __restrict__ idx, float* __restrict__ wout,
-    const float* __restrict__ logits, long ldl,
-    const float* __restrict__ correction, long N, int E, int top, int groups,
-    int keep, int act, int gtop) {
-  __shared__ float s_sh[4][ROUTE_MAX_E], c_sh[4][ROUTE_MAX_E];
-  __shared__ float g_sh[4][ROUTE_MAX_E];
-  const int wid = threadIdx.x >> 6, lane = threadIdx.x & 63;
-  const long n0 = (long)blockIdx.x * 4 + wid;
-  const bool live = n0 < N;           // idle waves shadow the last token
-  const long n = live ? n0 : N - 1;
-  float* s = s_sh[wid];
-  float* c = c_sh[wid];
-  float* gb = g_sh[wid];
-  const float* z = logits + n * ldl;
+// order of a wave's own LDS accesses (scratch that no other wave touches)
+DEV_INLINE void wave_sync() {
+  __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+  __builtin_amdgcn_wave_barrier();
+}
+
+// the choice for one token by one wave, on LDS scratch of its own; z: the
+// token's E logits
+DEV_INLINE void route_token(const float* z, float* s, float* c, float* gb,
+                            int* __restrict__ idx, float* __restrict__ wout,
+                            long n, bool live,
+                            const float* __restrict__ correction, int E,
+                            int top, int groups, int keep, int act, int gtop) {
+  const int lane = threadIdx.x & 63;
   if (act >= 1) {
     for (int e = lane; e < E; e += 64) {
       const float p = act == 1 ? sigmoidf_acc(z[e]) : z[e];
@@ -262,7 +324,7 @@ __global__ __launch_bounds__(256) void moe_route_kernel(
       c[e] = p + correction[e];
     }
   }
-  __syncthreads();
+  wave_sync();
   if (groups > 1) {
     const int per = E / groups;
     for (int g = lane; g < groups; g += 64) {
@@ -288,7 +350,7 @@ __global__ __launch_bounds__(256) void moe_route_kernel(
       }
       gb[g] = b;
     }
-    __syncthreads();
+    wave_sync();
     // mark the best ``keep`` groups: their best becomes +inf
     for (int r = 0; r < keep; ++r) {
       float bv = -INFINITY;
@@ -302,11 +364,11 @@ __global__ __launch_bounds__(256) void moe_route_kernel(
       }
       wave_argmax(bv, bi);
       if (lane == 0 && bi != 0x7fffffff) gb[bi] = INFINITY;
-      __syncthreads();
+      wave_sync();
     }
     for (int e = lane; e < E; e += 64)
       if (gb[e / per] != INFINITY) c[e] = -INFINITY;
-    __syncthreads();
+    wave_sync();
   }
   float best = 0.f;                   // the first pick is the largest
   for (int r = 0; r < top; ++r) {
@@ -329,8 +391,59 @@ __global__ __launch_bounds__(256) void moe_route_kernel(
       }
       c[bi] = -INFINITY;
     }
-    __syncthreads();
+    wave_sync();
   }
+}
+
+__global__ __launch_bounds__(256) void moe_route_kernel(
+    int* __restrict__ idx, float* __restrict__ wout,
+    const float* __restrict__ logits, long ldl,
+    const float* __restrict__ correction, long N, int E, int top, int groups,
+    int keep, int act, int gtop) {
+  __shared__ float s_sh[4][ROUTE_MAX_E], c_sh[4][ROUTE_MAX_E];
+  __shared__ float g_sh[4][ROUTE_MAX_E];
+  const int wid = threadIdx.x >> 6;
+  const long n0 = (long)blockIdx.x * 4 + wid;
+  const bool live = n0 < N;           // idle waves shadow the last token
+  const long n = live ? n0 : N - 1;
+  route_token(logits + n * ldl, s_sh[wid], c_sh[wid], g_sh[wid], idx, wout, n,
+              live, correction, E, top, groups, keep, act, gtop);
+}
+
+// Router product and choice in one launch, for batches of few tokens: one
+// block of sixteen waves per token, a wave per router row in turn (rows from
+// the XCD's L2, fp32 products and sums); the first wave makes the choice.
+// Rows past the E choices (R > E) are further numbers per token: they go to
+// ``extra``.
+template <typename T, bool VEC>
+__global__ __launch_bounds__(1024) void moe_router_kernel(
+    int* __restrict__ idx, float* __restrict__ wout, float* __restrict__ extra,
+    const T* __restrict__ h, long ldh, const float* __restrict__ w,
+    const float* __restrict__ correction, int W, int R, int E, int top,
+    int groups, int keep, int act, int gtop) {
+  constexpr int C = VEC ? 4 : 1;        // columns of a lane
+  __shared__ float z[ROUTE_MAX_E + 8], s_sh[ROUTE_MAX_E], c_sh[ROUTE_MAX_E];
+  __shared__ float g_sh[ROUTE_MAX_E];
+  const long n = blockIdx.x;
+  const int wid = threadIdx.x >> 6, lane = threadIdx.x & 63;
+  const T* hr = h + n * ldh;
+  for (int r = wid; r < R; r += 16) {
+    const float* wr = w + (long)r * W;
+    float a = 0.f;
+#pragma unroll 8
+    for (int i = lane * C; i < W; i += 64 * C) {
+      const f32x4v x = load4(hr + i, C, VEC), u = load4(wr + i, C, VEC);
+#pragma unroll
+      for (int c = 0; c < C; ++c) a += x.v[c] * u.v[c];
+    }
+    a = wave_reduce_sum(a);
+    if (lane == 0) z[r] = a;
+  }
+  __syncthreads();
+  if (wid) return;
+  if (lane < R - E) extra[n * (R - E) + lane] = z[E + lane];
+  route_token(z, s_sh, c_sh, g_sh, idx, wout, n, true, correction, E, top,
+              groups, keep, act, gtop);
 }
 
 void seq_moe_route(torch::Tensor idx, torch::Tensor w, torch::Tensor logits,
@@ -359,34 +472,77 @@ void seq_moe_route(torch::Tensor idx, torch::Tensor w, torch::Tensor logits,
   HIP_CHECK_KERNEL();
 }
 
+void seq_moe_router(torch::Tensor idx, torch::Tensor w, torch::Tensor extra,
+                    torch::Tensor h, torch::Tensor router,
+                    torch::Tensor correction, int64_t groups, int64_t keep,
+                    int64_t act, int64_t group_top) {
+  CHECK_I32(idx);
+  CHECK_F32(w); CHECK_F32(router); CHECK_F32(correction); CHECK_F32(extra);
+  CHECK_ROWS(h);
+  const long N = h.size(0), W = h.size(1);
+  TORCH_CHECK(router.dim() == 2 && router.size(1) == W);
+  const int R = router.size(0), E = correction.numel();
+  TORCH_CHECK(idx.dim() == 2 && idx.size(0) == N && w.sizes() == idx.sizes());
+  const int top = idx.size(1);
+  TORCH_CHECK(E >= 1 && E <= ROUTE_MAX_E && R >= E && R - E <= 8,
+              "router outputs above 512");
+  TORCH_CHECK(extra.numel() == N * (R - E) && top >= 1 && top <= E);
+  TORCH_CHECK(groups >= 1 && E % groups == 0 && keep >= 1 && keep <= groups);
+  TORCH_CHECK(act >= 0 && act <= 2 && group_top >= 1);
+  if (N == 0) return;
+  auto stream = at::hip::getCurrentHIPStream();
+  SEQ_DISPATCH_T(h.scalar_type(), {
+    const bool vec = W % 4 == 0 && rows_by4<T>(h, W) &&
+                     (uintptr_t)router.data_ptr() % 16 == 0;
+#define ROUTER_LAUNCH(VECV)                                                   \
+    hipLaunchKernelGGL((moe_router_kernel<T, VECV>), dim3(N), dim3(1024), 0,  \
+        stream, idx.data_ptr<int>(), w.data_ptr<float>(),                     \
+        extra.data_ptr<float>(), (const T*)h.data_ptr(), h.stride(0),         \
+        router.data_ptr<float>(), correction.data_ptr<float>(), (int)W, R, E, \
+        top, (int)groups, (int)keep, (int)act, (int)group_top)
+    if (vec) ROUTER_LAUNCH(true);
+    else ROUTER_LAUNCH(false); });
+  HIP_CHECK_KERNEL();
+}
+
 // out[n, d] = sum_k w'[n,k] * (idx[n,k] < E ? ys[n*top+k, d] : h[n, d])
 //             (+ shared[n, d] [* sigmoid(sgate[n])]),  w' = scale * w / (sum_k w + weight_eps)
+// (a slot's expert row is ys[slot], or ys[place[slot]] where the rows lie in
+// another order).  Four consecutive numbers per thread and step.
 template <typename T>
-__global__ void moe_weighted_combine_kernel(
+__global__ __launch_bounds__(256) void moe_weighted_combine_kernel(
     T* __restrict__ out, const T* __restrict__ ys, const int* __restrict__ idx,
     const float* __restrict__ w, const T* __restrict__ h, long ldh,
     const T* __restrict__ shared, long lds_, int top, int E, float weight_eps,
-    long rows, int D, float scale, const float* __restrict__ sgate,
-    long ldsg) {
-  long i = (long)blockIdx.x * blockDim.x + threadIdx.x;
+    long rows, int D, float scale, const float* __restrict__ sgate, long ldsg,
+    const int* __restrict__ place, bool vec) {
+  const int dq = (D + 3) / 4;
+  const long total = rows * dq;
   const long stride = (long)gridDim.x * blockDim.x;
-  for (; i < rows * D; i += stride) {
-    const long n = i / D;
-    const int d = i % D;
+  for (long i = (long)blockIdx.x * blockDim.x + threadIdx.x; i < total;
+       i += stride) {
+    const long n = i / dq;
+    const int d = (int)(i - n * dq) * 4;
     float wsum = 0.f;
     for (int k = 0; k < top; ++k) wsum += w[n * top + k];
     const float inv = scale / (wsum + weight_eps);
-    float acc = 0.f;
+    f32x4v acc = {{0.f, 0.f, 0.f, 0.f}};
     for (int k = 0; k < top; ++k) {
-      const float v = idx[n * top + k] < E ? ldf(ys + (n * top + k) * D + d)
-                                           : ldf(h + n * ldh + d);
-      acc += w[n * top + k] * inv * v;
+      const long slot = n * top + k;
+      const T* src = idx[slot] < E
+          ? ys + (place ? (long)place[slot] : slot) * D : h + n * ldh;
+      const f32x4v v = load4(src + d, D - d, vec);
+      const float wk = w[slot] * inv;
+#pragma unroll
+      for (int c = 0; c < 4; ++c) acc.v[c] += wk * v.v[c];
     }
     if (shared) {
-      const float sv = ldf(shared + n * lds_ + d);
-      acc += sgate ? sv * sigmoidf_acc(sgate[n * ldsg]) : sv;
+      const f32x4v v = load4(shared + n * lds_ + d, D - d, vec);
+      const float g = sgate ? sigmoidf_acc(sgate[n * ldsg]) : 1.f;
+#pragma unroll
+      for (int c = 0; c < 4; ++c) acc.v[c] += g * v.v[c];
     }
-    stf(out + i, acc);
+    store4(out + n * D + d, acc, D - d, vec);
   }
 }
 
@@ -394,7 +550,7 @@ void seq_moe_weighted_combine(torch::Tensor out, torch::Tensor ys,
                               torch::Tensor idx, torch::Tensor w,
                               torch::Tensor h, torch::Tensor shared,
                               int64_t E, double weight_eps, double scale,
-                              torch::Tensor shared_gate) {
+                              torch::Tensor shared_gate, torch::Tensor place) {
   CHECK_I32(idx);
   CHECK_F32(w);
   CHECK_ROWS(h);
@@ -420,15 +576,26 @@ void seq_moe_weighted_combine(torch::Tensor out, torch::Tensor ys,
                 shared_gate.size(0) == N && shared_gate.size(1) == 1 &&
                 shared_gate.scalar_type() == torch::kFloat32,
                 "shared gate: one fp32 number per token");
+  const bool has_place = place.defined() && place.numel() > 0;
+  if (has_place) {
+    CHECK_I32(place);
+    TORCH_CHECK(place.numel() == N * top, "one row per slot");
+  }
   if (N == 0) return;
-  const long nblk = std::min<long>((N * D + 255) / 256, MAX_RESIDENT_BLOCKS * 4);
+  const long nblk = std::min<long>((N * ((D + 3) / 4) + 255) / 256,
+                                   MAX_RESIDENT_BLOCKS * 4);
   auto stream = at::hip::getCurrentHIPStream();
-  SEQ_DISPATCH_T(ty, { hipLaunchKernelGGL((moe_weighted_combine_kernel<T>), dim3(nblk), dim3(256), 0, stream,
+  SEQ_DISPATCH_T(ty, {
+      const bool vec = D % 4 == 0 && rows_by4<T>(ys, D) && rows_by4<T>(h, D) &&
+                       rows_by4<T>(out, D) &&
+                       (!has_shared || rows_by4<T>(shared, D));
+      hipLaunchKernelGGL((moe_weighted_combine_kernel<T>), dim3(nblk), dim3(256), 0, stream,
       (T*)out.data_ptr(), (const T*)ys.data_ptr(), idx.data_ptr<int>(),
       w.data_ptr<float>(), (const T*)h.data_ptr(), h.stride(0),
       has_shared ? (const T*)shared.data_ptr() : nullptr,
       has_shared ? shared.stride(0) : 0, top, (int)E, (float)weight_eps, N,
       D, (float)scale, has_sg ? shared_gate.data_ptr<float>() : nullptr,
-      has_sg ? shared_gate.stride(0) : 0); });
+      has_sg ? shared_gate.stride(0) : 0,
+      has_place ? place.data_ptr<int>() : nullptr, vec); });
   HIP_CHECK_KERNEL();
 }

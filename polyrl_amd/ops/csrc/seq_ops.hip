@@ -561,6 +561,59 @@ __global__ __launch_bounds__(256) void group_rmsnorm_kernel(
   }
 }
 
+// Large groups in multiples of four numbers, up to 1024*EPT: the block keeps
+// the group in registers between the reduction and the stores.
+template <typename T, int EPT>
+__global__ __launch_bounds__(256) void group_rmsnorm_row_kernel(
+    T* __restrict__ out, const float* __restrict__ y,
+    const float* __restrict__ w, const T* __restrict__ gate, long ldg, int D,
+    int gs, float eps, bool w_shared, int gate_act) {
+  __shared__ float red[8];
+  const long row = blockIdx.x;
+  const int c0 = blockIdx.y * gs;
+  const float* yr = y + row * D + c0;
+  const float* wr = w_shared ? w : w + c0;
+  f32x4v x[EPT], gv[EPT];
+  float ss = 0.f;
+#pragma unroll
+  for (int e = 0; e < EPT; ++e) {
+    const int i = (threadIdx.x + e * 256) * 4;
+    x[e] = {{0.f, 0.f, 0.f, 0.f}};
+    if (i < gs) {
+      x[e] = load4(yr + i, 4, true);
+      if (gate) gv[e] = load4(gate + row * ldg + c0 + i, 4, true);
+    }
+  }
+#pragma unroll
+  for (int e = 0; e < EPT; ++e)
+#pragma unroll
+    for (int c = 0; c < 4; ++c) ss += x[e].v[c] * x[e].v[c];
+  const float inv = rsqrtf(block_reduce_sum<4>(ss, red) / gs + eps);
+#pragma unroll
+  for (int e = 0; e < EPT; ++e) {
+    const int i = (threadIdx.x + e * 256) * 4;
+    if (i < gs) {
+      const f32x4v wv = load4(wr + i, 4, true);
+      f32x4v o;
+#pragma unroll
+      for (int c = 0; c < 4; ++c) {
+        o.v[c] = x[e].v[c] * inv * wv.v[c];
+        if (gate)
+          o.v[c] *= gate_act == 2 ? siluf_acc(gv[e].v[c])
+                                  : sigmoidf_acc(gv[e].v[c]);
+      }
+      store4(out + row * D + c0 + i, o, 4, true);
+    }
+  }
+}
+
+#define GROUP_ROW_LAUNCH(EPTV)                                                \
+  hipLaunchKernelGGL((group_rmsnorm_row_kernel<T, EPTV>), grid, dim3(256), 0, \
+      stream, (T*)out.data_ptr(), y.data_ptr<float>(),                        \
+      weight.data_ptr<float>(), has_g ? (const T*)gate.data_ptr() : nullptr,  \
+      has_g ? gate.stride(0) : 0, D, (int)gs, (float)eps, w_shared,           \
+      (int)gate_act)
+
 void seq_group_rmsnorm(torch::Tensor out, torch::Tensor y,
                        torch::Tensor weight, int64_t groups, double eps,
                        torch::Tensor gate, int64_t gate_act) {
@@ -582,8 +635,17 @@ void seq_group_rmsnorm(torch::Tensor out, torch::Tensor y,
   auto stream = at::hip::getCurrentHIPStream();
   const bool big = D / groups >= 512;
   const dim3 grid(y.size(0), big ? groups : (groups + 3) / 4);
+  const long gs = D / groups;
   SEQ_DISPATCH_T(out.scalar_type(), {
-    if (big)
+    const bool rows4 = big && gs % 4 == 0 && gs <= 8192 &&
+                       rows_by4<float>(y, D) && rows_by4<T>(out, D) &&
+                       (uintptr_t)weight.data_ptr() % 16 == 0 &&
+                       (!has_g || rows_by4<T>(gate, D));
+    if (rows4 && gs <= 1024) GROUP_ROW_LAUNCH(1);
+    else if (rows4 && gs <= 2048) GROUP_ROW_LAUNCH(2);
+    else if (rows4 && gs <= 4096) GROUP_ROW_LAUNCH(4);
+    else if (rows4) GROUP_ROW_LAUNCH(8);
+    else if (big)
       hipLaunchKernelGGL((group_rmsnorm_kernel<T, true>), grid, dim3(256), 0,
           stream, (T*)out.data_ptr(), y.data_ptr<float>(),
           weight.data_ptr<float>(),
@@ -711,33 +773,40 @@ void seq_latent_kv_store(torch::Tensor dkv, int64_t rank, torch::Tensor norm_w,
 // mode 3: gelu(a), the exact (erf) form
 // mode 4: g * sigmoid(p1 * g) * (u + p2), g = min(a, p0), u = clamp(b, +-p0)
 // mode 5: max(a, 0) * b
+// Four consecutive columns per thread and step.
 template <typename T>
-__global__ void act_mul_kernel(T* __restrict__ out, const T* __restrict__ a,
-                               long lda, const T* __restrict__ b, long ldb,
-                               long rows, int cols, int mode, float p0,
-                               float p1, float p2) {
-  long i = (long)blockIdx.x * blockDim.x + threadIdx.x;
+__global__ __launch_bounds__(256) void act_mul_kernel(
+    T* __restrict__ out, const T* __restrict__ a, long lda,
+    const T* __restrict__ b, long ldb, long rows, int cols, int mode, float p0,
+    float p1, float p2, bool vec) {
+  const int cq = (cols + 3) / 4;
+  const long n = rows * cq;
   const long stride = (long)gridDim.x * blockDim.x;
-  const long n = rows * cols;
-  for (; i < n; i += stride) {
-    const long r = i / cols;
-    const int c = i % cols;
-    const float av = ldf(a + r * lda + c);
-    float v;
-    if (mode == 2) {
-      v = tanhf(av);
-    } else if (mode == 3) {
-      v = gelu_erff_acc(av);
-    } else if (mode == 4) {
-      const float g = fminf(av, p0);
-      const float u = fminf(fmaxf(ldf(b + r * ldb + c), -p0), p0);
-      v = g * sigmoidf_acc(p1 * g) * (u + p2);
-    } else {
-      const float bv = ldf(b + r * ldb + c);
-      v = (mode == 5   ? fmaxf(av, 0.f)
-           : mode == 0 ? siluf_acc(av) : sigmoidf_acc(av)) * bv;
+  for (long i = (long)blockIdx.x * blockDim.x + threadIdx.x; i < n;
+       i += stride) {
+    const long r = i / cq;
+    const int c0 = (int)(i - r * cq) * 4;
+    const f32x4v av = load4(a + r * lda + c0, cols - c0, vec);
+    f32x4v bv = av, v;
+    if (mode != 2 && mode != 3)
+      bv = load4(b + r * ldb + c0, cols - c0, vec);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const float x = av.v[e];
+      if (mode == 2) {
+        v.v[e] = tanhf(x);
+      } else if (mode == 3) {
+        v.v[e] = gelu_erff_acc(x);
+      } else if (mode == 4) {
+        const float g = fminf(x, p0);
+        const float u = fminf(fmaxf(bv.v[e], -p0), p0);
+        v.v[e] = g * sigmoidf_acc(p1 * g) * (u + p2);
+      } else {
+        v.v[e] = (mode == 5   ? fmaxf(x, 0.f)
+                  : mode == 0 ? siluf_acc(x) : sigmoidf_acc(x)) * bv.v[e];
+      }
     }
-    stf(out + i, v);
+    store4(out + r * cols + c0, v, cols - c0, vec);
   }
 }
 
@@ -752,12 +821,16 @@ void seq_act_mul(torch::Tensor out, torch::Tensor a, torch::Tensor b,
   const long rows = a.size(0);
   const int cols = a.size(1);
   if (rows * cols == 0) return;
-  const long nblk = std::min<long>((rows * cols + 255) / 256, MAX_RESIDENT_BLOCKS * 4);
+  const long nblk = std::min<long>((rows * ((cols + 3) / 4) + 255) / 256,
+                                   MAX_RESIDENT_BLOCKS * 4);
   auto stream = at::hip::getCurrentHIPStream();
-  SEQ_DISPATCH_T(a.scalar_type(), { hipLaunchKernelGGL((act_mul_kernel<T>), dim3(nblk), dim3(256), 0, stream, 
+  SEQ_DISPATCH_T(a.scalar_type(), {
+      const bool vec = rows_by4<T>(a, cols) && rows_by4<T>(b, cols) &&
+                       rows_by4<T>(out, cols);
+      hipLaunchKernelGGL((act_mul_kernel<T>), dim3(nblk), dim3(256), 0, stream,
       (T*)out.data_ptr(), (const T*)a.data_ptr(), a.stride(0),
       (const T*)b.data_ptr(), b.stride(0), rows, cols, (int)mode, (float)p0,
-      (float)p1, (float)p2); });
+      (float)p1, (float)p2, vec); });
   HIP_CHECK_KERNEL();
 }
 

@@ -613,6 +613,28 @@ def moe_route(logits, correction, top: int, groups: int, keep: int,
     return R.moe_route(logits, correction, top, groups, keep, act, group_top)
 
 
+def moe_router(h, router, correction, top: int, groups: int, keep: int,
+               act: str = "softmax", group_top: int = 1):
+    """Router product router (R, W) fp32 on h (N, W), and the choice of
+    :func:`moe_route` among its first E = len(correction) outputs.  Returns
+    (index, weights, the other R - E outputs (N, R - E) fp32).  Few tokens:
+    one launch; many: the vendor's fp32 product first."""
+    E, R_ = correction.numel(), router.shape[0]
+    if h.is_cuda and 0 < h.shape[0] <= 512:
+        N = h.shape[0]
+        idx = torch.empty(N, top, dtype=torch.int32, device=h.device)
+        w = torch.empty(N, top, dtype=torch.float32, device=h.device)
+        extra = torch.empty(N, R_ - E, dtype=torch.float32, device=h.device)
+        _ext().seq_moe_router(
+            idx, w, extra, h, router, correction, groups, keep,
+            {"softmax": 0, "sigmoid": 1, "logits": 2}[act], group_top)
+        return idx, w, extra
+    logits = h.float() @ router.t()
+    idx, w = moe_route(logits.narrow(1, 0, E), correction, top, groups, keep,
+                       act, group_top)
+    return idx, w, logits.narrow(1, E, R_ - E)
+
+
 def gelu_erf(x):
     """Exact (erf) GELU; x may be a column slice."""
     if x.is_cuda:
@@ -651,11 +673,11 @@ def moe_routed_ffn(h, idx, w_up, w_down, gated: bool = False,
 
 def moe_weighted_combine(ys, idx, w, h, shared, E: int, weight_eps: float,
                          out_dtype, scale: float = 1.0,
-                         shared_gate=None) -> torch.Tensor:
+                         shared_gate=None, place=None) -> torch.Tensor:
     """y[n] = sum_k w'[n,k] * (ys[n*top+k] if idx[n,k] < E else h[n])
     [+ shared[n], times sigmoid(shared_gate[n]) when a gate (N, 1) fp32 is
     given (a column slice is allowed)] with w' = scale * w / (sum_k w + weight_eps), fp32
-    sums."""
+    sums.  With ``place`` (N*top,) int32 slot i's row is ys[place[i]]."""
     if ys.is_cuda:
         out = torch.empty(h.shape, dtype=out_dtype, device=h.device)
         if h.shape[0]:
@@ -663,10 +685,11 @@ def moe_weighted_combine(ys, idx, w, h, shared, E: int, weight_eps: float,
                 out, ys, idx, w, h,
                 shared if shared is not None else torch.Tensor(), E,
                 weight_eps, scale,
-                shared_gate if shared_gate is not None else torch.Tensor())
+                shared_gate if shared_gate is not None else torch.Tensor(),
+                place if place is not None else torch.Tensor())
         return out
     return R.moe_weighted_combine(ys, idx, w, h, shared, E, weight_eps,
-                                  out_dtype, scale, shared_gate)
+                                  out_dtype, scale, shared_gate, place)
 
 
 def silu_mul_any(gate, up):

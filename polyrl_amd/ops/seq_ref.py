@@ -501,8 +501,10 @@ def moe_routed_ffn(h, idx, w_up, w_down, gated=False, clamp=None):
 
 
 def moe_weighted_combine(ys, idx, w, h, shared, E, weight_eps, out_dtype,
-                         scale=1.0, shared_gate=None):
+                         scale=1.0, shared_gate=None, place=None):
     N, top = idx.shape
+    if place is not None:
+        ys = ys[place.long()]
     wn = w.float() / (w.float().sum(-1, keepdim=True) + weight_eps) * scale
     rows = ys.float().view(N, top, -1)
     ident = (idx >= E).unsqueeze(-1)

@@ -996,7 +996,8 @@ class RoutedMoE(_Part):
         expert's rows of the sorted copy: the vendor library then sees a
         handful of shapes instead of a new one per call (a new shape costs
         more on the host than the product takes on the GPU).  The surplus
-        rows' results are dropped."""
+        rows' results are dropped.  Returns the rows sorted by expert and
+        each slot's place among them."""
         N, top = idx.shape
         S, W = N * top, h.shape[1]
         flat = idx.reshape(-1)
@@ -1013,9 +1014,10 @@ class RoutedMoE(_Part):
                 act = self._act(_mm(xs[o:o + cp], self.w_up[e]))
                 ys_sorted[o:o + c] = _mm(act, self.w_down[e])[:c]
                 o += c
-        ys = torch.empty_like(ys_sorted)
-        ys[order] = ys_sorted           # identity rows stay unread
-        return ys
+        # (identity slots come last: their rows stay unread)
+        place = torch.empty(S, dtype=torch.int32, device=h.device)
+        place[order] = torch.arange(S, dtype=torch.int32, device=h.device)
+        return ys_sorted, place
 
     def _act(self, a, limit=None):
         if self.gated:
@@ -1030,18 +1032,16 @@ class RoutedMoE(_Part):
 
     def forward(self, h, res, bt):
         f = self.spec
-        logits = _mm(h.float(), self.router)
-        gate = logits.narrow(1, self.R, 1) if f.shared_gate else None
-        if gate is not None:
-            logits = logits.narrow(1, 0, self.R)
-        idx, w = seq.moe_route(logits, self.correction, f.top, f.group_count,
-                               f.group_keep, f.router_act, f.group_top)
+        idx, w, gate = seq.moe_router(h, self.router, self.correction, f.top,
+                                      f.group_count, f.group_keep,
+                                      f.router_act, f.group_top)
+        place = None
         if h.shape[0] <= 256 and self.E and \
                 seq.moe_routed_ffn_supported(h, self.top, self.ff):
             ys = seq.moe_routed_ffn(h, idx, self.w_up, self.w_down,
                                     self.gated, self.clamp)
         elif self.E:
-            ys = self.experts_large(h, idx.long())
+            ys, place = self.experts_large(h, idx.long())
         else:
             ys = h.new_empty(h.shape[0] * f.top, h.shape[1])
         shared = None
@@ -1050,7 +1050,8 @@ class RoutedMoE(_Part):
                          self.s_down)
         return seq.moe_weighted_combine(ys, idx, w, h, shared, self.E,
                                         f.weight_eps, h.dtype, f.route_scale,
-                                        gate)
+                                        gate if f.shared_gate else None,
+                                        place)
 
 
 _MIXERS = {"general_delta": DeltaRuleMixer, "mamba2": SSMMixer,

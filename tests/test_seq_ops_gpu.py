@@ -1135,3 +1135,71 @@ def test_relu_glu(dt):
     torch.testing.assert_close(
         seq.relu_glu(d[:, :33], d[:, 37:]).cpu().float(),
         R.relu_glu(big[:, :33], big[:, 37:]).float(), **tol(dt))
+
+
+@pytest.mark.parametrize("dt", DTYPES)
+@pytest.mark.parametrize("N,W,E,extra,top,groups,keep,act,gtop", [
+    (1, 64, 4, 1, 1, 1, 1, "logits", 1), (37, 100, 16, 1, 3, 1, 1, "logits", 1),
+    (64, 2048, 16, 0, 2, 2, 1, "sigmoid", 2), (9, 37, 6, 3, 2, 3, 2, "softmax", 1),
+    (513, 40, 5, 1, 5, 1, 1, "logits", 1), (70, 260, 130, 1, 4, 1, 1, "softmax", 1),
+])
+def test_router_product_and_choice(dt, N, W, E, extra, top, groups, keep, act,
+                                   gtop):
+    big = rnd(N, W + 4, dt=dt)
+    rw, corr = rnd(E + extra, W), rnd(E) * 0.1
+    i0, w0, x0 = seq.moe_router(big[:, :W], rw, corr, top, groups, keep, act,
+                                gtop)
+    i1, w1, x1 = seq.moe_router(big.to(DEV)[:, :W], rw.to(DEV), corr.to(DEV),
+                                top, groups, keep, act, gtop)
+    assert torch.equal(i1.cpu(), i0)
+    torch.testing.assert_close(w1.cpu(), w0, rtol=2e-4, atol=1e-5)
+    torch.testing.assert_close(x1.cpu(), x0, rtol=1e-4, atol=1e-4)
+
+
+@pytest.mark.parametrize("dt", DTYPES)
+@pytest.mark.parametrize("D", [24, 37])
+def test_combine_gathers_rows_in_another_order(dt, D):
+    N, top, E = 21, 3, 5
+    ys, h = rnd(N * top, D, dt=dt), rnd(N, D, dt=dt)
+    idx = torch.randint(0, E + 1, (N, top), dtype=torch.int32)
+    w = torch.rand(N, top)
+    place = torch.randperm(N * top).int()
+    want = R.moe_weighted_combine(ys[place.long()], idx, w, h, None, E, 1e-20,
+                                  dt)
+    got = seq.moe_weighted_combine(ys.to(DEV), idx.to(DEV), w.to(DEV),
+                                   h.to(DEV), None, E, 1e-20, dt,
+                                   place=place.to(DEV))
+    torch.testing.assert_close(got.cpu().float(), want.float(), **tol(dt))
+
+
+@pytest.mark.parametrize("K,N", [(32, 64), (96, 32), (160, 96), (2048, 224)])
+@pytest.mark.parametrize("rows", [[1, 0, 16, 17], [33, 64, 65, 2],
+                                  [150, 5, 0, 32]])
+def test_expert_products_by_row_count(K, N, rows):
+    """Every row-tile form of the decode-sized expert kernel, with widths
+    whose k-steps do not divide among the waves."""
+    dt = torch.bfloat16
+    flat = torch.cat([torch.full((n,), e) for e, n in enumerate(rows)])
+    T = flat.numel()
+    idx = flat[torch.randperm(T)].view(T, 1).int()
+    h = rnd(T, K, dt=dt)
+    up, down = rnd(4, 2 * N, K, dt=dt, scale=K ** -0.5), \
+        rnd(4, K, N, dt=dt, scale=N ** -0.5)
+    want = R.moe_routed_ffn(h, idx, up, down, True, (1.5, 1.702, 1.0))
+    got = seq.moe_routed_ffn(h.to(DEV), idx.to(DEV), up.to(DEV),
+                             down.to(DEV), True, (1.5, 1.702, 1.0))
+    torch.testing.assert_close(got.cpu().float(), want.float(), **tol(dt))
+
+
+@pytest.mark.parametrize("dt", DTYPES)
+@pytest.mark.parametrize("groups,gs", [(1, 512), (2, 1500), (1, 2048),
+                                       (1, 3000), (3, 4100), (1, 8192),
+                                       (1, 9000), (1, 1026)])
+def test_group_rmsnorm_of_large_groups(dt, groups, gs):
+    y, w = rnd(5, groups * gs), rnd(groups * gs)
+    gate = rnd(5, groups * gs + 4, dt=dt)
+    for ww in (w, w[:gs].contiguous()):
+        want = R.group_rmsnorm(y, ww, groups, 1e-5, dt, gate[:, 4:])
+        got = seq.group_rmsnorm(y.to(DEV), ww.to(DEV), groups, 1e-5, dt,
+                                gate.to(DEV)[:, 4:])
+        torch.testing.assert_close(got.cpu().float(), want.float(), **tol(dt))
