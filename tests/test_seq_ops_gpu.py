@@ -972,7 +972,7 @@ def test_streams_join_open_and_tanh_norm(dt, S, D):
 
 @pytest.mark.parametrize("dt", DTYPES)
 @pytest.mark.parametrize("H,Dk,Dv,lens", [
-    (2, 32, 64, [5, 1, 20]), (3, 10, 14, [40, 2]), (1, 7, 5, [9, 1]),
+    (2, 28, 60, [5, 1, 20]), (3, 10, 14, [40, 2]), (1, 7, 5, [9, 1]),
     (2, 64, 68, [64, 65, 63, 1]), (2, 96, 128, [130, 1]),
     (1, 128, 192, [200, 3, 129]), (2, 20, 40, [128]), (1, 130, 8, [70]),
     (1, 300, 20, [33, 1]), (2, 512, 12, [6]), (4, 64, 64, [1, 1, 1, 1]),
@@ -1069,7 +1069,7 @@ def test_gqa_prepare_with_biases_and_pairs(dt, H, G, D, Dv, half, inter,
 
 @pytest.mark.parametrize("dt", DTYPES)
 @pytest.mark.parametrize("H,G,D,Dv,lens,starts", [
-    (4, 2, 96, 192, [70, 1, 130], [3, 300, 40]),
+    (6, 3, 88, 184, [70, 1, 130], [3, 300, 40]),
     (2, 1, 128, 256, [40, 1], [10, 65]), (3, 3, 40, 168, [66, 2], [0, 9]),
     (2, 2, 200, 48, [64, 5], [30, 0]), (1, 1, 256, 256, [65], [64]),
     (8, 8, 160, 144, [33, 1], [20, 90]), (4, 1, 8, 24, [1, 1, 1], [0, 31, 200]),
